@@ -1,5 +1,5 @@
 // Binding for the one-shot / two-shot IPC all-reduce (csrc/kernels/allreduce.hip):
-// operator_amd._C.CustomAllReduce. The handle exchange itself happens in
+// operator_amd._S.CustomAllReduce. The handle exchange itself happens in
 // Python over the process group (operator_amd/parallel/custom_ar.py); this
 // object owns the local fine-grained buffer and the opened peer mappings.
 #include <torch/extension.h>

@@ -1,0 +1,435 @@
+// Python bindings of the general decoder ops (operator_amd._C): hyper-connection streams,
+// QKV head preparation, attention with any head size, routed experts, fp32 products.
+//
+// As in bindings.cpp, every shape a kernel's grid or addressing relies on is checked on the
+// host before the launch.
+#include <torch/extension.h>
+#include <c10/hip/HIPStream.h>
+#include <ATen/hip/impl/HIPGuardImplMasqueradingAsCUDA.h>
+#include <ATen/hip/impl/HIPStreamMasqueradingAsCUDA.h>
+
+#include "kernels/kernels.h"
+
+namespace {
+
+using oamd::bf16_t;
+using OptT = c10::optional<at::Tensor>;
+
+hipStream_t cur_stream() { return c10::hip::getCurrentHIPStreamMasqueradingAsCUDA().stream(); }
+
+#define RC(call)                                                         \
+  do {                                                                   \
+    int rc__ = (call);                                                   \
+    TORCH_CHECK(rc__ == 0, "kernel launch failed: " #call " rc=", rc__); \
+  } while (0)
+
+// contiguous GPU tensor of `dt` with exactly (or at least) n elements
+void need(const at::Tensor& t, at::ScalarType dt, int64_t n, const char* what, bool at_least = false) {
+  TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == dt, what, ": contiguous GPU tensor of ", dt,
+              " expected, got ", t.scalar_type());
+  TORCH_CHECK(at_least ? t.numel() >= n : t.numel() == n, what, ": ", n, " elements expected, got ", t.numel());
+}
+
+template <typename T>
+T* p(const at::Tensor& t) { return reinterpret_cast<T*>(t.data_ptr()); }
+template <typename T>
+T* op(const OptT& t) { return t.has_value() ? reinterpret_cast<T*>(t->data_ptr()) : nullptr; }
+void* vp(const OptT& t) { return t.has_value() ? t->data_ptr() : nullptr; }
+
+bool elem_f32(const at::Tensor& t, const char* what) {
+  TORCH_CHECK(t.scalar_type() == at::kFloat || t.scalar_type() == at::kBFloat16, what, ": bf16 or fp32 expected");
+  return t.scalar_type() == at::kFloat;
+}
+
+// x [T, S, ld] fp32 streams; h [rows, ld] output. ids: first step. y / slabs / e: see StreamStep.
+void stream_step(at::Tensor& x, at::Tensor& h, int64_t width, const at::Tensor& w, double eps, const OptT& in,
+                 const OptT& ids, const OptT& table, double emb_scale, const OptT& y, const OptT& slabs,
+                 int64_t splits, const OptT& gate, const OptT& e, const OptT& epos, int64_t top, const OptT& mix,
+                 const OptT& out, const OptT& rows, bool write_x) {
+  TORCH_CHECK(x.dim() == 3 && h.dim() == 2 && h.size(1) == x.size(2), "stream_step: x [T, S, ld], h [rows, ld]");
+  const int64_t T = x.size(0), S = x.size(1), ld = x.size(2), n = h.size(0);
+  need(x, at::kFloat, T * S * ld, "x");
+  const bool f32 = elem_f32(h, "h");
+  const auto dt = h.scalar_type();
+  need(h, dt, n * ld, "h");
+  need(w, at::kFloat, ld, "norm weight");
+  TORCH_CHECK(width >= 1 && width <= ld, "stream_step: width");
+  oamd::StreamStep a{};
+  a.x = p<float>(x);
+  a.S = (int)S;
+  a.width = (int)width;
+  a.ld = (int)ld;
+  if (ids.has_value()) {
+    TORCH_CHECK(table.has_value() && table->dim() == 2 && table->size(1) == ld, "stream_step: table [vocab, ld]");
+    need(*ids, at::kLong, T, "ids");
+    need(*table, dt, table->numel(), "table");
+    a.ids = p<int64_t>(*ids);
+    a.table = table->data_ptr();
+    a.vocab = table->size(0);
+    a.emb_scale = (float)emb_scale;
+  } else {
+    TORCH_CHECK(mix.has_value() && out.has_value(), "stream_step: mix and out of the finished sublayer");
+    need(*mix, at::kFloat, S * S, "mix");
+    need(*out, at::kFloat, S, "out");
+    a.mix = p<float>(*mix);
+    a.out = p<float>(*out);
+    if (slabs.has_value()) {
+      TORCH_CHECK(splits >= 1, "stream_step: splits");
+      need(*slabs, at::kFloat, splits * T * ld, "slabs", true);
+      a.yp = p<float>(*slabs);
+      a.ys = (int)splits;
+      a.y_slab = T * ld;
+    } else if (y.has_value()) {
+      need(*y, dt, T * ld, "y");
+      a.y = y->data_ptr();
+    }
+    if (gate.has_value()) {
+      need(*gate, at::kFloat, T, "gate");
+      a.gate = p<float>(*gate);
+    }
+    if (top > 0) {
+      TORCH_CHECK(e.has_value() && e->dim() == 2 && e->size(1) == ld, "stream_step: e [rows, ld]");
+      need(*e, dt, e->numel(), "e");
+      if (epos.has_value()) need(*epos, at::kInt, T * top, "epos");   // values: moe_sort rows, all below e's row count
+      else TORCH_CHECK(e->size(0) >= T * top, "stream_step: e rows");
+      a.e = e->data_ptr();
+      a.epos = op<int>(epos);
+      a.top = (int)top;
+    }
+  }
+  if (in.has_value()) {
+    need(*in, at::kFloat, S, "in");
+    a.in = p<float>(*in);
+  }
+  a.sum = !in.has_value();
+  a.w = p<float>(w);
+  a.h = h.data_ptr();
+  a.eps = (float)eps;
+  a.f32 = f32;
+  a.write_x = write_x;
+  if (rows.has_value()) {
+    need(*rows, at::kLong, n, "rows");
+    TORCH_CHECK(a.sum && !ids.has_value() && !write_x, "stream_step: rows only in a last step that keeps the streams");
+    a.rows = p<int64_t>(*rows);
+  } else {
+    TORCH_CHECK(n == T, "stream_step: h rows");
+  }
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  RC(oamd::stream_step(a, (int)n, cur_stream()));
+}
+
+void qkv_heads(const at::Tensor& qkv, const OptT& slabs, int64_t splits, const OptT& bias, const at::Tensor& pos,
+               const OptT& cos_t, const OptT& sin_t, int64_t rot_pairs, int64_t Hq, int64_t Hkv, int64_t dk,
+               bool norm, double eps, const OptT& v_first, const OptT& lam, at::Tensor& q_out, const OptT& k_out,
+               const OptT& v_out, const OptT& k_cache, const OptT& v_cache, const OptT& slots, int64_t dvp,
+               int64_t ncol) {
+  const bool f32 = elem_f32(q_out, "q_out");
+  const auto dt = q_out.scalar_type();
+  const int64_t T = pos.numel();
+  TORCH_CHECK(q_out.dim() == 3 && q_out.size(0) == T && q_out.size(1) == Hq, "qkv_heads: q_out [T, Hq, dkp]");
+  const int64_t dkp = q_out.size(2);
+  need(q_out, dt, T * Hq * dkp, "q_out");
+  need(pos, at::kLong, T, "pos");
+  TORCH_CHECK(Hq >= 1 && Hkv >= 1 && dk >= 1 && dk <= dkp && ncol >= (Hq + Hkv) * dkp + Hkv * dvp && ncol % 8 == 0 &&
+                  dkp % 8 == 0 && dvp % 8 == 0 && 2 * rot_pairs <= dk,
+              "qkv_heads: head sizes");
+  oamd::QkvHeads a{};
+  if (slabs.has_value()) {
+    need(*slabs, at::kFloat, splits * T * ncol, "slabs", true);
+    a.xp = p<float>(*slabs);
+    a.S = (int)splits;
+    a.slab = T * ncol;
+  } else {
+    need(qkv, dt, T * ncol, "qkv");
+    a.row = qkv.data_ptr();
+    a.S = 1;
+  }
+  a.ncol = (int)ncol;
+  if (bias.has_value()) {
+    need(*bias, at::kFloat, ncol, "bias");
+    a.bias = p<float>(*bias);
+  }
+  a.pos = p<int64_t>(pos);
+  if (rot_pairs > 0) {
+    TORCH_CHECK(cos_t.has_value() && sin_t.has_value() && cos_t->dim() == 2 && cos_t->sizes() == sin_t->sizes() &&
+                    cos_t->size(1) % 4 == 0 && cos_t->size(1) >= rot_pairs && cos_t->size(0) >= 1,
+                "qkv_heads: cos / sin [max_pos, >= rot_pairs, % 4]");
+    need(*cos_t, at::kFloat, cos_t->numel(), "cos");
+    need(*sin_t, at::kFloat, sin_t->numel(), "sin");
+    a.cos_t = p<float>(*cos_t);
+    a.sin_t = p<float>(*sin_t);
+    a.rot_ld = (int)cos_t->size(1);
+    a.max_pos = cos_t->size(0);
+  }
+  a.rot_pairs = (int)rot_pairs;
+  a.Hq = (int)Hq; a.Hkv = (int)Hkv; a.dk = (int)dk; a.dkp = (int)dkp; a.dvp = (int)dvp;
+  a.norm = norm;
+  a.eps = (float)eps;
+  if (v_first.has_value()) {
+    TORCH_CHECK(lam.has_value(), "qkv_heads: lam");
+    need(*v_first, dt, T * Hkv * dvp, "v_first");
+    need(*lam, at::kFloat, 1, "lam");
+    a.v_first = v_first->data_ptr();
+    a.lam = p<float>(*lam);
+  }
+  a.q_out = q_out.data_ptr();
+  if (k_out.has_value()) need(*k_out, dt, T * Hkv * dkp, "k_out");
+  if (v_out.has_value()) need(*v_out, dt, T * Hkv * dvp, "v_out");
+  a.k_out = vp(k_out);
+  a.v_out = vp(v_out);
+  a.page_size = 16;
+  if (k_cache.has_value()) {
+    TORCH_CHECK(v_cache.has_value() && slots.has_value(), "qkv_heads: k_cache needs v_cache and slots");
+    TORCH_CHECK(k_cache->dim() == 4 && v_cache->dim() == 4 && k_cache->size(1) == Hkv && v_cache->size(1) == Hkv &&
+                    k_cache->size(0) == v_cache->size(0) && k_cache->size(2) == v_cache->size(2) &&
+                    k_cache->size(3) == dkp && v_cache->size(3) == dvp,
+                "qkv_heads: cache [pages, Hkv, page, size]");
+    need(*k_cache, dt, k_cache->numel(), "k_cache");
+    need(*v_cache, dt, v_cache->numel(), "v_cache");
+    need(*slots, at::kLong, T, "slots");
+    a.k_cache = k_cache->data_ptr();
+    a.v_cache = v_cache->data_ptr();
+    a.slots = p<int64_t>(*slots);
+    a.page_size = (int)k_cache->size(2);
+  }
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(pos.device());
+  RC(oamd::qkv_heads(a, (int)T, f32, cur_stream()));
+}
+
+// o: [T, o_ld] rows, head h at column h * dvp
+void attn_gd_prefill(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, at::Tensor& o,
+                     const at::Tensor& cu, const OptT& work_seq, const OptT& work_q0, double scale, const OptT& pk,
+                     const OptT& pv, const OptT& seq_pfx) {
+  TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && v.dim() == 3 && o.dim() == 2, "attn_gd_prefill: q, k, v [T, H, d], o [T, ld]");
+  const int64_t T = q.size(0), Hq = q.size(1), dkp = q.size(2), Hkv = k.size(1), dvp = v.size(2);
+  const bool f32 = elem_f32(q, "q");
+  const auto dt = q.scalar_type();
+  need(q, dt, T * Hq * dkp, "q");
+  need(k, dt, T * Hkv * dkp, "k");
+  need(v, dt, T * Hkv * dvp, "v");
+  need(o, dt, T * o.size(1), "o");
+  TORCH_CHECK(v.size(1) == Hkv && Hkv >= 1 && Hq % Hkv == 0 && o.size(1) >= Hq * dvp, "attn_gd_prefill: heads");
+  need(cu, at::kInt, cu.numel(), "cu_seqlens");
+  const int64_t seqs = cu.numel() - 1;
+  TORCH_CHECK(seqs >= 1, "attn_gd_prefill: cu_seqlens");
+  if (pk.has_value()) {
+    TORCH_CHECK(pv.has_value() && seq_pfx.has_value() && pk->dim() == 3 && pk->size(0) == pv->size(0), "attn_gd_prefill: prefix");
+    need(*pk, dt, pk->size(0) * Hkv * dkp, "pk");
+    need(*pv, dt, pk->size(0) * Hkv * dvp, "pv");
+    need(*seq_pfx, at::kInt, seqs, "seq_pfx");
+  }
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(q.device());
+  if (f32) {
+    oamd::AttnF32 a{};
+    a.q = p<float>(q); a.k = p<float>(k); a.v = p<float>(v); a.o = p<float>(o);
+    a.o_ld = (int)o.size(1);
+    a.cu_seqlens = p<int>(cu);
+    a.num_seqs = (int)seqs;
+    a.Hkv = (int)Hkv; a.dkp = (int)dkp; a.dvp = (int)dvp;
+    a.scale = (float)scale;
+    a.pk = op<float>(pk); a.pv = op<float>(pv); a.seq_pfx = op<int>(seq_pfx);
+    RC(oamd::attn_f32(a, (int)T, (int)Hq, false, cur_stream()));
+    return;
+  }
+  TORCH_CHECK(work_seq.has_value() && work_q0.has_value(), "attn_gd_prefill: work list");
+  need(*work_seq, at::kInt, work_seq->numel(), "work_seq");
+  need(*work_q0, at::kInt, work_seq->numel(), "work_q0");
+  oamd::AttnPrefill a{};
+  a.q = p<bf16_t>(q); a.k = p<bf16_t>(k); a.v = p<bf16_t>(v); a.o = p<bf16_t>(o);
+  a.o_ld = (int)o.size(1);
+  TORCH_CHECK(a.o_ld % 4 == 0, "attn_gd_prefill: o rows");
+  a.cu_seqlens = p<int>(cu); a.work_seq = p<int>(*work_seq); a.work_q0 = p<int>(*work_q0);
+  a.Hkv = (int)Hkv;
+  a.G = (int)(Hq / Hkv);
+  a.gc = a.G % 4 == 0 ? 4 : a.G % 3 == 0 ? 3 : a.G % 2 == 0 ? 2 : 1;
+  a.dkp = (int)dkp; a.dvp = (int)dvp;
+  a.scale_log2 = (float)(scale * 1.4426950408889634);
+  a.pk = op<bf16_t>(pk); a.pv = op<bf16_t>(pv); a.seq_pfx = op<int>(seq_pfx);
+  RC(oamd::attn_gd_prefill(a, (int)work_seq->numel(), cur_stream()));
+}
+
+void attn_gd_decode(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache, const at::Tensor& bt,
+                    const at::Tensor& lens, at::Tensor& o, const OptT& o_part, const OptT& ml_part,
+                    int64_t num_splits, double scale) {
+  TORCH_CHECK(q.dim() == 3 && k_cache.dim() == 4 && v_cache.dim() == 4 && bt.dim() == 2 && o.dim() == 2,
+              "attn_gd_decode: q [B, Hq, d], cache [pages, Hkv, page, d], bt [B, max_pages], o [B, ld]");
+  const int64_t B = q.size(0), Hq = q.size(1), dkp = q.size(2), Hkv = k_cache.size(1), P = k_cache.size(2),
+                dvp = v_cache.size(3);
+  const bool f32 = elem_f32(q, "q");
+  const auto dt = q.scalar_type();
+  need(q, dt, B * Hq * dkp, "q");
+  need(k_cache, dt, k_cache.numel(), "k_cache");
+  need(v_cache, dt, v_cache.numel(), "v_cache");
+  need(bt, at::kInt, B * bt.size(1), "block_tables");
+  need(lens, at::kInt, B, "seq_lens");
+  need(o, dt, B * o.size(1), "o");
+  TORCH_CHECK(k_cache.size(3) == dkp && v_cache.size(1) == Hkv && v_cache.size(2) == P && v_cache.size(0) == k_cache.size(0) &&
+                  Hq % Hkv == 0 && o.size(1) >= Hq * dvp && P >= 16 && (P & (P - 1)) == 0 && num_splits >= 1,
+              "attn_gd_decode: shapes");
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(q.device());
+  if (f32) {
+    oamd::AttnF32 a{};
+    a.q = p<float>(q); a.k = p<float>(k_cache); a.v = p<float>(v_cache); a.o = p<float>(o);
+    a.o_ld = (int)o.size(1);
+    a.block_tables = p<int>(bt); a.seq_lens = p<int>(lens);
+    a.Hkv = (int)Hkv; a.dkp = (int)dkp; a.dvp = (int)dvp;
+    a.page_size = (int)P; a.max_pages = (int)bt.size(1);
+    a.scale = (float)scale;
+    RC(oamd::attn_f32(a, (int)B, (int)Hq, true, cur_stream()));
+    return;
+  }
+  oamd::AttnDecode a{};
+  a.q = p<bf16_t>(q); a.k_cache = p<bf16_t>(k_cache); a.v_cache = p<bf16_t>(v_cache);
+  a.block_tables = p<int>(bt); a.seq_lens = p<int>(lens);
+  a.out = p<bf16_t>(o);
+  a.o_ld = (int)o.size(1);
+  if (num_splits > 1) {
+    TORCH_CHECK(o_part.has_value() && ml_part.has_value(), "attn_gd_decode: workspace");
+    need(*o_part, at::kFloat, B * Hq * num_splits * dvp, "o_part", true);
+    need(*ml_part, at::kFloat, B * Hq * num_splits * 2, "ml_part", true);
+    a.o_part = p<float>(*o_part); a.ml_part = p<float>(*ml_part);
+  }
+  a.Hkv = (int)Hkv; a.G = (int)(Hq / Hkv); a.dkp = (int)dkp; a.dvp = (int)dvp;
+  a.page_size = (int)P; a.max_pages = (int)bt.size(1); a.num_splits = (int)num_splits;
+  int lg = 0;
+  while ((1 << lg) < P) ++lg;
+  a.log2_page = lg;
+  a.scale_log2 = (float)(scale * 1.4426950408889634);
+  RC(oamd::attn_gd_decode(a, (int)B, cur_stream()));
+}
+
+void gemm_f32(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, bool silu_gu, const OptT& gtab, const OptT& rscale) {
+  TORCH_CHECK(x.dim() == 2 && y.dim() == 2, "gemm_f32: x [M, K], y [M, N]");
+  const int64_t M = x.size(0), K = x.size(1), N = w.size(-2);
+  need(x, at::kFloat, M * K, "x");
+  need(w, at::kFloat, w.numel(), "w");
+  need(y, at::kFloat, M * (silu_gu ? N / 2 : N), "y");
+  TORCH_CHECK(w.size(-1) == K && y.size(0) == M && K % 16 == 0 && (!silu_gu || N % 128 == 0), "gemm_f32: shapes");
+  if (gtab.has_value()) {
+    TORCH_CHECK(w.dim() == 3 && M % 64 == 0, "gemm_f32: expert rows come in 64-row tiles, w [experts, N, K]");
+    need(*gtab, at::kInt, 1 + M / 64, "gtab", true);
+  } else {
+    TORCH_CHECK(w.dim() == 2, "gemm_f32: w [N, K]");
+  }
+  if (rscale.has_value()) need(*rscale, at::kFloat, M, "rscale");
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  RC(oamd::gemm_f32(p<float>(x), p<float>(w), p<float>(y), (int)M, (int)N, (int)K, (int)y.size(1), silu_gu,
+                    op<int>(gtab), op<float>(rscale), cur_stream()));
+}
+
+void moe_route(const at::Tensor& h, const at::Tensor& wr, int64_t E, at::Tensor& ids, at::Tensor& weights,
+               const OptT& gate, const OptT& logits) {
+  TORCH_CHECK(h.dim() == 2 && wr.dim() == 2 && ids.dim() == 2 && wr.size(1) == h.size(1), "moe_route: h [T, K], wr [rows, K]");
+  const int64_t T = h.size(0), K = h.size(1), rows = wr.size(0), top = ids.size(1);
+  need(h, at::kBFloat16, T * K, "h");
+  need(wr, at::kBFloat16, rows * K, "wr");
+  need(ids, at::kInt, T * top, "ids");
+  need(weights, at::kFloat, T * top, "weights");
+  if (gate.has_value()) need(*gate, at::kFloat, T, "gate");
+  if (logits.has_value()) need(*logits, at::kFloat, T * E, "logits");
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(h.device());
+  RC(oamd::moe_route(p<bf16_t>(h), p<bf16_t>(wr), (int)T, (int)K, (int)E, (int)rows, (int)top, p<int>(ids),
+                     p<float>(weights), op<float>(gate), op<float>(logits), cur_stream()));
+}
+
+void moe_topk(const at::Tensor& logits, int64_t E, at::Tensor& ids, at::Tensor& weights, const OptT& gate) {
+  TORCH_CHECK(logits.dim() == 2 && ids.dim() == 2, "moe_topk: logits [T, ld], ids [T, top]");
+  const int64_t T = logits.size(0), top = ids.size(1);
+  need(logits, at::kFloat, logits.numel(), "logits");
+  need(ids, at::kInt, T * top, "ids");
+  need(weights, at::kFloat, T * top, "weights");
+  if (gate.has_value()) need(*gate, at::kFloat, T, "gate");
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(logits.device());
+  RC(oamd::moe_topk(p<float>(logits), (int)logits.size(1), (int)T, (int)E, (int)top, p<int>(ids), p<float>(weights),
+                    op<float>(gate), cur_stream()));
+}
+
+// ids must come from moe_route / moe_topk (every value inside [0, E))
+void moe_sort(const at::Tensor& ids, const at::Tensor& weights, int64_t E, int64_t bm, at::Tensor& pos, at::Tensor& src,
+              at::Tensor& rscale, at::Tensor& gtab) {
+  TORCH_CHECK(ids.dim() == 2, "moe_sort: ids [T, top]");
+  const int64_t slots = ids.numel(), rows = src.numel();
+  need(ids, at::kInt, slots, "ids");
+  need(weights, at::kFloat, slots, "weights");
+  need(pos, at::kInt, slots, "pos");
+  need(src, at::kInt, rows, "src");
+  need(rscale, at::kFloat, rows, "rscale");
+  TORCH_CHECK(bm > 0 && rows % bm == 0, "moe_sort: rows");
+  need(gtab, at::kInt, 1 + rows / bm, "gtab", true);
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(ids.device());
+  RC(oamd::moe_sort(p<int>(ids), p<float>(weights), (int)slots, (int)ids.size(1), (int)E, (int)bm, (int)rows,
+                    p<int>(pos), p<int>(src), p<float>(rscale), p<int>(gtab), cur_stream()));
+}
+
+void moe_gather(const at::Tensor& h, const at::Tensor& src, const at::Tensor& gtab, int64_t bm, at::Tensor& xp) {
+  TORCH_CHECK(h.dim() == 2 && xp.dim() == 2 && h.size(1) == xp.size(1) && h.scalar_type() == xp.scalar_type(), "moe_gather: shapes");
+  need(h, h.scalar_type(), h.numel(), "h");
+  need(xp, h.scalar_type(), xp.numel(), "xp");
+  need(src, at::kInt, xp.size(0), "src");
+  need(gtab, at::kInt, 1 + xp.size(0) / bm, "gtab", true);
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(h.device());
+  RC(oamd::moe_gather(h.data_ptr(), p<int>(src), p<int>(gtab), (int)bm, (int)xp.size(0), xp.data_ptr(),
+                      (int)(h.size(1) * h.element_size()), cur_stream()));
+}
+
+void moe_gemm_skinny(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const at::Tensor& ids,
+                     const at::Tensor& weights, int64_t div, bool silu_gu) {
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 3 && y.dim() == 2 && w.size(2) == x.size(1), "moe_gemm_skinny: x [.., K], w [E, N, K]");
+  const int64_t slots = ids.numel(), E = w.size(0), N = w.size(1), K = w.size(2);
+  need(x, at::kBFloat16, x.numel(), "x");
+  need(w, at::kBFloat16, w.numel(), "w");
+  need(ids, at::kInt, slots, "ids");
+  need(weights, at::kFloat, slots, "weights");
+  need(y, at::kBFloat16, slots * (silu_gu ? N / 2 : N), "y");
+  TORCH_CHECK(div >= 1 && x.size(0) * div >= slots && E <= 65535, "moe_gemm_skinny: rows");
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  RC(oamd::moe_gemm_skinny(p<bf16_t>(x), p<bf16_t>(w), p<bf16_t>(y), p<int>(ids), p<float>(weights), (int)slots,
+                           (int)div, (int)E, (int)N, (int)K, silu_gu, cur_stream()));
+}
+
+void moe_gemm_tile(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const at::Tensor& gtab, const OptT& rscale,
+                   bool silu_gu) {
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 3 && y.dim() == 2 && w.size(2) == x.size(1), "moe_gemm_tile: x [rows, K], w [E, N, K]");
+  const int64_t M = x.size(0), N = w.size(1), K = w.size(2);
+  need(x, at::kBFloat16, M * K, "x");
+  need(w, at::kBFloat16, w.numel(), "w");
+  need(y, at::kBFloat16, M * (silu_gu ? N / 2 : N), "y");
+  TORCH_CHECK(M % 256 == 0 && K <= (1 << 21), "moe_gemm_tile: 256-row tiles");
+  need(gtab, at::kInt, 1 + M / 256, "gtab", true);
+  if (rscale.has_value()) need(*rscale, at::kFloat, M, "rscale");
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  RC(oamd::moe_gemm_tile(p<bf16_t>(x), p<bf16_t>(w), p<bf16_t>(y), (int)M, (int)N, (int)K, silu_gu, p<int>(gtab),
+                         op<float>(rscale), cur_stream()));
+}
+
+}  // namespace
+
+void register_decoder_bindings(pybind11::module_& m) {
+  namespace py = pybind11;
+  const py::none no;
+  m.def("stream_step", &stream_step, py::arg("x"), py::arg("h"), py::arg("width"), py::arg("w"), py::arg("eps"),
+        py::arg("in_") = no, py::arg("ids") = no, py::arg("table") = no, py::arg("emb_scale") = 1.0, py::arg("y") = no,
+        py::arg("slabs") = no, py::arg("splits") = 1, py::arg("gate") = no, py::arg("e") = no, py::arg("epos") = no,
+        py::arg("top") = 0, py::arg("mix") = no, py::arg("out") = no, py::arg("rows") = no, py::arg("write_x") = true);
+  m.def("qkv_heads", &qkv_heads, py::arg("qkv"), py::arg("slabs"), py::arg("splits"), py::arg("bias"), py::arg("pos"),
+        py::arg("cos"), py::arg("sin"), py::arg("rot_pairs"), py::arg("Hq"), py::arg("Hkv"), py::arg("dk"),
+        py::arg("norm"), py::arg("eps"), py::arg("v_first"), py::arg("lam"), py::arg("q_out"), py::arg("k_out"),
+        py::arg("v_out"), py::arg("k_cache"), py::arg("v_cache"), py::arg("slots"), py::arg("dvp"), py::arg("ncol"));
+  m.def("attn_gd_prefill", &attn_gd_prefill, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("o"), py::arg("cu"),
+        py::arg("work_seq") = no, py::arg("work_q0") = no, py::arg("scale") = 1.0, py::arg("pk") = no,
+        py::arg("pv") = no, py::arg("seq_pfx") = no);
+  m.def("attn_gd_decode", &attn_gd_decode, py::arg("q"), py::arg("k_cache"), py::arg("v_cache"), py::arg("bt"),
+        py::arg("lens"), py::arg("o"), py::arg("o_part") = no, py::arg("ml_part") = no, py::arg("num_splits") = 1,
+        py::arg("scale") = 1.0);
+  m.def("gemm_f32", &gemm_f32, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("silu_gu") = false,
+        py::arg("gtab") = no, py::arg("rscale") = no);
+  m.def("moe_route", &moe_route, py::arg("h"), py::arg("wr"), py::arg("E"), py::arg("ids"), py::arg("weights"),
+        py::arg("gate") = no, py::arg("logits") = no);
+  m.def("moe_topk", &moe_topk, py::arg("logits"), py::arg("E"), py::arg("ids"), py::arg("weights"), py::arg("gate") = no);
+  m.def("moe_sort", &moe_sort);
+  m.def("moe_gather", &moe_gather);
+  m.def("moe_gemm_skinny", &moe_gemm_skinny, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("ids"),
+        py::arg("weights"), py::arg("div"), py::arg("silu_gu"));
+  m.def("moe_gemm_tile", &moe_gemm_tile, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("gtab"),
+        py::arg("rscale") = no, py::arg("silu_gu") = false);
+}

@@ -556,20 +556,31 @@ __global__ void __launch_bounds__(256) gemm_tile256_h4_kernel(const bf16_t* __re
 // W stays in the Infinity Cache), 2: W (wide N: the W panels come from HBM); 160 KiB of LDS.
 // OPT (A/B arms): bit 0 = s_setprio 1 over the MFMA streams; bit 1 = MFMA groups over W fragments
 // (srcA fixed for 8 MFMAs, as hipBLASLt's MT256x256x64 loop issues them)
-template <int EPI, int DEEP = 0, int OPT = 0>
+// GRP: routed experts. X's rows are expert segments padded to 256-row tiles (moe_sort): gtab[0] =
+// row tiles, gtab[1 + i] = expert of row tile i, W [experts][N][K]; rscale[row] multiplies both
+// SwiGLU operands (an expert reads its token scaled by the router weight).
+template <int EPI, int DEEP = 0, int OPT = 0, bool GRP = false>
 __global__ void __launch_bounds__(256) gemm_tile256_p5_kernel(const bf16_t* __restrict__ X,
                                                               const bf16_t* __restrict__ W, bf16_t* __restrict__ Y,
                                                               const bf16_t* __restrict__ bias, int M, int N, int K,
-                                                              int ldy, int group_m) {
+                                                              int ldy, int group_m,
+                                                              const int* __restrict__ gtab = nullptr,
+                                                              const float* __restrict__ rscale = nullptr) {
   constexpr int AUX = 16;
   constexpr int kHalf = 32768;   // one operand of a K-step: 256 rows x 128 B
   __shared__ __attribute__((aligned(1024))) char lds[DEEP ? 5 * kHalf : 4 * kHalf];
   const int tid = threadIdx.x, lane = tid & 63;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int wm = w >> 1, wn = w & 1;
-  const int mt = (M + kT - 1) / kT, nt = (N + kT - 1) / kT;
+  int mt = (M + kT - 1) / kT;
+  if constexpr (GRP) mt = min(mt, gtab[0]);   // tiles the router really filled
+  const int nt = (N + kT - 1) / kT;
   const int ntiles = mt * nt;
   const int G = gridDim.x;
+  auto wbase = [&](int m) -> const bf16_t* {   // the weight of row tile m0 / 256's expert
+    if constexpr (GRP) return W + (int64_t)gtab[1 + m / kT] * N * K;
+    else return W;
+  };
   const int slot = xcd_remap(blockIdx.x, G);
   const int T = K / kBK;
   const int gsz = group_m * nt;
@@ -613,10 +624,10 @@ __global__ void __launch_bounds__(256) gemm_tile256_p5_kernel(const bf16_t* __re
   Cur cx{0, 0, nullptr, 0}, cw{0, 0, nullptr, 0};
   {
     int m0 = 0, n0 = 0;
-    if (!tile_rc(0, m0, n0)) return;   // grid <= tiles: never taken
+    if (!tile_rc(0, m0, n0)) return;   // grid <= tiles: taken only when GRP has fewer tiles than the bound
     cx.p = X + (int64_t)m0 * K;
     cx.n = (int)((uint32_t)min(M - m0, kT) * (uint32_t)K * 2u);
-    cw.p = W + (int64_t)n0 * K;
+    cw.p = wbase(m0) + (int64_t)n0 * K;
     cw.n = (int)((uint32_t)min(N - n0, kT) * (uint32_t)K * 2u);
   }
   auto advance = [&](Cur& c, bool isx) {
@@ -626,7 +637,7 @@ __global__ void __launch_bounds__(256) gemm_tile256_p5_kernel(const bf16_t* __re
         ++c.r;
         c.kt = 0;
         const int row0 = isx ? m0n : n0n;
-        c.p = (isx ? X : W) + (int64_t)row0 * K;
+        c.p = (isx ? X : wbase(m0n)) + (int64_t)row0 * K;
         c.n = (int)((uint32_t)min((isx ? M : N) - row0, kT) * (uint32_t)K * 2u);
       } else {
         c.kt = T - 1;   // past the block's last tile: harmless re-loads of its last step
@@ -826,13 +837,19 @@ __global__ void __launch_bounds__(256) gemm_tile256_p5_kernel(const bf16_t* __re
     for (int i = 0; i < 8; ++i) {
       const int tok = m0 + wm * 128 + i * 16 + l15;
       bf16_t* yrow = Y + (int64_t)tok * ldy;
+      float rsc = 1.f;
+      if constexpr (GRP && EPI == kEpiSilu) rsc = rscale[min(tok, M - 1)];
 #pragma unroll
       for (int f = 0; f < 2; ++f) {
         if constexpr (EPI == kEpiSilu) {
           f32x4 o[2];
 #pragma unroll
           for (int jj = 0; jj < 2; ++jj) {
-            const f32x4 gt = acc[i][f * 4 + jj], up = acc[i][f * 4 + 2 + jj];
+            f32x4 gt = acc[i][f * 4 + jj], up = acc[i][f * 4 + 2 + jj];
+            if constexpr (GRP) {
+              gt *= rsc;
+              up *= rsc;
+            }
 #pragma unroll
             for (int rr = 0; rr < 4; ++rr) {
               const float gg = bf2f(f2bf(gt[rr]));
@@ -915,6 +932,20 @@ static int device_cus() {
     cus[dev] = n;
   }
   return cus[dev];
+}
+
+int moe_gemm_tile(const bf16_t* X, const bf16_t* W, bf16_t* Y, int max_rows, int N, int K, bool silu_gu,
+                  const int* gtab, const float* rscale, hipStream_t stream) {
+  if (max_rows == 0) return 0;
+  if (max_rows % kT != 0 || N < 16 || N % 16 != 0 || K < 2 * kBK || K % kBK != 0 || gtab == nullptr) return -1;
+  if (silu_gu && (N % 128 != 0 || rscale == nullptr)) return -2;
+  const int grid = min((max_rows / kT) * ((N + kT - 1) / kT), device_cus());
+  if (silu_gu)
+    gemm_tile256_p5_kernel<kEpiSilu, 0, 0, true><<<grid, 256, 0, stream>>>(X, W, Y, nullptr, max_rows, N, K, N / 2, 4, gtab, rscale);
+  else
+    gemm_tile256_p5_kernel<kEpiStore, 0, 0, true><<<grid, 256, 0, stream>>>(X, W, Y, nullptr, max_rows, N, K, N, 4, gtab, rscale);
+  OAMD_LAUNCH_CHECK();
+  return 0;
 }
 
 int gemm_tile(const bf16_t* X, const bf16_t* W, bf16_t* Y, const bf16_t* bias, int M, int N, int K, int ldy,

@@ -146,4 +146,121 @@ int car_all_reduce(const void* in, void* out, int64_t bytes, bool bf16, int rank
                    size_t cap_bytes, int blocks, uint32_t* herr_dev, double timeout_s, int proto,
                    hipStream_t stream);
 
+// Hyper-connection step over S parallel fp32 residual streams (streams.hip): finishes one
+// sublayer (mix [from][to], out) and starts the next (in, norm weight w).
+struct StreamStep {
+  float* x;                 // [T][S][ld] streams
+  int S, width, ld;         // true width and padded row length (ld % 8 == 0)
+  const int64_t* ids;       // first step: token ids (streams written from the embedding), else nullptr
+  const void* table;        // [vocab][ld], element type of h
+  int64_t vocab;
+  float emb_scale;
+  const float* yp;          // sublayer output as ys fp32 slabs, y_slab elements apart, or
+  int ys;
+  int64_t y_slab;
+  const void* y;            // as rows [T][ld] of h's type (nullptr: none)
+  const float* gate;        // [T] logits; sigmoid(gate) scales yp / y (nullptr: 1)
+  const void* e;            // rows added on top: row epos[t * top + k] (epos nullptr: t * top + k) of e [.][ld]
+  const int* epos;
+  int top;                  // 0: none
+  const float *mix, *out;   // [S][S], [S] (fp32)
+  const float* in;          // [S]
+  const float* w;           // [ld] norm weight (fp32, zero past width)
+  void* h;                  // [rows][ld] bf16 or fp32
+  float eps;
+  bool f32;                 // element type of table / y / e / h
+  bool sum;                 // last step: u is the plain sum of the streams
+  bool write_x;             // write the new streams back
+  const int64_t* rows;      // last step: rows to produce (nullptr: all)
+};
+int stream_step(const StreamStep& a, int n_rows, hipStream_t stream);
+
+// Packed QKV rows -> rotated, per-head-normalised q / k, (mixed) v and the paged cache
+// (qkv_heads.hip).
+struct QkvHeads {
+  const float* xp;          // S fp32 slabs [S][T][ncol], slab elements apart, or nullptr
+  int S;
+  int64_t slab;
+  const void* row;          // [T][ncol] rows (bf16 / fp32)
+  int ncol;
+  const float* bias;        // [ncol] or nullptr
+  const int64_t* pos;
+  const float *cos_t, *sin_t;   // [max_pos][rot_ld]
+  int rot_pairs, rot_ld;
+  int64_t max_pos;
+  int Hq, Hkv, dk, dkp, dvp;    // dk: true q/k size (the norm's mean); dkp, dvp: stored sizes
+  bool norm;
+  float eps;
+  const void* v_first;      // [T][Hkv][dvp] or nullptr: v <- (1 - lam) v + lam v_first
+  const float* lam;
+  void *q_out, *k_out, *v_out;
+  void *k_cache, *v_cache;
+  const int64_t* slots;     // < 0: not cached
+  int page_size;
+};
+int qkv_heads(const QkvHeads& a, int tokens, bool f32, hipStream_t stream);
+
+// General-head-size attention, bf16 (attn_gd_prefill.hip, attn_gd_decode.hip)
+struct AttnPrefill {
+  const bf16_t *q, *k, *v;      // [T][Hq][dkp], [T][Hkv][dkp], [T][Hkv][dvp]
+  bf16_t* o;                    // row t, head h at t * o_ld + h * dvp
+  int o_ld;
+  const int *cu_seqlens, *work_seq, *work_q0;   // work items of 128 query rows
+  int Hkv, G, gc, dkp, dvp;     // G query heads per kv head, gc of them (<= 4, divides G) per workgroup
+  float scale_log2;
+  const bf16_t *pk, *pv;        // shared-prefix rows and per-sequence prefix lengths, or nullptr
+  const int* seq_pfx;
+};
+int attn_gd_prefill(const AttnPrefill& a, int num_work, hipStream_t stream);
+struct AttnDecode {
+  const bf16_t* q;              // [B][Hq][dkp]
+  const bf16_t *k_cache, *v_cache;
+  const int *block_tables, *seq_lens;
+  bf16_t* out;
+  int o_ld;
+  float *o_part, *ml_part;      // [B][Hq][num_splits][dvp], [..][2] when num_splits > 1
+  int Hkv, G, dkp, dvp, page_size, log2_page, max_pages, num_splits;
+  float scale_log2;
+};
+int attn_gd_decode(const AttnDecode& a, int B, hipStream_t stream);
+
+// fp32 forms (f32.hip)
+int gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, int ldy, bool silu_gu, const int* gtab,
+             const float* rscale, hipStream_t stream);
+struct AttnF32 {
+  const float *q, *k, *v;       // k / v: packed rows, or the paged cache (token rows)
+  float* o;
+  int o_ld;
+  const int *cu_seqlens;        // packed: [num_seqs + 1]
+  int num_seqs;
+  const int *block_tables, *seq_lens;   // paged
+  int Hkv, dkp, dvp, page_size, max_pages;
+  float scale;
+  const float *pk, *pv;
+  const int* seq_pfx;
+};
+int attn_f32(const AttnF32& a, int rows, int Hq, bool paged, hipStream_t stream);
+
+// Routed experts (moe.hip)
+// Router: logits of E experts (rows 0..E-1 of wr) and, with `gate`, one more row E, in fp32;
+// per token the `top` largest, scored by sigmoid.
+int moe_route(const bf16_t* h, const bf16_t* wr, int T, int K, int E, int rows_w, int top, int* ids, float* weights,
+              float* gate, float* logits, hipStream_t stream);
+int moe_topk(const float* logits, int ld, int T, int E, int top, int* ids, float* weights, float* gate,
+             hipStream_t stream);
+// Expert-sorted row order, every expert's segment padded to bm rows: pos[slot] = row, src[row] =
+// token (-1: padding), rscale[row], gtab = {tiles, expert of tile i ...}; slots = T * top.
+int moe_sort(const int* ids, const float* weights, int slots, int top, int E, int bm, int max_rows, int* pos, int* src,
+             float* rscale, int* gtab, hipStream_t stream);
+// xp[row] = h[src[row]] (zeros for padding) for the rows of gtab's tiles; row_bytes % 16 == 0
+int moe_gather(const void* h, const int* src, const int* gtab, int bm, int max_rows, void* xp, int row_bytes,
+               hipStream_t stream);
+// Decode: row slot of Y = X row (slot / div) . W[ids[slot]]^T; silu_gu: SwiGLU of weights[slot] * the
+// products over the 64-row interleaved gate|up weight. W [E][N][K], K % 64 == 0, N % 16 == 0 (silu: 128).
+int moe_gemm_skinny(const bf16_t* X, const bf16_t* W, bf16_t* Y, const int* ids, const float* weights, int slots,
+                    int div, int E, int N, int K, bool silu_gu, hipStream_t stream);
+// Prefill: rows sorted by moe_sort with bm = 256, persistent 256 x 256 tiles (gemm_tile.hip).
+int moe_gemm_tile(const bf16_t* X, const bf16_t* W, bf16_t* Y, int max_rows, int N, int K, bool silu_gu,
+                  const int* gtab, const float* rscale, hipStream_t stream);
+
 }  // namespace oamd

@@ -1,0 +1,181 @@
+// From a packed QKV projection to attention operands, one pass per token:
+//   q, k  (+ bias) -> rotary positions on the first rot_pairs pairs of a head (dimension
+//         2i with 2i + 1) -> divided by their root mean square over the head (no weight)
+//   v     (+ bias) -> (1 - lam) v + lam v_first when the layer mixes values
+//   k, v  -> paged cache (and, for a prefill, packed copies the attention reads)
+// Any head size: a head occupies dkp (q, k) or dvp (v) columns, the true size rounded up
+// by the loader with zero weights, so the tail is zero everywhere.
+// Row layout: [q Hq x dkp | k Hkv x dkp | v Hkv x dvp | unused up to ncol].
+//
+// bf16 cache layout (read by attn_gd.hip): 16-token tiles. K tile [dkp/8 chunk][16 token]
+// [8 dims]; V tile [dvp/32][4 token group][16 dims][2 half][4 token] (dim d = 32 b + 16 half
+// + i). Every MFMA fragment of the decode kernel is then one contiguous 1 KiB wave access.
+// fp32 cache: token rows.
+#include "common.h"
+#include "kernels.h"
+
+namespace oamd {
+
+namespace {
+
+template <typename T>
+__device__ __forceinline__ void st8(T* p, const float (&v)[8]);
+template <>
+__device__ __forceinline__ void st8<float>(float* p, const float (&v)[8]) {
+  *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
+  *reinterpret_cast<f32x4*>(p + 4) = f32x4{v[4], v[5], v[6], v[7]};
+}
+template <>
+__device__ __forceinline__ void st8<bf16_t>(bf16_t* p, const float (&v)[8]) {
+  *reinterpret_cast<uint4*>(p) =
+      make_uint4(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]), pack_bf2(v[4], v[5]), pack_bf2(v[6], v[7]));
+}
+
+template <typename T>
+__device__ __forceinline__ void ld8(const T* p, float (&v)[8]);
+template <>
+__device__ __forceinline__ void ld8<float>(const float* p, float (&v)[8]) {
+  const f32x4 a = *reinterpret_cast<const f32x4*>(p), b = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] = a[j], v[4 + j] = b[j];
+}
+template <>
+__device__ __forceinline__ void ld8<bf16_t>(const bf16_t* p, float (&v)[8]) {
+  const u16x8 a = *reinterpret_cast<const u16x8*>(p);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] = bf2f(a[j]);
+}
+
+}  // namespace
+
+// GW lanes (a power of two >= dkp / 8) share a q / k head, 8 dims each; v is copied in
+// 8-dim items. Grid (tokens, items / 256).
+template <typename T, int GW>
+__global__ void __launch_bounds__(256) qkv_heads_kernel(const QkvHeads a) {
+  const int t = blockIdx.x;
+  const int it = blockIdx.y * 256 + threadIdx.x;
+  const int rot_items = (a.Hq + a.Hkv) * GW;
+  const int vch = a.dvp >> 3;
+  if (it >= rot_items + a.Hkv * vch) return;
+  auto load = [&](int col, float (&v)[8]) {
+    if (a.xp) {
+      const float* p = a.xp + (int64_t)t * a.ncol + col;
+      ld8<float>(p, v);
+      for (int s = 1; s < a.S; ++s) {
+        float w[8];
+        ld8<float>(p + s * a.slab, w);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] += w[j];
+      }
+    } else {
+      ld8<T>(static_cast<const T*>(a.row) + (int64_t)t * a.ncol + col, v);
+    }
+    if (a.bias) {
+      float b[8];
+      ld8<float>(a.bias + col, b);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] += b[j];
+    }
+  };
+  const int64_t slot = a.slots ? a.slots[t] : -1;
+  const int64_t page = slot >= 0 ? slot / a.page_size : 0;
+  const int off = slot >= 0 ? static_cast<int>(slot % a.page_size) : 0;
+  constexpr bool kF32 = sizeof(T) == 4;
+
+  if (it < rot_items) {
+    const int h = it / GW, c = it % GW;   // head, 8-dim chunk
+    const bool live = 8 * c < a.dkp;
+    float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (live) load(h * a.dkp + 8 * c, x);   // q heads then k heads: the same stride
+    if (live && 4 * c < a.rot_pairs) {
+      int64_t p = a.pos[t];
+      p = p < 0 ? 0 : (p >= a.max_pos ? a.max_pos - 1 : p);
+      const f32x4 cs = *reinterpret_cast<const f32x4*>(a.cos_t + p * a.rot_ld + 4 * c);
+      const f32x4 sn = *reinterpret_cast<const f32x4*>(a.sin_t + p * a.rot_ld + 4 * c);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (4 * c + j < a.rot_pairs) {
+          const float u = x[2 * j], v = x[2 * j + 1];
+          x[2 * j] = __builtin_fmaf(u, cs[j], -(v * sn[j]));
+          x[2 * j + 1] = __builtin_fmaf(v, cs[j], u * sn[j]);
+        }
+    }
+    if (a.norm) {
+      float ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss += x[j] * x[j];
+      ss = group_sum<GW>(ss);
+      const float rs = 1.f / sqrtf(ss / static_cast<float>(a.dk) + a.eps);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] *= rs;
+    }
+    if (!live) return;
+    if (h < a.Hq) {
+      st8<T>(static_cast<T*>(a.q_out) + ((int64_t)t * a.Hq + h) * a.dkp + 8 * c, x);
+    } else {
+      const int kh = h - a.Hq;
+      if (a.k_out) st8<T>(static_cast<T*>(a.k_out) + ((int64_t)t * a.Hkv + kh) * a.dkp + 8 * c, x);
+      if (slot >= 0 && a.k_cache) {
+        const int64_t head = (page * a.Hkv + kh) * a.page_size;
+        T* dst = static_cast<T*>(a.k_cache);
+        if constexpr (kF32) dst += (head + off) * a.dkp + 8 * c;
+        else dst += (head + (off & ~15)) * a.dkp + (c * 16 + (off & 15)) * 8;
+        st8<T>(dst, x);
+      }
+    }
+  } else {
+    const int vi = it - rot_items;
+    const int kh = vi / vch, c = vi % vch;
+    float x[8];
+    load((a.Hq + a.Hkv) * a.dkp + kh * a.dvp + 8 * c, x);
+    const int64_t at = ((int64_t)t * a.Hkv + kh) * a.dvp + 8 * c;
+    if (a.v_first) {
+      float f[8];
+      ld8<T>(static_cast<const T*>(a.v_first) + at, f);
+      const float lam = *a.lam;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] = (1.f - lam) * x[j] + lam * f[j];
+    }
+    if (a.v_out) st8<T>(static_cast<T*>(a.v_out) + at, x);
+    if (slot >= 0 && a.v_cache) {
+      const int64_t head = (page * a.Hkv + kh) * a.page_size;
+      T* dst = static_cast<T*>(a.v_cache);
+      if constexpr (kF32) {
+        st8<T>(dst + (head + off) * a.dvp + 8 * c, x);
+      } else {
+        const int d0 = 8 * c, t16 = off & 15;
+        dst += (head + (off & ~15)) * a.dvp + (((d0 >> 5) * 4 + (t16 >> 2)) * 16 + (d0 & 15)) * 8 + ((d0 >> 4) & 1) * 4 + (t16 & 3);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) dst[8 * j] = f2bf(x[j]);
+      }
+    }
+  }
+}
+
+template <typename T>
+static int launch_qkv_heads(const QkvHeads& a, int tokens, hipStream_t stream) {
+  int gw = 1;
+  while (gw * 8 < a.dkp) gw *= 2;
+  const int items = (a.Hq + a.Hkv) * gw + a.Hkv * (a.dvp / 8);
+  const dim3 grid(tokens, (items + 255) / 256);
+  switch (gw) {
+    case 1: qkv_heads_kernel<T, 1><<<grid, 256, 0, stream>>>(a); break;
+    case 2: qkv_heads_kernel<T, 2><<<grid, 256, 0, stream>>>(a); break;
+    case 4: qkv_heads_kernel<T, 4><<<grid, 256, 0, stream>>>(a); break;
+    case 8: qkv_heads_kernel<T, 8><<<grid, 256, 0, stream>>>(a); break;
+    case 16: qkv_heads_kernel<T, 16><<<grid, 256, 0, stream>>>(a); break;
+    case 32: qkv_heads_kernel<T, 32><<<grid, 256, 0, stream>>>(a); break;
+    default: return -2;
+  }
+  OAMD_LAUNCH_CHECK();
+  return 0;
+}
+
+int qkv_heads(const QkvHeads& a, int tokens, bool f32, hipStream_t stream) {
+  if (tokens == 0) return 0;
+  if (a.dkp % 8 || a.dvp % 8 || a.dkp > 256 || a.Hkv < 1 || a.Hq < 1) return -1;
+  if (a.k_cache && !f32 && (a.dvp % 32 || a.page_size % 16)) return -1;
+  return f32 ? launch_qkv_heads<float>(a, tokens, stream) : launch_qkv_heads<bf16_t>(a, tokens, stream);
+}
+
+}  // namespace oamd

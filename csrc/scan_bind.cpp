@@ -1,9 +1,11 @@
-// Bindings for the log-scan kernels (operator_amd._C.ac_scan / scan_fixup).
+// Bindings of the log-scan and scoring kernels, and the module (operator_amd._S) that holds them
+// together with the collectives of comm_bind.cpp: a process that only serves a model needs neither.
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
 #include <ATen/hip/impl/HIPGuardImplMasqueradingAsCUDA.h>
 #include <ATen/hip/impl/HIPStreamMasqueradingAsCUDA.h>
 
+#include "kernels/kernels.h"
 #include "kernels/scan.h"
 
 namespace {
@@ -119,15 +121,52 @@ void context_spans(const at::Tensor& text, const at::Tensor& doc_base, const at:
   TORCH_CHECK(rc == 0, "context_spans launch failed rc=", rc);
 }
 
+void score_events(const at::Tensor& keys, const at::Tensor& hit_doc, const at::Tensor& doc_ptr,
+                  const at::Tensor& prim_ptr, const at::Tensor& prim_pat, const at::Tensor& ev_ptr,
+                  const at::Tensor& ev_doc_ptr, const at::Tensor& sec_ptr, const at::Tensor& sec_matcher,
+                  const at::Tensor& sec_w, const at::Tensor& sec_win, const at::Tensor& conf,
+                  const at::Tensor& severity, double significance, at::Tensor& ev_score, at::Tensor& ev_pat,
+                  at::Tensor& ev_line, at::Tensor& order, at::Tensor& summary) {
+  CHECK_T(keys, at::kLong);
+  for (auto* t : {&hit_doc, &doc_ptr, &prim_ptr, &prim_pat, &ev_ptr, &ev_doc_ptr, &sec_ptr, &sec_matcher, &sec_win,
+                  &severity}) {
+    CHECK_T(*t, at::kInt);
+  }
+  for (auto* t : {&sec_w, &conf}) CHECK_T(*t, at::kDouble);
+  CHECK_T(ev_score, at::kDouble);
+  for (auto* t : {&ev_pat, &ev_line, &order, &summary}) CHECK_T(*t, at::kInt);
+  const int64_t n_hits = keys.numel(), n_docs = doc_ptr.numel() - 1;
+  const int64_t n_pat = conf.numel(), n_m = prim_ptr.numel() - 1;
+  TORCH_CHECK(hit_doc.numel() == n_hits && ev_ptr.numel() == n_hits + 1 && ev_doc_ptr.numel() == n_docs + 1,
+              "score_events: hit index shapes");
+  TORCH_CHECK(sec_ptr.numel() == n_pat + 1 && severity.numel() == n_pat && sec_matcher.numel() == sec_w.numel() &&
+                  sec_w.numel() == sec_win.numel(), "score_events: pattern table shapes");
+  TORCH_CHECK(summary.numel() >= 3 * n_docs, "summary [docs, 3]");
+  const int64_t n_ev = ev_score.numel();
+  TORCH_CHECK(ev_pat.numel() == n_ev && ev_line.numel() == n_ev && order.numel() == n_ev, "event buffer shapes");
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(keys.device());
+  const int rc = oamd::score_events(keys.data_ptr<int64_t>(), hit_doc.data_ptr<int>(), doc_ptr.data_ptr<int>(), (int)n_hits, (int)n_docs,
+                        prim_ptr.data_ptr<int>(), prim_pat.data_ptr<int>(), ev_ptr.data_ptr<int>(), ev_doc_ptr.data_ptr<int>(),
+                        sec_ptr.data_ptr<int>(), sec_matcher.data_ptr<int>(), sec_w.data_ptr<double>(), sec_win.data_ptr<int>(),
+                        conf.data_ptr<double>(), severity.data_ptr<int>(), (int)n_m, significance, ev_score.data_ptr<double>(),
+                        ev_pat.data_ptr<int>(), ev_line.data_ptr<int>(), order.data_ptr<int>(), summary.data_ptr<int>(), c10::hip::getCurrentHIPStreamMasqueradingAsCUDA().stream());
+  TORCH_CHECK(rc == 0, "score_events launch failed rc=", rc);
+}
+
 }  // namespace
 
-void register_scan_bindings(pybind11::module_& m) {
+void register_comm_bindings(pybind11::module_& m);
+
+PYBIND11_MODULE(_S, m) {
+  m.doc() = "operator_amd gfx950 log-scan kernels and collectives";
   m.def("line_prefix", &line_prefix);
   m.def("doc_lines", &doc_lines);
   m.def("context_spans", &context_spans);
   m.def("line_prefix_state_words", [](int64_t n) { return (oamd::line_prefix_state_words(n) + 1) & ~1ll; });
   m.def("ac_scan", &ac_scan);
+  m.def("score_events", &score_events);
   m.def("scan_fixup", &scan_fixup);
   m.def("max_hot_states", [](int64_t log2c) { return oamd::max_hot_states((int)log2c); });
   m.attr("SCAN_HOT_STRIDE") = oamd::kScanHotStride;
+  register_comm_bindings(m);
 }

@@ -1,16 +1,18 @@
 """In-tree native build for operator_amd (no pip install, no JIT cache).
 
-Produces two shared objects next to this file:
+Produces three shared objects next to this file:
 
-* ``_C.*.so``        — the gfx950 HIP kernels (csrc/kernels/*.hip, compiled by
-  ``hipcc --offload-arch=gfx950``) + torch bindings (csrc/*.cpp, g++ against
+* ``_C.*.so``        — the gfx950 HIP kernels of the language models (csrc/kernels/*.hip,
+  compiled by ``hipcc --offload-arch=gfx950``) + torch bindings (csrc/*.cpp, g++ against
   the installed PyTorch-ROCm headers). Linked with an rpath to torch/lib first
   so the process has exactly one HIP runtime (torch's ``libamdhip64.so.7``).
+* ``_S.*.so``        — the same for the log scanner, the event scoring and the collectives;
+  built and loaded on its own, so serving a model does not wait for it.
 * ``_patterns.*.so`` — the CPU pattern compiler / log packer / scorer
   (csrc/patterns/*.cpp, pybind11, no HIP or torch dependency).
 
 Objects are cached under ``build/`` and rebuilt when a source or any header
-under csrc/ is newer. ``python -m operator_amd._build`` builds both.
+under csrc/ is newer. ``python -m operator_amd._build`` builds all.
 """
 from __future__ import annotations
 
@@ -30,6 +32,20 @@ PKG = ROOT / "operator_amd"
 ARCH = os.environ.get("OAMD_OFFLOAD_ARCH", "gfx950")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 CXX = os.environ.get("CXX", "g++")
+
+
+# the sources of _S; every other csrc/kernels/*.hip and csrc/*.cpp belongs to _C
+SERVICE_SOURCES = ("scan.hip", "score.hip", "line_index.hip", "allreduce.hip", "scan_bind.cpp", "comm_bind.cpp")
+# hipcc otherwise forms packed fp32 instructions from ordinary float code; their results are
+# not reliable on this hardware, so the feature is off for every kernel
+HIP_FLAGS = ["-O3", "-std=c++17", "-fPIC", "-munsafe-fp-atomics", "-Xclang", "-target-feature", "-Xclang",
+             "-packed-fp32-ops"]
+
+
+def module_sources(name: str) -> list[Path]:
+    """Sources of native module ``name`` (``_C`` or ``_S``)."""
+    srcs = sorted((CSRC / "kernels").glob("*.hip")) + sorted(CSRC.glob("*.cpp"))
+    return [s for s in srcs if (s.name in SERVICE_SOURCES) == (name == "_S")]
 
 
 def _ext_suffix() -> str:
@@ -89,43 +105,47 @@ def build_patterns(verbose: bool = False, force: bool = False, out_dir: Path | N
     return out
 
 
-def build_kernels(verbose: bool = False, force: bool = False, jobs: int | None = None) -> Path:
+def build_kernels(verbose: bool = False, force: bool = False, jobs: int | None = None,
+                  modules: tuple[str, ...] = ("_C", "_S")) -> list[Path]:
+    """Compile and link the named kernel modules (all objects in one parallel pool)."""
     inc, libdirs, abi, torch_lib = _torch_flags()
     BUILD.mkdir(parents=True, exist_ok=True)
     hdr = _newest_header_mtime()
-    hip_srcs = sorted((CSRC / "kernels").glob("*.hip"))
-    cpp_srcs = sorted(CSRC.glob("*.cpp"))
     jobs = jobs or min(16, os.cpu_count() or 4)
-    defs = [f"-D_GLIBCXX_USE_CXX11_ABI={abi}", "-DTORCH_EXTENSION_NAME=_C", "-DTORCH_API_INCLUDE_EXTENSION_H",
+    defs = [f"-D_GLIBCXX_USE_CXX11_ABI={abi}", "-DTORCH_API_INCLUDE_EXTENSION_H",
             "-D__HIP_PLATFORM_AMD__=1", "-DUSE_ROCM=1"]
     pyinc = f"-I{sysconfig.get_paths()['include']}"
 
-    tasks = []
-    objs = []
-    for s in hip_srcs:
-        o = BUILD / (s.stem + ".hip.o")
-        objs.append(o)
-        if force or _stale(o, s, hdr):
-            tasks.append([HIPCC, f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-c", str(s),
-                          f"-I{CSRC / 'kernels'}", "-munsafe-fp-atomics", "-o", str(o)])
-    for s in cpp_srcs:
-        o = BUILD / (s.stem + ".cpp.o")
-        objs.append(o)
-        if force or _stale(o, s, hdr):
-            tasks.append([CXX, "-O2", "-std=c++17", "-fPIC", "-c", str(s), f"-I{CSRC}", pyinc,
-                          *[f"-isystem{i}" for i in inc], *defs, "-Wno-deprecated-declarations", "-o", str(o)])
+    tasks, objs = [], {}
+    for name in modules:
+        objs[name] = []
+        for s in module_sources(name):
+            o = BUILD / (s.name + ".o")
+            objs[name].append(o)
+            if not force and not _stale(o, s, hdr):
+                continue
+            if s.suffix == ".hip":
+                tasks.append([HIPCC, f"--offload-arch={ARCH}", *HIP_FLAGS, "-c", str(s), f"-I{CSRC / 'kernels'}",
+                              "-o", str(o)])
+            else:
+                tasks.append([CXX, "-O2", "-std=c++17", "-fPIC", "-c", str(s), f"-I{CSRC}", pyinc,
+                              *[f"-isystem{i}" for i in inc], *defs, f"-DTORCH_EXTENSION_NAME={name}",
+                              "-Wno-deprecated-declarations", "-o", str(o)])
     if tasks:
         with cf.ThreadPoolExecutor(max_workers=jobs) as ex:
             list(ex.map(lambda c: _run(c, verbose), tasks))
-    out = PKG / f"_C{_ext_suffix()}"
-    if force or tasks or not out.exists() or any(out.stat().st_mtime < o.stat().st_mtime for o in objs):
-        link = [HIPCC, f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, objs), "-o", str(out),
-                f"-Wl,-rpath,{torch_lib}", f"-L{torch_lib}",
-                *[f"-L{d}" for d in libdirs if d != torch_lib],
-                "-lc10", "-lc10_hip", "-ltorch", "-ltorch_cpu", "-ltorch_hip", "-ltorch_python", "-lamdhip64"]
-        _run(link, verbose)
-        _check_stubs(out)
-    return out
+    outs = []
+    for name in modules:
+        out = PKG / f"{name}{_ext_suffix()}"
+        if force or not out.exists() or any(out.stat().st_mtime < o.stat().st_mtime for o in objs[name]):
+            link = [HIPCC, f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, objs[name]), "-o", str(out),
+                    f"-Wl,-rpath,{torch_lib}", f"-L{torch_lib}",
+                    *[f"-L{d}" for d in libdirs if d != torch_lib],
+                    "-lc10", "-lc10_hip", "-ltorch", "-ltorch_cpu", "-ltorch_hip", "-ltorch_python", "-lamdhip64"]
+            _run(link, verbose)
+            _check_stubs(out)
+        outs.append(out)
+    return outs
 
 
 def _check_stubs(so: Path) -> None:
@@ -145,7 +165,7 @@ def build(verbose: bool = False, force: bool = False) -> list[Path]:
     """Compile every native component for gfx950 (CPU-only host; hipcc cross-compiles)."""
     if shutil.which(HIPCC) is None and not os.path.exists(HIPCC):
         raise RuntimeError(f"hipcc not found at {HIPCC}")
-    return [build_patterns(verbose, force), build_kernels(verbose, force)]
+    return [build_patterns(verbose, force), *build_kernels(verbose, force)]
 
 
 if __name__ == "__main__":
