@@ -5,6 +5,7 @@
   scan           pattern-analyse log files -> AnalysisResult JSON
   explain        scan + explain log files with the local LLM -> AIResponse JSON
   serve-compat   REST server speaking the reference's log-parser / ai-interface contracts
+  replay         feed given token ids through a model step by step and write logits (bin/trace_run)
   bench          run bench.py (flagship benchmark)
 """
 from __future__ import annotations
@@ -304,6 +305,12 @@ def cmd_serve_compat(args) -> int:
     return 0
 
 
+def cmd_replay(args) -> int:
+    from operator_amd.engine.replay import replay
+
+    return replay(args.model, args.dtype, args.out, args.max_tokens, _settings(args))
+
+
 def cmd_bench(args, rest) -> int:
     import subprocess
 
@@ -359,6 +366,12 @@ def main(argv: list[str] | None = None) -> int:
     common(p)
     p.add_argument("--patterns", action="append")
     p.add_argument("--port", type=int, default=None)
+    p = sub.add_parser("replay", help="steps as JSON lines on stdin, logits as <step>.f32 files in --out")
+    common(p)
+    p.add_argument("--model", required=True, help="checkpoint directory (config.json, *.safetensors)")
+    p.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16")
+    p.add_argument("--out", required=True)
+    p.add_argument("--max-tokens", type=int, required=True, help="most tokens that live requests hold at once")
     sub.add_parser("bench", add_help=False)
     args, rest = ap.parse_known_args(argv)
     if args.cmd == "bench":
@@ -366,7 +379,7 @@ def main(argv: list[str] | None = None) -> int:
     if rest:
         ap.error(f"unrecognized arguments: {rest}")
     return {"run": cmd_run, "manifests": cmd_manifests, "scan": cmd_scan, "explain": cmd_explain,
-            "serve-compat": cmd_serve_compat}[args.cmd](args)
+            "serve-compat": cmd_serve_compat, "replay": cmd_replay}[args.cmd](args)
 
 
 if __name__ == "__main__":

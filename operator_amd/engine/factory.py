@@ -40,38 +40,38 @@ def calibrate_allreduce(tp, hidden: int, max_batch: int, iters: int = 20) -> dic
     return rep
 
 
-def build_llm(s: Settings, device: str | torch.device | None = None, tp=None):
-    """(model, kv, LLMEngine, Tokenizer) for the configured explanation model."""
+def build_engine(s: Settings, device: str | torch.device | None = None, tp=None, kv_pages: int | None = None):
+    """(model, kv, LLMEngine) for the configured model: the registry picks the class by the
+    checkpoint's config.json (or the preset). ``kv_pages`` overrides the cache budget."""
+    from dataclasses import replace
+
     from operator_amd.engine.llm import LLMEngine
-    from operator_amd.engine.tokenizer import Tokenizer, load_chat_template
-    from operator_amd.models.config import config_from_hf, get_config
-    from operator_amd.models.kv_cache import PagedKVCache
     from operator_amd.models import weight_cache
-    from operator_amd.models.llama import LlamaModel
+    from operator_amd.models.kv_cache import PagedKVCache
+    from operator_amd.models.registry import build_model, load_config
 
     e = s.engine
     dev = torch.device(device or e.device)
-    # a checkpoint's own config.json defines the architecture (llama / mistral / qwen2)
-    if e.model_path and os.path.exists(os.path.join(e.model_path, "config.json")):
-        cfg = config_from_hf(e.model_path, name=e.model)
-    else:
-        cfg = get_config(e.model)
+    cfg = load_config(e.model, e.model_path)
+    if cfg.arch == "sufolix" and cfg.max_position < e.max_context:
+        cfg = replace(cfg, max_position=e.max_context)   # a table length there, not a property of the model
     dtype = getattr(torch, e.dtype)
     if tp is not None and tp.world > 1 and dev.type == "cuda" and e.oneshot_allreduce_mb > 0 \
             and getattr(tp, "oneshot", None) is None:
         if tp.enable_oneshot(dev, int(e.oneshot_allreduce_mb * (1 << 20)), int(max(e.oneshot_max_kb, 0) * 1024) or None) \
                 and e.oneshot_max_kb <= 0:
             calibrate_allreduce(tp, cfg.hidden, e.max_batch, e.allreduce_calibrate_iters)
-    model = LlamaModel(cfg, device=dev, tp=tp, dtype=dtype, weight_dtype=e.weight_dtype)
+    model = build_model(cfg, device=dev, tp=tp, dtype=dtype, weight_dtype=e.weight_dtype)
     weight_cache.load_or_build(model, e.weight_cache_dir, e.model_path, e.seed)
     # KV cache: the compute dtype, or OCP fp8 (e4m3fn, per-tensor scales) with engine.kv_dtype=fp8
     if e.kv_dtype not in ("auto", "fp8"):
         raise ValueError(f"engine.kv_dtype must be auto or fp8, not {e.kv_dtype!r}")
+    if e.kv_dtype == "fp8" and cfg.arch == "sufolix":
+        raise ValueError("engine.kv_dtype=fp8: sufolix models keep keys and values in the compute dtype")
     kv_dtype = torch.float8_e4m3fn if e.kv_dtype == "fp8" else dtype
-    pages = PagedKVCache.pages_for_budget(int(e.kv_cache_gb * 1e9), cfg.layers, model.hkv, cfg.head_dim,
-                                          e.page_size, torch.finfo(kv_dtype).bits // 8)
-    kv = PagedKVCache(cfg.layers, pages, model.hkv, cfg.head_dim, e.page_size, device=dev, dtype=kv_dtype,
-                      k_scale=e.kv_scale, v_scale=e.kv_scale)
+    pages = kv_pages or PagedKVCache.pages_for_shapes(int(e.kv_cache_gb * 1e9), model.kv_shapes(), e.page_size,
+                                                      torch.finfo(kv_dtype).bits // 8)
+    kv = PagedKVCache.for_model(model, pages, e.page_size, dtype=kv_dtype, k_scale=e.kv_scale, v_scale=e.kv_scale)
     kw = dict(max_batch=e.max_batch, max_prefill_tokens=e.max_prefill_tokens, max_context=e.max_context,
               use_graphs=e.use_graphs, multi_step=e.multi_step, admit_wait_s=e.admit_wait_ms / 1e3,
               prefill_graphs=e.prefill_graphs, prefix_sharing=e.prefix_sharing)
@@ -81,11 +81,21 @@ def build_llm(s: Settings, device: str | torch.device | None = None, tp=None):
         llm = TPLLMEngine(model, kv, tp_group=tp, ctrl_group=control_group(tp), **kw)
     else:
         llm = LLMEngine(model, kv, **kw)
+    log.info("explanation model %s: %.1f GB weights, %d KV pages (%d tokens)", cfg.name,
+             model.weight_bytes() / 1e9, pages, pages * e.page_size)
+    return model, kv, llm
+
+
+def build_llm(s: Settings, device: str | torch.device | None = None, tp=None):
+    """(model, kv, LLMEngine, Tokenizer) for the configured explanation model."""
+    from operator_amd.engine.tokenizer import Tokenizer, load_chat_template
+
+    e = s.engine
+    model, kv, llm = build_engine(s, device, tp)
+    cfg = model.cfg
     tok = Tokenizer(cfg.vocab_size, cfg.bos_id, cfg.eos_ids[0],
                     path=(f"{e.model_path}/tokenizer.json" if e.model_path else None), add_bos=cfg.add_bos,
                     chat_template=load_chat_template(e.chat_template, e.model_path))
-    log.info("explanation model %s: %.1f GB weights, %d KV pages (%d tokens)", cfg.name,
-             model.weight_bytes() / 1e9, pages, pages * e.page_size)
     return model, kv, llm, tok
 
 

@@ -35,7 +35,7 @@ import torch
 
 from operator_amd import ops
 from operator_amd.models.kv_cache import PagedKVCache
-from operator_amd.models.llama import ForwardBatch, LlamaModel
+from operator_amd.models.base import DecoderModel, ForwardBatch
 from operator_amd.utils.tracing import trace_range
 
 
@@ -236,6 +236,7 @@ class _DecodeGraph:
     def __init__(self, eng: "LLMEngine", st: _BucketState, splits: int):
         self.eng, self.st, self.splits = eng, st, splits
         self.graph: torch.cuda.CUDAGraph | None = None
+        self.logits: torch.Tensor | None = None
 
     def _run(self) -> None:
         e, st = self.eng, self.st
@@ -251,8 +252,8 @@ class _DecodeGraph:
             spos = st.pos + 1
         fb = ForwardBatch(st.ids, st.pos, slots, False, None, block_tables=st.bt, context_lens=st.ctx,
                           num_splits=self.splits)
-        logits = e.model.forward(fb, e.kv)
-        tok = e.model.sample(logits, st.temp, st.seeds, spos)
+        self.logits = e.model.forward(fb, e.kv)   # [bp, vocab]: a replay overwrites them in place
+        tok = e.model.sample(self.logits, st.temp, st.seeds, spos)
         if gpu:
             ops.kernels().decode_advance(tok, st.ids, st.hist, st.pos, st.ctx, st.step)
         else:
@@ -429,7 +430,7 @@ class LLMEngine:
     PREFIX_MIN_SEEN = 2
     PREFIX_WINDOW = 64
 
-    def __init__(self, model: LlamaModel, kv: PagedKVCache, max_batch: int = 256, max_prefill_tokens: int = 16384,
+    def __init__(self, model: DecoderModel, kv: PagedKVCache, max_batch: int = 256, max_prefill_tokens: int = 16384,
                  max_context: int | None = None, use_graphs: bool = True, multi_step: int = 8,
                  admit_wait_s: float = 0.0, prefill_graphs: bool = True, prefix_sharing: bool = True):
         self.model, self.kv = model, kv
@@ -492,21 +493,22 @@ class LLMEngine:
         if self.device.type == "cuda":
             self._host_bufs = [torch.empty(max_batch, self.multi_step, dtype=torch.long, pin_memory=True)
                                for _ in range(2)]
-        # shared prompt prefix: the GPU path needs the v3 / v4 prefill attention kernel; TP
+        # shared prompt prefix: the prefill attention must take one (model.prefix_ok); TP
         # followers replay the leader's admissions, so every rank builds the same prefix at
         # the same step (tests/test_tp_scale.py::test_tp_prefix_sharing_matches_tp1)
-        self.prefix_sharing = prefix_sharing and (
-            self.device.type != "cuda" or ops.prefill_variant(model.hq, model.hkv) in (3, 4))
+        self.prefix_sharing = prefix_sharing and model.prefix_ok()
         self._pfx: _SharedPrefix | None = None
         self._pfx_seen: deque = deque()
         self._pfx_count: dict = {}
         self._pfx_last: list = []   # the page-aligned prefixes of the last admitted prompt
-        self._pk = self._pv = None
+        self._pk = self._pv = None   # per layer: the shared prefix's K / V rows [cap, kv heads, size]
+        self._pfx_cap = max(kv.page_size, self.PREFIX_MAX_TOKENS // kv.page_size * kv.page_size)
+        self._pfx_dtype = torch.bfloat16 if model.dtype == torch.bfloat16 else model.dtype
         if self.prefix_sharing:
-            n = max(kv.page_size, self.PREFIX_MAX_TOKENS // kv.page_size * kv.page_size)
-            shape = (model.cfg.layers, n, model.hkv, model.cfg.head_dim)
-            self._pk = torch.zeros(shape, dtype=torch.bfloat16, device=self.device)
-            self._pv = torch.zeros(shape, dtype=torch.bfloat16, device=self.device)
+            n = self._pfx_cap
+            new = lambda h, d: torch.zeros(n, h, d, dtype=self._pfx_dtype, device=self.device)  # noqa: E731
+            self._pk = [new(h, dk) for h, dk, _ in model.kv_shapes()]
+            self._pv = [new(h, dv) for h, _, dv in model.kv_shapes()]
 
     # ------------------------------------------------------------------ API
     def submit(self, req: GenRequest) -> GenRequest:
@@ -576,7 +578,7 @@ class LLMEngine:
         """Page-aligned prompt prefixes a request could share (longest last), each leaving
         at least one token of its own to prefill (its logits sample the first output)."""
         P = self.kv.page_size
-        k = min(self._pk.shape[1] // P, (len(prompt) - 1) // P)
+        k = min(self._pfx_cap // P, (len(prompt) - 1) // P)
         return [tuple(prompt[:j * P]) for j in range(1, k + 1)]
 
     def _note_prefix(self, prompt: list[int]) -> None:
@@ -584,7 +586,7 @@ class LLMEngine:
         for key in self._pfx_last:
             self._pfx_seen.append(key)
             self._pfx_count[key] = self._pfx_count.get(key, 0) + 1
-        while len(self._pfx_seen) > self.PREFIX_WINDOW * (self._pk.shape[1] // self.kv.page_size):
+        while len(self._pfx_seen) > self.PREFIX_WINDOW * (self._pfx_cap // self.kv.page_size):
             old = self._pfx_seen.popleft()
             c = self._pfx_count[old] - 1
             if c:
@@ -615,13 +617,13 @@ class LLMEngine:
         slots = torch.tensor([pages[j // P] * P + j % P for j in range(n)], dtype=torch.long, device=dev)
 
         def sink(i, k, v):
-            self._pk[i, :n].copy_(k.reshape(n, *self._pk.shape[2:]))
-            self._pv[i, :n].copy_(v.reshape(n, *self._pv.shape[2:]))
+            self._pk[i][:n].copy_(k.reshape(n, *self._pk[i].shape[1:]))
+            self._pv[i][:n].copy_(v.reshape(n, *self._pv[i].shape[1:]))
 
         work = None
         if dev.type == "cuda":
-            var = ops.prefill_variant(self.model.hq, self.model.hkv)
-            ws, wq = ops.prefill_work_list([n], ops.prefill_block_q(self.model.hq, self.model.hkv, var))
+            var, bq = self.model.prefill_plan()
+            ws, wq = ops.prefill_work_list([n], bq)
             work = (torch.tensor([0, n], dtype=torch.int32, device=dev), torch.tensor(ws, dtype=torch.int32, device=dev),
                     torch.tensor(wq, dtype=torch.int32, device=dev), var)
         fb = ForwardBatch(torch.tensor(best, dtype=torch.long, device=dev), torch.arange(n, device=dev), slots, True,
@@ -816,55 +818,68 @@ class LLMEngine:
         self.stats.prefill_tokens += pf.tokens
         self.stats.prefill_s += now - pf.t0
 
-    def _prefill_impl(self, batch: list[GenRequest]) -> _PendingPrefill:
-        t0 = time.perf_counter()
-        dev = self.device
-        # packed token ids / positions / cache slots built with numpy: this runs on the
-        # engine thread between prefill batches, while the GPU waits for it
+    def _pack_prefill(self, batch: list[GenRequest]) -> dict:
+        """Packed token ids / positions / cache slots of a prefill batch, built with numpy: this
+        runs on the engine thread between prefill batches, while the GPU waits for it."""
         P = self.kv.page_size
         # a request holding the shared prefix prefills only its own tokens (positions n..)
         skip = [r.prefix.n if r.prefix is not None else 0 for r in batch]
         full = [len(r.prompt) for r in batch]
         lens = [f - n for f, n in zip(full, skip)]
         ar = [np.arange(n, f, dtype=np.int64) for n, f in zip(skip, full)]
-        ids = np.concatenate([np.asarray(r.prompt[n:], dtype=np.int64) for r, n in zip(batch, skip)])
-        pos = np.concatenate(ar)
-        slots = np.concatenate([np.asarray(r.pages, dtype=np.int64)[a // P] * P + a % P for r, a in zip(batch, ar)])
         cu = np.zeros(len(lens) + 1, dtype=np.int64)
         cu[1:] = np.cumsum(lens)
-        pfx = skip if any(skip) else None
-        last = cu[1:] - 1
-        var = ops.prefill_variant(self.model.hq, self.model.hkv)
-        ws, wq = ops.prefill_work_list(lens, ops.prefill_block_q(self.model.hq, self.model.hkv, var))
+        var, bq = self.model.prefill_plan()
+        ws, wq = ops.prefill_work_list(lens, bq)
+        return dict(ids=np.concatenate([np.asarray(r.prompt[n:], dtype=np.int64) for r, n in zip(batch, skip)]),
+                    pos=np.concatenate(ar),
+                    slots=np.concatenate([np.asarray(r.pages, dtype=np.int64)[a // P] * P + a % P for r, a in zip(batch, ar)]),
+                    cu=cu, ws=ws, wq=wq, var=var, lens=lens, skip=skip, full=full)
+
+    def _to_device(self, x, dt=torch.long) -> torch.Tensor:
+        return torch.as_tensor(np.asarray(x)).to(dtype=dt).to(self.device, non_blocking=True)
+
+    def _eager_prefill(self, p: dict, last) -> torch.Tensor:
+        """Logits of rows ``last`` of a packed prefill batch, computed without a graph."""
+        t = self._to_device
+        work = (t(p["cu"], torch.int32), t(p["ws"], torch.int32), t(p["wq"], torch.int32), p["var"]) \
+            if self.device.type == "cuda" else None
+        pre = (self._pk, self._pv, t(p["skip"], torch.int32), p["skip"]) if any(p["skip"]) else None
+        fb = ForwardBatch(t(p["ids"]), t(p["pos"]), t(p["slots"]), True, t(last), seq_lens=p["lens"], prefill_work=work,
+                          prefix=pre)
+        return self.model.forward(fb, self.kv)
+
+    def _prefill_impl(self, batch: list[GenRequest]) -> _PendingPrefill:
+        t0 = time.perf_counter()
+        p = self._pack_prefill(batch)
+        last = p["cu"][1:] - 1
         temps = [r.temperature for r in batch]
         seeds = [r.seed for r in batch]
-        g = self._prefill_graph_for(len(ids), len(batch))
+        n = len(p["ids"])
+        g = self._prefill_graph_for(n, len(batch))
         if g is not None:
-            toks, ev = g.launch(ids, pos, slots, cu, ws, wq, last, temps, seeds, full, skip)
+            toks, ev = g.launch(p["ids"], p["pos"], p["slots"], p["cu"], p["ws"], p["wq"], last, temps, seeds, p["full"],
+                                p["skip"])
             self.stats.prefill_graph_replays += 1
-            self.stats.prefill_padded_tokens += g.T - len(ids)
+            self.stats.prefill_padded_tokens += g.T - n
         else:
             self.stats.prefill_eager += 1
-            t = lambda x, dt=torch.long: torch.as_tensor(np.asarray(x)).to(dtype=dt).to(dev, non_blocking=True)  # noqa: E731
-            work = (t(cu, torch.int32), t(ws, torch.int32), t(wq, torch.int32), var) if dev.type == "cuda" else None
-            pre = None if pfx is None else (self._pk, self._pv, t(pfx, torch.int32), pfx)
-            fb = ForwardBatch(t(ids), t(pos), t(slots), True, t(last), seq_lens=lens, prefill_work=work, prefix=pre)
-            logits = self.model.forward(fb, self.kv)
-            tk = self.model.sample(logits, t(temps, torch.float32), t(seeds), t(full))
-            if dev.type == "cuda":
+            t = self._to_device
+            logits = self._eager_prefill(p, last)
+            tk = self.model.sample(logits, t(temps, torch.float32), t(seeds), t(p["full"]))
+            if self.device.type == "cuda":
                 toks = torch.empty(len(batch), dtype=torch.long, pin_memory=True)
                 toks.copy_(tk, non_blocking=True)
                 ev = torch.cuda.Event()
                 ev.record()
             else:
                 toks, ev = tk.tolist(), None
-        return _PendingPrefill(batch, toks, ev, t0, len(ids))
+        return _PendingPrefill(batch, toks, ev, t0, n)
 
     def _prefill_graph(self, T: int) -> _PrefillGraph:
         g = self._prefill_g.get(T)
         if g is None:
-            var = ops.prefill_variant(self.model.hq, self.model.hkv)
-            g = _PrefillGraph(self, T, self.max_batch, var, ops.prefill_block_q(self.model.hq, self.model.hkv, var))
+            g = _PrefillGraph(self, T, self.max_batch, *self.model.prefill_plan())
             if self._prefill_pool is None:   # its own pool: prefill and decode graphs never share memory
                 self._prefill_pool = torch.cuda.graph_pool_handle()
             g.capture(self._prefill_pool)
@@ -902,12 +917,62 @@ class LLMEngine:
             self._graphs[(bp, splits)] = g
         return g
 
+    def _bucket(self, n: int) -> int:
+        return next(b for b in self.buckets if b >= n)
+
+    # ------------------------------------------------------------------ given tokens
+    # Requests whose tokens the caller supplies (trace replay, scoring): the same packing,
+    # prefill, decode graphs, page tables and cache as generation; only the token that joins a
+    # sequence comes from outside and the logits go out. Not mixed with submitted requests.
+    def _reserve(self, r: GenRequest) -> None:
+        """Pages for every token ``r`` holds."""
+        if r.length > self.max_context:
+            raise ValueError(f"request of {r.length} tokens exceeds max_context {self.max_context}")
+        need = self.kv.pages_needed(r.length) - len(r.pages)
+        if need > 0:
+            r.pages = r.pages + self.kv.allocator.alloc(need)
+
+    def given_start(self, prompts: list[list[int]], want: list[list[int]]) -> tuple[list[GenRequest], torch.Tensor | None]:
+        """Prefill new sequences as one batch: (requests, logits [wanted, vocab] of the places
+        ``want`` of each prompt, in order)."""
+        reqs = [GenRequest(list(p), max_tokens=0) for p in prompts]
+        for r in reqs:
+            self._reserve(r)
+        p = self._pack_prefill(reqs)
+        rows = [int(p["cu"][i]) + j for i, w in enumerate(want) for j in w]
+        logits = self._eager_prefill(p, rows or [0])
+        self.stats.prefill_tokens += len(p["ids"])
+        return reqs, logits if rows else None
+
+    def given_next(self, reqs: list[GenRequest], tokens: list[int]) -> torch.Tensor:
+        """One decode step of ``reqs`` with the given next tokens: logits [len(reqs), vocab]."""
+        out = torch.empty(len(reqs), self.model.cfg.vocab_size, dtype=torch.float32, device=self.device)
+        for r, t in zip(reqs, tokens):
+            r.output.append(int(t))
+            self._reserve(r)
+        order = sorted(range(len(reqs)), key=lambda i: -reqs[i].length)
+        for a in range(0, len(order), self.max_batch):
+            part = order[a:a + self.max_batch]
+            rows = [reqs[i] for i in part]
+            bp = self._bucket(len(rows))
+            g = self._graph(bp, ops.decode_splits(rows[0].length, bp, self.hkv))
+            g.st.load(rows, self.max_pages)
+            g.run(self.use_graphs)
+            out[torch.tensor(part, device=self.device)] = g.logits[:len(rows)].float()
+            self.stats.decode_tokens += len(rows)
+        self._active = None
+        return out
+
+    def given_end(self, r: GenRequest) -> None:
+        self._release(r)
+        r.done = True
+
     def _launch(self, ahead: int = 0) -> _Window:
         """Launch one window of up to ``multi_step`` decode steps for ``self.running``;
         ``ahead`` tokens per request are already in flight in an earlier window."""
         reqs = list(self.running)
         B = len(reqs)
-        bp = next(b for b in self.buckets if b >= B)
+        bp = self._bucket(B)
         k = max(1, min(self.multi_step, min(r.max_tokens - len(r.output) - ahead for r in reqs)))
         # decode-attention split count for the longest context reached in this window
         splits = ops.decode_splits(max(r.length for r in reqs) + ahead + k - 1, bp, self.hkv)

@@ -13,6 +13,10 @@ BASELINE.json names Llama-3-8B (TP=1) and Llama-3-70B (TP=8) as the configs.
 There are no checkpoints offline, so weights are random-initialised with the
 exact architecture, or loaded from a local HF safetensors directory whose
 ``config.json`` then defines the architecture (``config_from_hf``).
+
+  sufolix  Sufolix (``config_from_dir``): hyper-connected residual streams, attention layers
+           with their own head sizes, per-head q/k norm and value mixing, dense or
+           routed-expert feed-forwards; ``SufolixConfig``
 """
 from __future__ import annotations
 
@@ -101,10 +105,103 @@ PRESETS: dict[str, LlamaConfig] = {
 }
 
 
-def get_config(name: str, **overrides) -> LlamaConfig:
-    if name not in PRESETS:
-        raise KeyError(f"unknown model preset {name!r}; known: {sorted(PRESETS)}")
-    c = PRESETS[name]
+@dataclass(frozen=True)
+class AttentionSpec:
+    """One attention mixer: head counts and sizes, rotary positions on the first ``rot_dims``
+    dimensions, the score scale, and whether its values mix with the first mixing layer's."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot_base: float = 10000.0
+    rot_dims: int = 0
+    v_mix: bool = False
+
+
+@dataclass(frozen=True)
+class FeedForwardSpec:
+    """A SwiGLU feed-forward of ``ff`` features (experts == 0), or ``experts`` of them of which a
+    token uses ``top``, with a shared one of ``shared_ff`` features (0: none)."""
+    ff: int
+    experts: int = 0
+    top: int = 0
+    shared_ff: int = 0
+
+
+@dataclass(frozen=True)
+class DecoderLayerSpec:
+    mixer: AttentionSpec
+    mlp: FeedForwardSpec | None = None
+
+
+@dataclass(frozen=True)
+class SufolixConfig:
+    name: str = "sufolix"
+    vocab_size: int = 32000
+    hidden: int = 1024
+    streams: int = 4                 # parallel residual streams
+    embed_scale: float = 1.0
+    rms_eps: float = 1e-6
+    layer_specs: tuple[DecoderLayerSpec, ...] = ()
+    max_position: int = 32768        # rotary table length, not a limit of the design
+    bos_id: int = -1
+    eos_ids: tuple[int, ...] = (-1,)
+    arch: str = "sufolix"
+    add_bos: bool = False
+
+    @property
+    def layers(self) -> int:
+        return len(self.layer_specs)
+
+    def param_count(self) -> int:
+        h, s = self.hidden, self.streams
+        n = 2 * self.vocab_size * h + h
+        for sp in self.layer_specs:
+            a, m = sp.mixer, sp.mlp
+            qkv = (a.heads + a.kv_heads) * a.dim + a.kv_heads * a.vdim
+            n += qkv * (h + 1) + h * a.heads * a.vdim + h + s * (s + 2) + (1 if a.v_mix else 0)
+            if m is not None:
+                n += 3 * h * m.ff * max(1, m.experts) + h + s * (s + 2)
+                n += h * m.experts + (3 * h * m.shared_ff + h if m.shared_ff else 0)
+        return n
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
+        return sum(sp.mixer.kv_heads * (sp.mixer.dim + sp.mixer.vdim) for sp in self.layer_specs) * dtype_bytes
+
+    def to_dict(self) -> dict:
+        return asdict(self)
+
+
+def _sufolix(name: str, layers: int, mixer: AttentionSpec, dense: FeedForwardSpec, moe: FeedForwardSpec, **kw) -> SufolixConfig:
+    """Alternating dense / expert layers of one mixer."""
+    return SufolixConfig(name=name, layer_specs=tuple(DecoderLayerSpec(mixer, moe if i % 2 else dense)
+                                                      for i in range(layers)), **kw)
+
+
+DESIGN_PRESETS: dict[str, SufolixConfig] = {
+    "tiny-sufolix": _sufolix("tiny-sufolix", 4, AttentionSpec(6, 3, 40, 24, 0.2, 20000.0, 32, True),
+                             FeedForwardSpec(160), FeedForwardSpec(72, experts=5, top=2, shared_ff=96),
+                             vocab_size=1000, hidden=192, streams=3, embed_scale=8.0, bos_id=990, eos_ids=(991,)),
+    # Llama-3-8B's widths and heads: the same projections per layer, hyper-connected, every
+    # second feed-forward 8 experts of which 2 run (the active width stays near the dense one)
+    "sufolix-8b": _sufolix("sufolix-8b", 32, AttentionSpec(32, 8, 128, 128, 0.088388, 500000.0, 128, True),
+                           FeedForwardSpec(14336), FeedForwardSpec(4096, experts=8, top=2, shared_ff=4096),
+                           vocab_size=128256, hidden=4096, streams=4, bos_id=128000, eos_ids=(128001, 128009)),
+    # the width of a ~1B model with narrower values and a partial rotation
+    "sufolix-1b": _sufolix("sufolix-1b", 16, AttentionSpec(16, 4, 128, 96, 0.1, 100000.0, 64, True),
+                           FeedForwardSpec(8192), FeedForwardSpec(1024, experts=32, top=4, shared_ff=2048),
+                           vocab_size=32000, hidden=2048, streams=4, bos_id=1, eos_ids=(2,)),
+}
+
+
+def get_config(name: str, **overrides) -> "LlamaConfig | SufolixConfig":
+    if name in DESIGN_PRESETS:
+        c = DESIGN_PRESETS[name]
+    elif name in PRESETS:
+        c = PRESETS[name]
+    else:
+        raise KeyError(f"unknown model preset {name!r}; known: {sorted([*PRESETS, *DESIGN_PRESETS])}")
     return replace(c, **overrides) if overrides else c
 
 
@@ -159,3 +256,57 @@ def config_from_hf(path: str, name: str | None = None) -> LlamaConfig:
         bos_id=int(bos) if bos is not None else -1, eos_ids=eos or (-1,),
         qkv_bias=bool(hc.get("attention_bias", mt == "qwen2")),
         add_bos=mt != "qwen2" and bos is not None)
+
+
+def sufolix_from_dict(hc: dict, name: str = "sufolix") -> SufolixConfig:
+    """SufolixConfig from a checkpoint's config.json contents."""
+    specs = []
+    for i, lay in enumerate(hc["layers"]):
+        if lay["type"] != "attention":
+            raise ValueError(f"layer {i}: mixer type {lay['type']!r} not supported")
+        m, f = lay["mixer"], lay.get("mlp")
+        rot = m.get("rot") or {"base": 1.0, "dims": 0}
+        mixer = AttentionSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                              scale=float(m["scale"]), rot_base=float(rot["base"]), rot_dims=int(rot["dims"]),
+                              v_mix=bool(m.get("v_mix", False)))
+        if mixer.heads % mixer.kv_heads:
+            raise ValueError(f"layer {i}: {mixer.heads} query heads over {mixer.kv_heads} kv heads")
+        if max(mixer.dim, mixer.vdim) > 256:
+            raise ValueError(f"layer {i}: head sizes {mixer.dim}/{mixer.vdim}; the attention kernels go up to 256")
+        if mixer.rot_dims % 2 or mixer.rot_dims > mixer.dim:
+            raise ValueError(f"layer {i}: {mixer.rot_dims} rotated dimensions of {mixer.dim}")
+        mlp = None
+        if f is not None:
+            if f["kind"] == "dense":
+                mlp = FeedForwardSpec(int(f["ff"]))
+            elif f["kind"] == "moe":
+                mlp = FeedForwardSpec(int(f["expert"]["ff"]), experts=int(f["router"]["experts"]),
+                                      top=int(f["router"]["top"]), shared_ff=int((f.get("shared") or {}).get("ff", 0)))
+                if not 1 <= mlp.top <= mlp.experts <= 496:
+                    raise ValueError(f"layer {i}: top {mlp.top} of {mlp.experts} experts")
+            else:
+                raise ValueError(f"layer {i}: feed-forward kind {f['kind']!r} not supported")
+        specs.append(DecoderLayerSpec(mixer, mlp))
+    shapes = {(sp.mixer.kv_heads, sp.mixer.vdim) for sp in specs if sp.mixer.v_mix}
+    if len(shapes) > 1:
+        raise ValueError(f"value-mixing layers disagree on the value shape: {sorted(shapes)}")
+    streams = int(hc.get("streams", 1))
+    if not specs or not 1 <= streams <= 8:
+        raise ValueError(f"{len(specs)} layers, {streams} residual streams (1..8 supported)")
+    return SufolixConfig(name=name, vocab_size=int(hc["vocab"]), hidden=int(hc["width"]), streams=streams,
+                         embed_scale=float((hc.get("embedding") or {}).get("scale", 1.0)),
+                         rms_eps=float(hc["norm"]["eps"]), layer_specs=tuple(specs))
+
+
+def config_from_dir(path: str, name: str | None = None) -> "LlamaConfig | SufolixConfig":
+    """The configuration a checkpoint directory's config.json describes, whichever of the
+    supported architectures it is (``architecture``: a design of its own; ``model_type``: a
+    HuggingFace Llama-architecture checkpoint)."""
+    with open(os.path.join(path, "config.json")) as f:
+        hc = json.load(f)
+    arch = hc.get("architecture")
+    if arch is None:
+        return config_from_hf(path, name)
+    if str(arch).lower() != "sufolix":
+        raise ValueError(f"{path}: architecture {arch!r} not supported")
+    return sufolix_from_dict(hc, name or os.path.basename(os.path.normpath(path)))

@@ -14,6 +14,10 @@ O(pages) per request; block tables are uploaded as int32 rows.
 so twice the tokens per GB and half the HBM traffic of decode attention, at
 fp8 precision for the cached keys and values (queries and all compute stay
 bf16 / fp32). Not the default.
+
+``shapes`` gives every layer its own (kv heads, key size, value size): one K and one V
+tensor per layer instead of the two stacked ones. How a layer arranges a page's bytes is its
+kernels' business (attn_decode.hip's K tiles, qkv_heads.hip's K / V tiles).
 """
 from __future__ import annotations
 
@@ -50,7 +54,7 @@ class PageAllocator:
 class PagedKVCache:
     def __init__(self, layers: int, num_pages: int, kv_heads: int, head_dim: int, page_size: int = 64,
                  device: str | torch.device = "cuda", dtype: torch.dtype = torch.bfloat16,
-                 k_scale: float = 1.0, v_scale: float = 1.0):
+                 k_scale: float = 1.0, v_scale: float = 1.0, shapes: list[tuple[int, int, int]] | None = None):
         if page_size & (page_size - 1):
             raise ValueError("page_size must be a power of two")
         if k_scale <= 0 or v_scale <= 0:
@@ -58,10 +62,30 @@ class PagedKVCache:
         self.dtype, self.k_scale, self.v_scale = dtype, float(k_scale), float(v_scale)
         self.layers, self.num_pages, self.kv_heads, self.head_dim, self.page_size = (
             layers, num_pages, kv_heads, head_dim, page_size)
-        shape = (layers, num_pages, kv_heads, page_size, head_dim)
-        self.k = torch.zeros(shape, dtype=dtype, device=device)
-        self.v = torch.zeros(shape, dtype=dtype, device=device)
+        if shapes is None:
+            shape = (layers, num_pages, kv_heads, page_size, head_dim)
+            self.k = torch.zeros(shape, dtype=dtype, device=device)
+            self.v = torch.zeros(shape, dtype=dtype, device=device)
+        else:
+            new = lambda h, d: torch.zeros(num_pages, h, page_size, d, dtype=dtype, device=device)  # noqa: E731
+            self.k = [new(h, dk) for h, dk, _ in shapes]
+            self.v = [new(h, dv) for h, _, dv in shapes]
         self.allocator = PageAllocator(num_pages)
+
+    @classmethod
+    def for_model(cls, model, num_pages: int, page_size: int = 64, dtype: torch.dtype | None = None, k_scale: float = 1.0,
+                  v_scale: float = 1.0) -> "PagedKVCache":
+        """The cache ``model`` needs (its ``kv_shapes``), in its compute dtype unless given."""
+        shapes = model.kv_shapes()
+        h, dk, dv = shapes[0]
+        alike = dk == dv and all(s == shapes[0] for s in shapes)
+        return cls(len(shapes), num_pages, h, dk, page_size, device=model.device, dtype=dtype or model.dtype,
+                   k_scale=k_scale, v_scale=v_scale, shapes=None if alike else shapes)
+
+    @staticmethod
+    def pages_for_shapes(budget_bytes: int, shapes: list[tuple[int, int, int]], page_size: int, dtype_bytes: int = 2) -> int:
+        per_page = sum(h * (dk + dv) for h, dk, dv in shapes) * page_size * dtype_bytes
+        return max(1, int(budget_bytes // per_page))
 
     @staticmethod
     def pages_for_budget(budget_bytes: int, layers: int, kv_heads: int, head_dim: int, page_size: int,

@@ -26,11 +26,9 @@ everything else is a hand-written HIP kernel too (operator_amd.ops).
 """
 from __future__ import annotations
 
-import hashlib
-import json
 import math
 import os
-from dataclasses import dataclass, field
+from dataclasses import dataclass
 
 import torch
 
@@ -38,29 +36,9 @@ from operator_amd import ops
 from operator_amd.ops import reference as ref
 from operator_amd.parallel.comm import Group
 
+from .base import DecoderModel, ForwardBatch
 from .config import LlamaConfig
 from .kv_cache import PagedKVCache
-
-
-@dataclass
-class ForwardBatch:
-    """Flattened tokens of one engine step (prefill or decode, never mixed)."""
-    input_ids: torch.Tensor            # [T] int64
-    positions: torch.Tensor            # [T] int64
-    slots: torch.Tensor                # [T] int64 (cache slot, -1 = do not write)
-    is_prefill: bool
-    logits_index: torch.Tensor | None  # [n_out] int64 rows to produce logits for (None = all)
-    # prefill
-    seq_lens: list[int] = field(default_factory=list)
-    prefill_work: tuple | None = None
-    # shared prompt prefix (LLMEngine prefix sharing): (pk, pv, seq_pfx, pfx_lens), pk / pv the
-    # cached post-RoPE K/V [layers, P, Hkv, D]; sequence s's tokens follow pfx_lens[s] of them
-    prefix: tuple | None = None
-    kv_sink: object = None   # called (layer, k, v) with each prefill layer's K/V (prefix capture)
-    # decode
-    block_tables: torch.Tensor | None = None   # [B, max_pages] int32
-    context_lens: torch.Tensor | None = None   # [B] int32 (including the new token)
-    num_splits: int = 1
 
 
 @dataclass
@@ -79,11 +57,10 @@ class LayerWeights:
     bqkv: torch.Tensor | None = None   # q|k|v projection bias (Qwen2), bf16 [(hq + 2 hkv) D]
 
 
-def _seed_for(seed: int, name: str) -> int:
-    return int.from_bytes(hashlib.sha256(f"{seed}:{name}".encode()).digest()[:8], "little") & ((1 << 63) - 1)
+class LlamaModel(DecoderModel):
+    LAYER = LayerWeights
+    LAYOUT_FUNCS = ("init_random", "_randn", "_quantize_layer", "_shard_layer", "split_gate_up", "load_hf")
 
-
-class LlamaModel:
     def __init__(self, cfg: LlamaConfig, device: str | torch.device = "cuda", tp: Group | None = None,
                  dtype: torch.dtype = torch.bfloat16, weight_dtype: str = "bfloat16"):
         self.cfg = cfg
@@ -112,12 +89,6 @@ class LlamaModel:
         self.embed = self.final_norm = self.lm_head = None
 
     # ------------------------------------------------------------------ weights
-    def _randn(self, seed: int, name: str, shape, std: float) -> torch.Tensor:
-        g = torch.Generator(device=self.device)
-        g.manual_seed(_seed_for(seed, name))
-        t = torch.randn(shape, generator=g, device=self.device, dtype=self.dtype)
-        return t.mul_(std)
-
     def init_random(self, seed: int = 0) -> "LlamaModel":
         """Random weights of the exact architecture. Each full tensor is generated from a
         name-derived seed and then sharded, so every TP degree sees the same global model."""
@@ -230,12 +201,20 @@ class LlamaModel:
         self.lm_head = lm[r * self.vocab_local:(r + 1) * self.vocab_local].contiguous()
         return self
 
-    def weight_bytes(self) -> int:
-        n = sum(t.numel() * t.element_size() for t in (self.embed, self.final_norm, self.lm_head))
-        for lw in self.layers:
-            n += sum(t.numel() * t.element_size() for t in (lw.wqkv, lw.wo, lw.wgu, lw.wd, lw.attn_norm, lw.mlp_norm,
-                                                            lw.sqkv, lw.so, lw.sgu, lw.sd, lw.bqkv) if t is not None)
-        return n
+    def load_checkpoint(self, path: str) -> "LlamaModel":
+        return self.load_hf(path)
+
+    # ------------------------------------------------------------------ engine surface
+    def kv_shapes(self) -> list[tuple[int, int, int]]:
+        return [(self.hkv, self.cfg.head_dim, self.cfg.head_dim)] * self.cfg.layers
+
+    def prefill_plan(self) -> tuple[int, int]:
+        var = ops.prefill_variant(self.hq, self.hkv)
+        return var, ops.prefill_block_q(self.hq, self.hkv, var)
+
+    def prefix_ok(self) -> bool:
+        """The grouped GPU kernels (v3, v4) take a prefix; the CPU reference always does."""
+        return self.device.type != "cuda" or ops.prefill_variant(self.hq, self.hkv) in (3, 4)
 
     # ------------------------------------------------------------------ forward
     def forward(self, fb: ForwardBatch, kv: PagedKVCache) -> torch.Tensor:
@@ -287,19 +266,3 @@ class LlamaModel:
         if fb.logits_index is not None:
             x = x.index_select(0, fb.logits_index)
         return ops.linear(x, self.lm_head)
-
-    def sample(self, logits: torch.Tensor, temperature: torch.Tensor, seeds: torch.Tensor,
-               positions: torch.Tensor) -> torch.Tensor:
-        """Sample one token per row; under TP each rank samples its vocab shard and the
-        global winner is the max perturbed value (ties -> smaller token id)."""
-        if self.tp.world == 1:
-            return ops.sample(logits, temperature, seeds, positions)
-        n = logits.shape[0]
-        val = torch.empty(n, dtype=torch.float32, device=logits.device)
-        tok = ops.sample(logits, temperature, seeds, positions, col_offset=self.vocab_offset, out_val=val)
-        pair = torch.stack([val, tok.to(torch.float32)], 1)             # exact for ids < 2^24
-        allp = self.tp.all_gather_into(pair)                             # [W, n, 2]
-        vals, toks = allp[..., 0], allp[..., 1]
-        best = vals.max(0).values
-        cand = torch.where(vals == best.unsqueeze(0), toks, torch.full_like(toks, float("inf")))
-        return cand.min(0).values.to(torch.long)

@@ -28,7 +28,11 @@ import torch
 log = logging.getLogger(__name__)
 
 FORMAT = 1
-LAYER_FIELDS = ("wqkv", "wo", "wgu", "wd", "attn_norm", "mlp_norm", "sqkv", "so", "sgu", "sd", "bqkv")
+
+
+def layer_fields(model) -> tuple[str, ...]:
+    """Tensor fields of one layer of ``model`` (None where a layer does not have one)."""
+    return tuple(f.name for f in dataclasses.fields(model.LAYER))
 
 
 def source_id(model_path: str | None, seed: int) -> str:
@@ -46,8 +50,8 @@ def source_id(model_path: str | None, seed: int) -> str:
 
 # the code that lays a shard out: TP slicing, QKV packing, gate|up interleave, fp8 scale
 # rounding, the random init. Its source text is part of the key, so an edit to any of it
-# misses every cache file written before the edit instead of mapping a stale layout back.
-LAYOUT_FUNCS = ("init_random", "_randn", "_quantize_layer", "_shard_layer", "split_gate_up", "load_hf")
+# misses every cache file written before the edit instead of mapping a stale layout back
+# (each model class names its own: ``LAYOUT_FUNCS``).
 
 
 def layout_version(model_cls=None) -> str:
@@ -57,7 +61,7 @@ def layout_version(model_cls=None) -> str:
 
     if model_cls is None:
         from .llama import LlamaModel as model_cls
-    src = "".join(inspect.getsource(getattr(model_cls, f)) for f in LAYOUT_FUNCS)
+    src = "".join(inspect.getsource(getattr(model_cls, f)) for f in model_cls.LAYOUT_FUNCS)
     src += inspect.getsource(ops.interleave_gate_up) + inspect.getsource(ops.quantize_fp8)
     return hashlib.sha256(src.encode()).hexdigest()[:16]
 
@@ -76,7 +80,7 @@ def save(model, path: str) -> None:
 
     t = {"embed": model.embed, "final_norm": model.final_norm, "lm_head": model.lm_head}
     for i, lw in enumerate(model.layers):
-        for f in LAYER_FIELDS:
+        for f in layer_fields(model):
             v = getattr(lw, f)
             if v is not None:
                 t[f"l{i}.{f}"] = v
@@ -92,8 +96,6 @@ def load(model, path: str) -> None:
     """Fill ``model``'s weights from a cache file written by ``save`` for the same key."""
     from safetensors import safe_open
 
-    from .llama import LayerWeights
-
     dev = str(model.device)
     with safe_open(path, framework="pt", device=dev) as f:
         n = int(f.metadata()["layers"])
@@ -103,8 +105,9 @@ def load(model, path: str) -> None:
         model.lm_head = f.get_tensor("lm_head")
         layers = []
         for i in range(n):
-            kw = {fld: (f.get_tensor(f"l{i}.{fld}") if f"l{i}.{fld}" in names else None) for fld in LAYER_FIELDS}
-            layers.append(LayerWeights(**kw))
+            kw = {fld: (f.get_tensor(f"l{i}.{fld}") if f"l{i}.{fld}" in names else None)
+                  for fld in layer_fields(model)}
+            layers.append(model.LAYER(**kw))
         model.layers = layers
     if model.device.type == "cuda":
         torch.cuda.synchronize(model.device)
@@ -113,7 +116,7 @@ def load(model, path: str) -> None:
 def load_or_build(model, cache_dir: str | None, model_path: str | None, seed: int) -> str:
     """Weights from the cache when a file for this exact shard exists, else built (HF
     load or random init) and written to the cache. Returns 'hit', 'miss' or 'off'."""
-    build = (lambda: model.load_hf(model_path)) if model_path else (lambda: model.init_random(seed))
+    build = (lambda: model.load_checkpoint(model_path)) if model_path else (lambda: model.init_random(seed))
     if not cache_dir:
         build()
         return "off"

@@ -20,6 +20,7 @@ __all__ = [
     "kernels", "patterns", "native_available", "reference", "prefill_work_list", "prefill_block_q", "prefill_variant", "decode_splits",
     "decode_workspace", "linear", "gemm_splits", "gemm_plan", "gate_up_silu", "interleave_gate_up",
     "quantize_fp8", "silu_quantize_fp8", "linear_fp8", "fp8_plan", "SplitK", "linear_tile", "tile_ok", "BLAS_CALLS",
+    "linear_f32", "decoder",
 ]
 
 # never split a sequence into pieces shorter than this / split only while B x Hkv
@@ -100,6 +101,8 @@ def gate_up_silu(x: torch.Tensor, wgu: torch.Tensor, block: int | None) -> torch
     other shapes run the GEMM then the silu_mul kernel."""
     M, K = x.shape
     N = wgu.shape[0]
+    if x.is_cuda and block == 64 and f32_ok(x, wgu):
+        return linear_f32(x, wgu, silu_gu=True)
     if (x.is_cuda and block == 64 and x.dtype == torch.bfloat16 and M <= SKINNY_MAX_M and N % 128 == 0
             and K % 128 == 0 and x.is_contiguous() and wgu.is_contiguous()
             and skinny_plan(M, N, K) is not None and _gemm_table_get().get(("silu", M, N, K)) != "blas"):
@@ -412,6 +415,20 @@ def linear_tile(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = Non
     return y
 
 
+def f32_ok(x: torch.Tensor, w: torch.Tensor) -> bool:
+    """Shapes the fp32 GEMM (gemm_f32) takes."""
+    return (x.dtype == torch.float32 and w.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous()
+            and w.is_contiguous() and x.shape[1] % 16 == 0)
+
+
+def linear_f32(x: torch.Tensor, w: torch.Tensor, silu_gu: bool = False) -> torch.Tensor:
+    """True 32-bit x @ w^T (fp32 FMA), optionally with the SwiGLU epilogue over a 64-row
+    interleaved gate|up weight."""
+    y = torch.empty(x.shape[0], w.shape[0] // 2 if silu_gu else w.shape[0], dtype=x.dtype, device=x.device)
+    kernels().gemm_f32(x, w, y, silu_gu)
+    return y
+
+
 def linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, splits: int | None = None,
            partial: torch.Tensor | None = None, bn: int | None = None, bm: int | None = None,
            defer_reduce: bool = False, stages: int | None = None, bias: torch.Tensor | None = None):
@@ -424,6 +441,8 @@ def linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, sp
     M, K = x.shape
     N = w.shape[0]
     plan = None
+    if x.is_cuda and bias is None and out is None and f32_ok(x, w):
+        return linear_f32(x, w)
     if bias is not None:
         if tile_ok(x, w) and tile_out_ok(out):
             return linear_tile(x, w, out, bias)
@@ -666,3 +685,6 @@ def sample(logits: torch.Tensor, temperature: torch.Tensor, seeds: torch.Tensor,
     o = out if out is not None else torch.empty(logits.shape[0], dtype=torch.long, device=logits.device)
     kernels().sample(logits, temperature, seeds, positions, o, col_offset, out_val)
     return o
+
+
+from . import decoder  # noqa: E402 - uses SplitK and prefill_work_list above

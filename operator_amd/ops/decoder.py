@@ -1,0 +1,280 @@
+"""Ops of decoders beyond the Llama block: hyper-connection residual streams, QKV heads of any
+size with rotary positions and per-head norm, attention over them, routed experts, and the
+fp32 forms of all of them.
+
+As in :mod:`operator_amd.ops`: GPU tensors go to the gfx950 kernels (csrc/kernels/streams.hip,
+qkv_heads.hip, attn_gd_*.hip, moe.hip, f32.hip), CPU tensors to the fp32 references. Widths,
+head sizes and feature counts are stored padded (``pad_to``) with zero weights, so every GEMM
+meets the tile kernels' alignment whatever the model's sizes.
+"""
+from __future__ import annotations
+
+from dataclasses import dataclass
+
+import torch
+
+from . import reference
+from ._native import kernels
+
+# general attention work items: 128 query rows whatever the head layout (attn_gd_prefill.hip)
+GD_VARIANT = 5
+GD_BLOCK_Q = 128
+# expert GEMMs: rows per expert from which the 256-row tile kernel beats the weight-streaming one
+MOE_TILE_MIN_ROWS = 64
+MOE_SKINNY_MAX_SLOTS = 4096   # moe.hip kMaxSlots
+
+
+def pad_to(n: int, m: int) -> int:
+    return -(-n // m) * m
+
+
+def head_pads(dim: int, vdim: int) -> tuple[int, int]:
+    """Stored sizes of a query/key head and a value head (the cache tiles' granularity)."""
+    return pad_to(dim, 16), pad_to(vdim, 32)
+
+
+# ---------------------------------------------------------------- hyper-connection streams
+@dataclass
+class Stream:
+    """Coefficients of one sublayer of a hyper-connected model (fp32): how it reads the S
+    residual streams (``inp`` [S]), how they mix ([S, S], [from, to]) and take its output (``out`` [S])."""
+    inp: torch.Tensor
+    mix: torch.Tensor
+    out: torch.Tensor
+
+
+@dataclass
+class SublayerOut:
+    """A sublayer's output as its producers left it, summed by the next stream step:
+    sigmoid(gate) * y + sum_k e[row of (token, k)]; every part may be absent."""
+    y: object = None                     # [T, ld] rows, or SplitK slabs
+    gate: torch.Tensor | None = None     # [T] fp32 logits
+    e: torch.Tensor | None = None        # [rows, ld]
+    epos: torch.Tensor | None = None     # [T, top] int32 row of e; None: row t * top + k
+    top: int = 0
+
+
+def stream_init(ids: torch.Tensor, table: torch.Tensor, scale: float, streams: int, width: int, inp: torch.Tensor,
+                w: torch.Tensor, eps: float):
+    """Embedding -> (streams [T, S, ld] fp32, all equal to scale * row; the first sublayer's
+    normalised input [T, ld] in the table's dtype)."""
+    T, ld = ids.numel(), table.shape[1]
+    x = torch.empty(T, streams, ld, dtype=torch.float32, device=ids.device)
+    h = torch.empty(T, ld, dtype=table.dtype, device=ids.device)
+    if ids.is_cuda:
+        kernels().stream_step(x, h, width, w, eps, in_=inp, ids=ids, table=table, emb_scale=scale)
+    else:
+        x.copy_((reference.embedding(ids, table).float() * scale)[:, None])
+        h.copy_(reference.stream_norm(x, inp, w, width, eps))
+    return x, h
+
+
+def stream_step(x: torch.Tensor, o: SublayerOut, hc: Stream, nxt: torch.Tensor | None, w: torch.Tensor, width: int,
+                eps: float, dtype: torch.dtype, rows: torch.Tensor | None = None, write_x: bool = True) -> torch.Tensor:
+    """Finish a sublayer (``hc`` with its output ``o``) and return the next one's normalised
+    input: ``nxt`` are its stream coefficients, None the plain sum at the model's end, where
+    ``rows`` picks the rows wanted and ``write_x`` False leaves the streams alone."""
+    from . import SplitK
+
+    n = x.shape[0] if rows is None else rows.numel()
+    if not x.is_cuda:
+        y = reference.sublayer_out(o.y, o.gate, o.e, o.epos, o.top, x.shape[0], x.shape[2])
+        xn = reference.stream_mix(x, y, hc.mix, hc.out)
+        if write_x:
+            x.copy_(xn)
+        if rows is not None:
+            xn = xn[rows]
+        return reference.stream_norm(xn, nxt, w, width, eps).to(dtype)
+    h = torch.empty(n, x.shape[2], dtype=dtype, device=x.device)
+    slab = isinstance(o.y, SplitK)
+    kernels().stream_step(x, h, width, w, eps, in_=nxt, y=None if slab else o.y, slabs=o.y.p if slab else None,
+                          splits=o.y.S if slab else 1, gate=o.gate, e=o.e, epos=o.epos, top=o.top, mix=hc.mix,
+                          out=hc.out, rows=rows, write_x=write_x)
+    return h
+
+
+# ---------------------------------------------------------------- attention, any head size
+@dataclass(frozen=True)
+class HeadLayout:
+    """Shapes and constants of one attention layer (true sizes; the rows hold padded ones)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    rot_dims: int = 0
+    norm: bool = True      # q, k divided by their root mean square after rotation
+    eps: float = 1e-6
+
+    @property
+    def pads(self) -> tuple[int, int]:
+        return head_pads(self.dim, self.vdim)
+
+    @property
+    def ncol(self) -> int:
+        """Columns of the packed QKV projection."""
+        dk, dv = self.pads
+        return pad_to((self.heads + self.kv_heads) * dk + self.kv_heads * dv, 64)
+
+    @property
+    def ocol(self) -> int:
+        """Columns of the attention output the o-projection reads."""
+        return pad_to(self.heads * self.pads[1], 64)
+
+
+def rotary_tables(max_pos: int, base: float, dims: int, device=None) -> tuple[torch.Tensor, torch.Tensor]:
+    """cos / sin [max_pos, dims / 2 padded to 4] of position * base^(-2 i / dims), fp32 from fp64 angles."""
+    n = dims // 2
+    inv = 1.0 / (base ** (torch.arange(n, dtype=torch.float64) * 2.0 / dims))
+    a = torch.zeros(max_pos, pad_to(max(n, 1), 4), dtype=torch.float64)
+    a[:, :n] = torch.outer(torch.arange(max_pos, dtype=torch.float64), inv)
+    return a.cos().float().to(device), a.sin().float().to(device)
+
+
+def qkv_heads(qkv, pos: torch.Tensor, rot: tuple | None, L: HeadLayout, dtype: torch.dtype, bias: torch.Tensor | None = None,
+              cache: tuple | None = None, slots: torch.Tensor | None = None, want_k: bool = True, want_v: bool = True,
+              v_first: torch.Tensor | None = None, lam: torch.Tensor | None = None):
+    """Packed projection rows (or SplitK slabs) -> (q [T, H, dk], k [T, G, dk] | None,
+    v [T, G, dv] | None) rotated, normalised and mixed with ``v_first``, k / v also written to
+    the paged ``cache`` at ``slots`` (< 0: not cached)."""
+    from . import SplitK
+
+    T, dev = pos.numel(), pos.device
+    dk, dv = L.pads
+    cos, sin = rot if rot is not None else (None, None)
+    if not pos.is_cuda:
+        q, k, v = reference.qkv_heads(qkv, bias, pos, cos, sin, L, v_first, lam)
+        q, k, v = q.to(dtype), k.to(dtype), v.to(dtype)
+        if cache is not None:
+            reference.cache_rows(cache[0], cache[1], k, v, slots)
+        return q, k if want_k else None, v if want_v else None
+    q = torch.empty(T, L.heads, dk, dtype=dtype, device=dev)
+    k = torch.empty(T, L.kv_heads, dk, dtype=dtype, device=dev) if want_k else None
+    v = torch.empty(T, L.kv_heads, dv, dtype=dtype, device=dev) if want_v else None
+    slab = isinstance(qkv, SplitK)
+    kc, vc = cache if cache is not None else (None, None)
+    kernels().qkv_heads(q if slab else qkv, qkv.p if slab else None, qkv.S if slab else 1, bias, pos, cos, sin,
+                        L.rot_dims // 2 if rot is not None else 0, L.heads, L.kv_heads, L.dim, L.norm, L.eps, v_first,
+                        lam, q, k, v, kc, vc, slots, dv, L.ncol)
+    return q, k, v
+
+
+def _o_rows(T: int, L: HeadLayout, dtype, dev) -> torch.Tensor:
+    o = torch.empty(T, L.ocol, dtype=dtype, device=dev)
+    used = L.heads * L.pads[1]
+    if used < L.ocol:
+        o[:, used:].zero_()
+    return o
+
+
+def attn_gd_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, seq_lens: list[int], L: HeadLayout, scale: float,
+                    work: tuple | None = None, prefix: tuple | None = None) -> torch.Tensor:
+    """Causal attention over packed sequences -> [T, ocol] rows for the o-projection.
+    ``work`` = (cu_seqlens, work_seq, work_q0, GD_VARIANT); ``prefix`` as in ``attn_prefill``."""
+    if not q.is_cuda:
+        cu = [0]
+        for n in seq_lens:
+            cu.append(cu[-1] + int(n))
+        r = reference.attn_prefill(q, k, v, cu, scale, prefix=None if prefix is None else (prefix[0], prefix[1], prefix[3]))
+        o = torch.zeros(q.shape[0], L.ocol, dtype=q.dtype)
+        o[:, :L.heads * L.pads[1]] = r.reshape(q.shape[0], -1)
+        return o
+    if work is None:
+        from . import prefill_work_list
+
+        cu = [0]
+        for n in seq_lens:
+            cu.append(cu[-1] + int(n))
+        ws, wq = prefill_work_list([int(n) for n in seq_lens], GD_BLOCK_Q)
+        work = tuple(torch.tensor(t, dtype=torch.int32, device=q.device) for t in (cu, ws, wq)) + (GD_VARIANT,)
+    if work[3] != GD_VARIANT:
+        raise ValueError("attn_gd_prefill needs a work list cut at GD_BLOCK_Q rows")
+    o = _o_rows(q.shape[0], L, q.dtype, q.device)
+    pk, pv, sp = (None, None, None) if prefix is None else prefix[:3]
+    kernels().attn_gd_prefill(q, k, v, o, work[0], work[1], work[2], scale, pk, pv, sp)
+    return o
+
+
+def attn_gd_workspace(B: int, layouts, num_splits: int, device):
+    """fp32 partials of split decode attention, shared by a model's layers (None: one split)."""
+    if num_splits <= 1:
+        return None
+    n = max(B * L.heads * num_splits * L.pads[1] for L in layouts)
+    m = max(B * L.heads * num_splits * 2 for L in layouts)
+    return (torch.empty(n, dtype=torch.float32, device=device), torch.empty(m, dtype=torch.float32, device=device))
+
+
+def attn_gd_decode(q: torch.Tensor, cache: tuple, block_tables: torch.Tensor, seq_lens: torch.Tensor, L: HeadLayout,
+                   scale: float, num_splits: int = 1, workspace: tuple | None = None) -> torch.Tensor:
+    """One query token per sequence over the paged cache -> [B, ocol] rows."""
+    if not q.is_cuda:
+        r = reference.attn_decode_rows(q, cache[0], cache[1], block_tables, seq_lens, scale)
+        o = torch.zeros(q.shape[0], L.ocol, dtype=q.dtype)
+        o[:, :L.heads * L.pads[1]] = r.reshape(q.shape[0], -1)
+        return o
+    o = _o_rows(q.shape[0], L, q.dtype, q.device)
+    if num_splits > 1 and workspace is None:
+        workspace = attn_gd_workspace(q.shape[0], [L], num_splits, q.device)
+    ws = workspace if num_splits > 1 else (None, None)
+    kernels().attn_gd_decode(q, cache[0], cache[1], block_tables, seq_lens, o, ws[0], ws[1], num_splits, scale)
+    return o
+
+
+# ---------------------------------------------------------------- routed experts
+def route(h: torch.Tensor, wr: torch.Tensor, experts: int, top: int, gated: bool):
+    """Router: (ids [T, top] int32, weights [T, top] fp32 sigmoid scores of the largest logits,
+    gate [T] fp32 | None). ``wr`` rows: the experts', then (``gated``) the shared expert's gate,
+    then zeros to a multiple of 16; logits in fp32."""
+    T, dev = h.shape[0], h.device
+    if not h.is_cuda:
+        return reference.route(h, wr, experts, top, gated)
+    ids = torch.empty(T, top, dtype=torch.int32, device=dev)
+    wt = torch.empty(T, top, dtype=torch.float32, device=dev)
+    gate = torch.empty(T, dtype=torch.float32, device=dev) if gated else None
+    if h.dtype == torch.bfloat16:
+        kernels().moe_route(h, wr, experts, ids, wt, gate)
+    else:
+        z = torch.empty(T, wr.shape[0], dtype=torch.float32, device=dev)
+        kernels().gemm_f32(h, wr, z)
+        kernels().moe_topk(z, experts, ids, wt, gate)
+    return ids, wt, gate
+
+
+def expert_rows_bound(slots: int, experts: int, bm: int) -> int:
+    """Rows an expert-sorted batch can need: every segment padded to ``bm``."""
+    return pad_to(slots + min(experts, slots) * (bm - 1), bm)
+
+
+def experts(h: torch.Tensor, ids: torch.Tensor, wt: torch.Tensor, wgu: torch.Tensor, wd: torch.Tensor):
+    """SwiGLU experts on their tokens scaled by the router weight: (rows, epos) such that
+    token t's contributions are rows[epos[t, k]] (epos None: row t * top + k).
+    wgu [E, 2 ff, ld] with gate | up interleaved in 64-row blocks, wd [E, ld, ff]."""
+    T, top = ids.shape
+    E, ld, ff = wd.shape
+    slots = T * top
+    if not h.is_cuda:
+        return reference.experts(h, ids, wt, wgu, wd), None
+    C, dev = kernels(), h.device
+    bf16 = h.dtype == torch.bfloat16
+    if bf16 and slots <= MOE_SKINNY_MAX_SLOTS and slots < MOE_TILE_MIN_ROWS * E:
+        m = torch.empty(slots, ff, dtype=h.dtype, device=dev)
+        C.moe_gemm_skinny(h, wgu, m, ids, wt, top, True)
+        y = torch.empty(slots, ld, dtype=h.dtype, device=dev)
+        C.moe_gemm_skinny(m, wd, y, ids, wt, 1, False)
+        return y, None
+    bm = 256 if bf16 else 64
+    rows = expert_rows_bound(slots, E, bm)
+    i32 = dict(dtype=torch.int32, device=dev)
+    pos, src, gtab = torch.empty(T, top, **i32), torch.empty(rows, **i32), torch.empty(1 + rows // bm, **i32)
+    rs = torch.empty(rows, dtype=torch.float32, device=dev)
+    C.moe_sort(ids, wt, E, bm, pos, src, rs, gtab)
+    xp = torch.empty(rows, ld, dtype=h.dtype, device=dev)
+    C.moe_gather(h, src, gtab, bm, xp)
+    m = torch.empty(rows, ff, dtype=h.dtype, device=dev)
+    y = torch.empty(rows, ld, dtype=h.dtype, device=dev)
+    if bf16:
+        C.moe_gemm_tile(xp, wgu, m, gtab, rs, True)
+        C.moe_gemm_tile(m, wd, y, gtab)
+    else:
+        C.gemm_f32(xp, wgu, m, True, gtab, rs)
+        C.gemm_f32(m, wd, y, False, gtab)
+    return y, pos

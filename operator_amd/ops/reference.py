@@ -150,7 +150,7 @@ def attn_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, cu_seqlens: 
     cu = [int(x) for x in cu_seqlens]
     Hq, Hkv = q.shape[1], k.shape[1]
     G = Hq // Hkv
-    out = torch.empty_like(q)
+    out = torch.zeros(q.shape[0], Hq, v.shape[2], dtype=q.dtype, device=q.device)
     for i in range(len(cu) - 1):
         a, b = cu[i], cu[i + 1]
         if b == a:
@@ -245,3 +245,100 @@ def sample_shard(logits: torch.Tensor, temperature: torch.Tensor, seeds: torch.T
 def sample(logits: torch.Tensor, temperature: torch.Tensor, seeds: torch.Tensor,
            positions: torch.Tensor) -> torch.Tensor:
     return sample_shard(logits, temperature, seeds, positions)[0]
+
+
+# ---------------------------------------------------------------- ops/decoder.py
+def stream_norm(x: torch.Tensor, inp: torch.Tensor | None, w: torch.Tensor, width: int, eps: float) -> torch.Tensor:
+    """RMS norm of the weighted (``inp`` None: plain) sum of the streams [T, S, ld]; fp32."""
+    u = x.sum(1) if inp is None else torch.matmul(x.transpose(1, 2), inp)
+    return u * torch.rsqrt(u.pow(2).sum(-1, keepdim=True) / width + eps) * w
+
+
+def stream_mix(x: torch.Tensor, y: torch.Tensor, mix: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """New streams: x'_t = sum_s mix[s, t] x_s + out[t] y."""
+    return torch.matmul(mix.t(), x) + out[None, :, None] * y[:, None, :]
+
+
+def sublayer_out(y, gate, e, epos, top: int, T: int, ld: int) -> torch.Tensor:
+    """A sublayer's output in fp32 from its parts (ops.decoder.SublayerOut)."""
+    r = torch.zeros(T, ld) if y is None else y.float()
+    if gate is not None:
+        r = r * torch.sigmoid(gate)[:, None]
+    if top:
+        rows = torch.arange(T * top).view(T, top) if epos is None else epos.long()
+        r = r + e.float()[rows].sum(1)
+    return r
+
+
+def qkv_heads(qkv: torch.Tensor, bias, pos: torch.Tensor, cos, sin, L, v_first, lam):
+    """fp32 (q, k, v) of packed projection rows: + bias, neighbours-paired rotation of the first
+    rot_dims dimensions, per-head RMS norm of q and k, value mixing."""
+    T = qkv.shape[0]
+    dk, dv = L.pads
+    x = qkv.float() if bias is None else qkv.float() + bias
+    nq, nk = L.heads * dk, L.kv_heads * dk
+    q, k = x[:, :nq].reshape(T, L.heads, dk), x[:, nq:nq + nk].reshape(T, L.kv_heads, dk)
+    v = x[:, nq + nk:nq + nk + L.kv_heads * dv].reshape(T, L.kv_heads, dv)
+
+    def turn(t):
+        if cos is None or L.rot_dims < 2:
+            return t
+        n = L.rot_dims // 2
+        c, s = cos[pos][:, None, :n], sin[pos][:, None, :n]
+        a, b = t[..., 0:2 * n:2], t[..., 1:2 * n:2]
+        r = t.clone()
+        r[..., 0:2 * n:2], r[..., 1:2 * n:2] = a * c - b * s, b * c + a * s
+        return r
+
+    def unit(t):
+        return t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) / L.dim + L.eps) if L.norm else t
+
+    q, k = unit(turn(q)), unit(turn(k))
+    if v_first is not None:
+        v = (1 - lam) * v + lam * v_first.float()
+    return q, k, v
+
+
+def cache_rows(k_cache: torch.Tensor, v_cache: torch.Tensor, k: torch.Tensor, v: torch.Tensor, slots: torch.Tensor) -> None:
+    """Write k / v [T, G, d] to a token-row paged cache [pages, G, P, d]."""
+    P = k_cache.shape[2]
+    ok = slots >= 0
+    pg, off = slots[ok] // P, slots[ok] % P
+    k_cache[pg, :, off] = k[ok].to(k_cache.dtype)
+    v_cache[pg, :, off] = v[ok].to(v_cache.dtype)
+
+
+def attn_decode_rows(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
+                     seq_lens: torch.Tensor, scale: float) -> torch.Tensor:
+    """One query token per sequence over a token-row paged cache; keys and values of any size."""
+    B, Hq, _ = q.shape
+    Hkv, P = k_cache.shape[1], k_cache.shape[2]
+    out = torch.zeros(B, Hq, v_cache.shape[3], dtype=q.dtype, device=q.device)
+    for b in range(B):
+        n = int(seq_lens[b])
+        if n == 0:
+            continue
+        pages = block_tables[b, :(n + P - 1) // P].long()
+        k = k_cache[pages].permute(1, 0, 2, 3).reshape(Hkv, -1, k_cache.shape[3])[:, :n].float()
+        v = v_cache[pages].permute(1, 0, 2, 3).reshape(Hkv, -1, v_cache.shape[3])[:, :n].float()
+        s = torch.matmul(q[b].float().view(Hkv, Hq // Hkv, -1), k.transpose(1, 2)) * scale
+        out[b] = torch.matmul(torch.softmax(s, -1), v).reshape(Hq, -1).to(q.dtype)
+    return out
+
+
+def route(h: torch.Tensor, wr: torch.Tensor, experts: int, top: int, gated: bool):
+    z = h.float() @ wr.float().t()
+    v, i = torch.topk(z[:, :experts], top, dim=-1)
+    return i.to(torch.int32), torch.sigmoid(v), z[:, experts].contiguous() if gated else None
+
+
+def experts(h: torch.Tensor, ids: torch.Tensor, wt: torch.Tensor, wgu: torch.Tensor, wd: torch.Tensor) -> torch.Tensor:
+    """Row t * top + k: expert ids[t, k] on wt[t, k] * h[t] (gate | up interleaved in 64-row blocks)."""
+    T, top = ids.shape
+    y = torch.zeros(T * top, wd.shape[1], dtype=h.dtype)
+    flat, xs = ids.reshape(-1), h.float().repeat_interleave(top, 0) * wt.reshape(-1, 1)
+    for e in flat.unique().tolist():
+        r = flat == e
+        gu = (xs[r] @ wgu[e].float().t()).to(h.dtype)
+        y[r] = (silu_mul(gu, 64).float() @ wd[e].float().t()).to(h.dtype)
+    return y

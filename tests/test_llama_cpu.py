@@ -279,7 +279,7 @@ def test_weight_cache_roundtrip(tmp_path, wd):
     for t0, t1 in [(a.embed, b.embed), (a.lm_head, b.lm_head), (a.final_norm, b.final_norm)]:
         assert torch.equal(t0, t1)
     for la, lb in zip(a.layers, b.layers):
-        for f in weight_cache.LAYER_FIELDS:
+        for f in weight_cache.layer_fields(a):
             x, y = getattr(la, f), getattr(lb, f)
             assert (x is None) == (y is None)
             if x is not None:
