@@ -179,13 +179,13 @@ class SufolixModel(DecoderModel):
     def init_random(self, seed: int = 0) -> "SufolixModel":
         """Random weights of the exact architecture: O(1) activations, streams that mix mildly."""
         def get(name, shape):
-            leaf = name.rsplit(".", 1)[-1]
+            owner, leaf = ([""] + name.split("."))[-2:]
             t = self._randn(seed, name, shape, 1.0)
             if leaf.startswith("norm"):
                 return 1.0 + 0.1 * t
             if leaf in ("in", "out"):
                 return (1.0 / self.cfg.streams if leaf == "in" else 1.0) + 0.1 * t
-            if len(shape) == 2 and name.split(".")[-2].startswith("hc"):
+            if owner.startswith("hc"):
                 return 0.05 * t + torch.eye(shape[0], dtype=t.dtype, device=t.device)
             if leaf == "vmix":
                 return 0.5 + 0.1 * t

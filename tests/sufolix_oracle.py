@@ -82,15 +82,21 @@ def gated(h, w, pre):
     return (g * torch.sigmoid(g) * u) @ w[pre + "down"].T
 
 
-def route(h, w, pre, router):
-    """(expert ids, weights) [T, top]: the largest sigmoid scores, used as they are."""
-    s = torch.sigmoid(h @ w[pre + "router"].T)
+def route(h, w, pre, router, close=None):
+    """(expert ids, weights) [T, top]: the largest sigmoid scores, used as they are. ``close``: a
+    list that receives, per token, the gap between the last expert taken and the first one left,
+    relative to the spread of the logits."""
+    z = h @ w[pre + "router"].T
+    s = torch.sigmoid(z)
     val, idx = torch.topk(s, router["top"], dim=-1)
+    if close is not None and router["top"] < router["experts"]:
+        v = torch.sort(z, dim=-1, descending=True)[0]
+        close.append((v[:, router["top"] - 1] - v[:, router["top"]]) / z.std())
     return idx, val
 
 
-def experts(h, w, pre, c):
-    idx, val = route(h, w, pre, c["router"])
+def experts(h, w, pre, c, close=None):
+    idx, val = route(h, w, pre, c["router"], close)
     y = torch.zeros_like(h)
     for t in range(h.shape[0]):
         for e, s in zip(idx[t].tolist(), val[t]):
@@ -110,9 +116,9 @@ def sublayer_out(xs, y, w, pre):
     return torch.einsum("tsw,sr->trw", xs, w[pre + "mix"]) + w[pre + "out"][None, :, None] * y[:, None, :]
 
 
-def forward(cfg, w, tokens, dtype=torch.float64, layer_out=None):
+def forward(cfg, w, tokens, dtype=torch.float64, layer_out=None, close=None):
     """Logits [T, vocab] of one sequence; ``layer_out``: a list that receives the stream sum
-    after every layer."""
+    after every layer; ``close``: one that receives every router's gaps (``route``)."""
     w = {k: v.to(dtype) for k, v in w.items()}
     eps = cfg["norm"]["eps"]
     x = w["embed"][torch.as_tensor(tokens, dtype=torch.long)] * cfg["embedding"]["scale"]
@@ -124,7 +130,7 @@ def forward(cfg, w, tokens, dtype=torch.float64, layer_out=None):
         xs = sublayer_out(xs, attention(u, w, pre + "mix.", lay["mixer"], eps, first), w, pre + "hc1.")
         if lay.get("mlp") is not None:
             u = rms(sublayer_in(xs, w, pre + "hc2."), eps, w[pre + "norm2"])
-            y = gated(u, w, pre + "mlp.") if lay["mlp"]["kind"] == "dense" else experts(u, w, pre + "mlp.", lay["mlp"])
+            y = gated(u, w, pre + "mlp.") if lay["mlp"]["kind"] == "dense" else experts(u, w, pre + "mlp.", lay["mlp"], close)
             xs = sublayer_out(xs, y, w, pre + "hc2.")
         if layer_out is not None:
             layer_out.append(xs.sum(1))

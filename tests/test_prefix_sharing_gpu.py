@@ -110,7 +110,8 @@ def test_shared_prefix_kv_equals_full_prompt_kv():
                       torch.arange(n, device="cuda"), True, torch.tensor([n - 1], device="cuda"), seq_lens=[n],
                       prefill_work=(i32([0, n]), i32(ws), i32(wq), var), kv_sink=sink)
     m.forward(fb, kv2)
-    for name, got, ref in (("k", eng._pk[:, :pf.n], cap_k[:, :pf.n]), ("v", eng._pv[:, :pf.n], cap_v[:, :pf.n])):
+    for name, got, ref in (("k", torch.stack([t[:pf.n] for t in eng._pk]), cap_k[:, :pf.n]),
+                           ("v", torch.stack([t[:pf.n] for t in eng._pv]), cap_v[:, :pf.n])):
         err = (got.float() - ref.float()).abs()
         scale = ref.float().abs().amax()
         assert float(err.amax()) <= 0.03 * float(scale) + 1e-3, (name, float(err.amax()), float(scale))
