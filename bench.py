@@ -93,6 +93,10 @@ def parse_args():
                     help="pipelined waves: wave w+1 fails when wave w's explanations are generated (the "
                          "engine's finish hook) or once every pipeline thread has its explanation back")
     ap.add_argument("--json-out", default=None)
+    ap.add_argument("--model-speed", nargs="+", metavar="MODEL", default=None,
+                    help="instead of the flagship step: prefill and decode throughput of these model presets, cut to "
+                         "--speed-layers layers, one JSON line per case (operator_amd/engine/speed.py)")
+    ap.add_argument("--speed-layers", type=int, default=4)
     ap.add_argument("--cpu", action="store_true",
                     help="CPU rehearsal (gloo, tiny models): allows --gpus N > 1 on a host without N GPUs")
     return ap.parse_args()
@@ -167,6 +171,11 @@ def shard_read(kid, what: str) -> str:
 
 def main() -> int:
     a = parse_args()
+    if a.model_speed:
+        from operator_amd.engine import speed
+
+        speed.run(a.model_speed, a.speed_layers, emit=lambda line: print(line, flush=True))
+        return 0
     child = a.shard_index is not None
     if not child and a.gpus > 1 and "WORLD_SIZE" not in os.environ:
         return launch_ranks(a)

@@ -177,7 +177,6 @@ void qkv_heads(const at::Tensor& qkv, const OptT& slabs, int64_t splits, const O
   if (v_out.has_value()) need(*v_out, dt, T * Hkv * dvp, "v_out");
   a.k_out = vp(k_out);
   a.v_out = vp(v_out);
-  a.page_size = 16;
   if (k_cache.has_value()) {
     TORCH_CHECK(v_cache.has_value() && slots.has_value(), "qkv_heads: k_cache needs v_cache and slots");
     TORCH_CHECK(k_cache->dim() == 4 && v_cache->dim() == 4 && k_cache->size(1) == Hkv && v_cache->size(1) == Hkv &&
@@ -190,7 +189,9 @@ void qkv_heads(const at::Tensor& qkv, const OptT& slabs, int64_t splits, const O
     a.k_cache = k_cache->data_ptr();
     a.v_cache = v_cache->data_ptr();
     a.slots = p<int64_t>(*slots);
-    a.page_size = (int)k_cache->size(2);
+    const int64_t P = k_cache->size(2);
+    TORCH_CHECK(P >= 1 && (P & (P - 1)) == 0, "qkv_heads: pages of a power of two tokens");
+    while ((1 << a.log2_page) < P) ++a.log2_page;
   }
   const c10::hip::HIPGuardMasqueradingAsCUDA g(pos.device());
   RC(oamd::qkv_heads(a, (int)T, f32, cur_stream()));
@@ -387,6 +388,31 @@ void moe_gemm_skinny(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, co
                            (int)div, (int)E, (int)N, (int)K, silu_gu, cur_stream()));
 }
 
+// rows: moe_sort's, in tiles of bm; src given: x [T, K] is gathered by it (values < T)
+void moe_gemm_rows(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, int64_t bm, const at::Tensor& gtab,
+                   const OptT& src, const OptT& rscale, bool silu_gu) {
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 3 && y.dim() == 2 && w.size(2) == x.size(1), "moe_gemm_rows: x [.., K], w [E, N, K]");
+  const int64_t M = y.size(0), N = w.size(1), K = w.size(2);
+  need(x, at::kBFloat16, x.numel(), "x");
+  need(w, at::kBFloat16, w.numel(), "w");
+  need(y, at::kBFloat16, M * (silu_gu ? N / 2 : N), "y");
+  TORCH_CHECK((bm == 64 || bm == 128) && M % bm == 0 && (src.has_value() || x.size(0) == M) && x.size(0) >= 1, "moe_gemm_rows: rows");
+  need(gtab, at::kInt, 1 + M / bm, "gtab", true);
+  if (src.has_value()) need(*src, at::kInt, M, "src");
+  if (rscale.has_value()) need(*rscale, at::kFloat, M, "rscale");
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  RC(oamd::moe_gemm_rows(p<bf16_t>(x), p<bf16_t>(w), p<bf16_t>(y), (int)M, (int)N, (int)K, (int)bm, silu_gu, p<int>(gtab),
+                         op<int>(src), op<float>(rscale), cur_stream()));
+}
+
+void splitk_silu(const at::Tensor& slabs, at::Tensor& y, int64_t splits) {
+  TORCH_CHECK(y.dim() == 2 && splits >= 1, "splitk_silu: y [M, N / 2]");
+  need(y, at::kBFloat16, y.numel(), "y");
+  need(slabs, at::kFloat, splits * y.numel() * 2, "slabs", true);
+  const c10::hip::HIPGuardMasqueradingAsCUDA g(y.device());
+  RC(oamd::splitk_silu(p<float>(slabs), p<bf16_t>(y), (int)y.size(0), (int)y.size(1) * 2, (int)splits, cur_stream()));
+}
+
 void moe_gemm_tile(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const at::Tensor& gtab, const OptT& rscale,
                    bool silu_gu) {
   TORCH_CHECK(x.dim() == 2 && w.dim() == 3 && y.dim() == 2 && w.size(2) == x.size(1), "moe_gemm_tile: x [rows, K], w [E, N, K]");
@@ -430,6 +456,9 @@ void register_decoder_bindings(pybind11::module_& m) {
   m.def("moe_gather", &moe_gather);
   m.def("moe_gemm_skinny", &moe_gemm_skinny, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("ids"),
         py::arg("weights"), py::arg("div"), py::arg("silu_gu"));
+  m.def("moe_gemm_rows", &moe_gemm_rows, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("bm"), py::arg("gtab"),
+        py::arg("src") = no, py::arg("rscale") = no, py::arg("silu_gu") = false);
+  m.def("splitk_silu", &splitk_silu);
   m.def("moe_gemm_tile", &moe_gemm_tile, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("gtab"),
         py::arg("rscale") = no, py::arg("silu_gu") = false);
 }

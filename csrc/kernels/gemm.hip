@@ -66,11 +66,16 @@ __device__ __forceinline__ void wait_vmcnt() {
 // [0,64) = gate, [64,128) = up of the same 64 features; output [M, N/2]).
 enum { kEpiStore = 0, kEpiPartial = 1, kEpiSiluGU = 2 };
 
-template <int BM, int BN, int EPI, int NS = kStages>
+// GRP: routed experts. Row tile y holds rows of one expert (moe_sort with bm = BM): gtab[0] = row
+// tiles, gtab[1 + y] = its expert, W [experts][N][K]; src != nullptr: row r reads X row src[r]
+// (< 0: padding, any row), and rscale[r] multiplies both SwiGLU operands.
+template <int BM, int BN, int EPI, int NS = kStages, bool GRP = false>
 __global__ void __launch_bounds__(kWaves * 64, NS == 2 ? 2 : 1) gemm_tn_kernel(const bf16_t* __restrict__ X,
                                                                  const bf16_t* __restrict__ W, bf16_t* __restrict__ Y,
                                                                  float* __restrict__ P, int M, int N, int K, int S,
-                                                                 int w_tiled) {
+                                                                 int w_tiled, const int* __restrict__ gtab = nullptr,
+                                                                 const int* __restrict__ src = nullptr,
+                                                                 const float* __restrict__ rscale = nullptr) {
   using C = GemmCfg<BM, BN, NS>;
   __shared__ __attribute__((aligned(1024))) char lds[C::LDS_BYTES];
   const int tid = threadIdx.x, lane = tid & 63;
@@ -78,7 +83,11 @@ __global__ void __launch_bounds__(kWaves * 64, NS == 2 ? 2 : 1) gemm_tn_kernel(c
   const int kz = blockIdx.x % S, nt = blockIdx.x / S;
   const int n0 = nt * BN;
   const int m0 = blockIdx.y * BM;  // row tile (M may be split into BM-row tiles)
-  X += (int64_t)m0 * K;
+  if constexpr (GRP) {
+    if ((int)blockIdx.y >= gtab[0]) return;
+    W += (int64_t)gtab[1 + blockIdx.y] * N * K;
+  }
+  if (!GRP || src == nullptr) X += (int64_t)m0 * K;
   // K-slice kz = K-steps [kz * TK / S, (kz + 1) * TK / S): slices differ by at most one step
   // when S does not divide TK (S = 5 puts 240 workgroups of the 48-tile qkv on 256 CUs)
   const int TK = K / kBK;
@@ -90,6 +99,14 @@ __global__ void __launch_bounds__(kWaves * 64, NS == 2 ? 2 : 1) gemm_tn_kernel(c
   // stage (A rows [0, BM), then B rows [BM, BM + BN)); lane l -> row 8q + l/8,
   // LDS slot l%8, global chunk swz(row, slot).
   const int lrow = lane >> 3, lslot = lane & 7;
+  int xrow[C::GL];   // X row of this lane's piece i (rows past BM are W's)
+#pragma unroll
+  for (int i = 0; i < C::GL; ++i) {
+    xrow[i] = 8 * (w + kWaves * i) + lrow;
+    if constexpr (GRP) {
+      if (src != nullptr && xrow[i] < BM) xrow[i] = max(src[m0 + xrow[i]], 0);
+    }
+  }
   auto issue_one = [&](int t, int buf, int i) {
     const int k0 = kbase + t * kBK;
     char* sbase = lds + buf * C::STAGE_BYTES;
@@ -102,11 +119,11 @@ __global__ void __launch_bounds__(kWaves * 64, NS == 2 ? 2 : 1) gemm_tn_kernel(c
       // contiguous 1 KB of HBM instead of 8 separate 128-B row segments
       const bf16_t* wsrc = (w_tiled & 1) ? W + ((int64_t)(wn_ >> 6) * (K >> 6) + (k0 >> 6)) * 4096 + (wn_ & 63) * 64 + chunk * 8
                                    : W + (int64_t)wn_ * K + k0 + chunk * 8;
-      const bf16_t* src = (row < BM) ? X + (int64_t)row * K + k0 + chunk * 8 : wsrc;
+      const bf16_t* from = (row < BM) ? X + (int64_t)xrow[i] * K + k0 + chunk * 8 : wsrc;
       if ((w_tiled & 2) && row >= BM)   // wave-uniform (8-row pieces): weights stream non-temporal
-        __builtin_amdgcn_global_load_lds(src, (__attribute__((address_space(3))) void*)(sbase + q * 1024), 16, 0, 2);
+        __builtin_amdgcn_global_load_lds(from, (__attribute__((address_space(3))) void*)(sbase + q * 1024), 16, 0, 2);
       else
-        __builtin_amdgcn_global_load_lds(src, (__attribute__((address_space(3))) void*)(sbase + q * 1024), 16, 0, 0);
+        __builtin_amdgcn_global_load_lds(from, (__attribute__((address_space(3))) void*)(sbase + q * 1024), 16, 0, 0);
     }
   };
   auto issue = [&](int t, int buf) {
@@ -200,11 +217,13 @@ __global__ void __launch_bounds__(kWaves * 64, NS == 2 ? 2 : 1) gemm_tn_kernel(c
     for (int v = tid; v < BM * 8; v += kWaves * 64) {
       const int row = v >> 3, f0 = (v & 7) * 8;
       const float* cr = ct + row * LD;
+      float c = 1.f;
+      if constexpr (GRP) c = rscale[m0 + row];
       u16x8 o;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        const float g = bf2f(f2bf(cr[f0 + e]));
-        const float u = bf2f(f2bf(cr[64 + f0 + e]));
+        const float g = bf2f(f2bf(GRP ? c * cr[f0 + e] : cr[f0 + e]));
+        const float u = bf2f(f2bf(GRP ? c * cr[64 + f0 + e] : cr[64 + f0 + e]));
         const float sg = bf2f(f2bf(g / (1.f + __expf(-g))));
         o[e] = f2bf(sg * u);
       }
@@ -243,6 +262,24 @@ int splitk_reduce(const float* P, bf16_t* Y, int64_t MN, int S, hipStream_t stre
   if (MN % 4 != 0 || S < 1) return -1;
   const int64_t threads = MN / 4;
   gemm_splitk_reduce_kernel<<<(threads + 255) / 256, 256, 0, stream>>>(P, Y, MN, S);
+  OAMD_LAUNCH_CHECK();
+  return 0;
+}
+
+int moe_gemm_rows(const bf16_t* X, const bf16_t* W, bf16_t* Y, int max_rows, int N, int K, int bm, bool silu_gu,
+                  const int* gtab, const int* src, const float* rscale, hipStream_t stream) {
+  if (max_rows == 0) return 0;
+  if ((bm != 64 && bm != 128) || max_rows % bm != 0 || N % 128 != 0 || K % kBK != 0 || gtab == nullptr) return -1;
+  if (silu_gu && rscale == nullptr) return -2;
+  const dim3 grid(N / 128, max_rows / bm);
+  if (bm == 64 && silu_gu)
+    gemm_tn_kernel<64, 128, kEpiSiluGU, 3, true><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, nullptr, max_rows, N, K, 1, 2, gtab, src, rscale);
+  else if (bm == 64)
+    gemm_tn_kernel<64, 128, kEpiStore, 3, true><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, nullptr, max_rows, N, K, 1, 2, gtab, src, rscale);
+  else if (silu_gu)
+    gemm_tn_kernel<128, 128, kEpiSiluGU, 3, true><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, nullptr, max_rows, N, K, 1, 2, gtab, src, rscale);
+  else
+    gemm_tn_kernel<128, 128, kEpiStore, 3, true><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, nullptr, max_rows, N, K, 1, 2, gtab, src, rscale);
   OAMD_LAUNCH_CHECK();
   return 0;
 }

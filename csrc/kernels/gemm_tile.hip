@@ -913,6 +913,14 @@ __global__ void splitk_silu_reduce_kernel(const float* __restrict__ P, bf16_t* _
   *reinterpret_cast<uint2*>(Y + (int64_t)m * ldy + f) = pack4(o);
 }
 
+int splitk_silu(const float* P, bf16_t* Y, int M, int N, int S, hipStream_t stream) {
+  if (M < 1 || N % 128 != 0 || S < 1) return -1;
+  const int64_t threads = (int64_t)M * (N / 2) / 4;
+  splitk_silu_reduce_kernel<<<(threads + 255) / 256, 256, 0, stream>>>(P, Y, M, N, S, N / 2);
+  OAMD_LAUNCH_CHECK();
+  return 0;
+}
+
 template <int DEEP>
 static void launch_p5(const bf16_t* X, const bf16_t* W, bf16_t* Y, const bf16_t* bias, int M, int N, int K, int ldy,
                       bool silu_gu, int grid, hipStream_t stream, int gm = kGroupM) {

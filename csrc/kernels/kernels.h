@@ -57,6 +57,8 @@ int gemm_xr(const bf16_t* Xt, const bf16_t* W, bf16_t* Y, float* P, int M, int N
 int tile_rows(const bf16_t* x, bf16_t* xt, int rows, int K, hipStream_t stream);
 // Y[M, N] = bf16(sum_s P[s][M][N]) (fp32 split-K slabs).
 int splitk_reduce(const float* P, bf16_t* Y, int64_t MN, int S, hipStream_t stream);
+// Y [M, N/2] = SwiGLU of the summed fp32 slabs [S][M][N] of a 64-row interleaved gate|up projection.
+int splitk_silu(const float* P, bf16_t* Y, int M, int N, int S, hipStream_t stream);
 // Skinny-M decode GEMM (M <= 32, gemm_skinny.hip): N % 16 == 0, K % (128 S) == 0; S-way split-K slabs P
 // reduced into Y (Y == nullptr: left for the consumer); silu_gu: fused SwiGLU over the 64-row
 // interleaved gate|up weight, Y [M, N/2].
@@ -196,7 +198,7 @@ struct QkvHeads {
   void *q_out, *k_out, *v_out;
   void *k_cache, *v_cache;
   const int64_t* slots;     // < 0: not cached
-  int page_size;
+  int log2_page;            // tokens per cache page = 1 << log2_page
 };
 int qkv_heads(const QkvHeads& a, int tokens, bool f32, hipStream_t stream);
 
@@ -259,6 +261,9 @@ int moe_gather(const void* h, const int* src, const int* gtab, int bm, int max_r
 // products over the 64-row interleaved gate|up weight. W [E][N][K], K % 64 == 0, N % 16 == 0 (silu: 128).
 int moe_gemm_skinny(const bf16_t* X, const bf16_t* W, bf16_t* Y, const int* ids, const float* weights, int slots,
                     int div, int E, int N, int K, bool silu_gu, hipStream_t stream);
+// Row tiles of bm = 64 or 128 sorted rows on the decode GEMM (gemm.hip); src: gathers X rows on the way in.
+int moe_gemm_rows(const bf16_t* X, const bf16_t* W, bf16_t* Y, int max_rows, int N, int K, int bm, bool silu_gu,
+                  const int* gtab, const int* src, const float* rscale, hipStream_t stream);
 // Prefill: rows sorted by moe_sort with bm = 256, persistent 256 x 256 tiles (gemm_tile.hip).
 int moe_gemm_tile(const bf16_t* X, const bf16_t* W, bf16_t* Y, int max_rows, int N, int K, bool silu_gu,
                   const int* gtab, const float* rscale, hipStream_t stream);

@@ -18,10 +18,12 @@ constexpr int kMaxExperts = 512;
 
 // One wave: the `top` largest of z[0..E) (ties to the smaller index), their sigmoid scores and
 // the ids, always inside [0, E). A NaN logit (a padding row's) counts as the smallest.
+// NE: E <= 64 NE.
+template <int NE>
 __device__ __forceinline__ void wave_topk(const float* z, int E, int top, int lane, int* ids, float* weights) {
-  float v[kMaxExperts / 64];
+  float v[NE];
 #pragma unroll
-  for (int i = 0; i < kMaxExperts / 64; ++i) {
+  for (int i = 0; i < NE; ++i) {
     const int e = lane + 64 * i;
     const float x = e < E ? z[e] : -INFINITY;
     v[i] = x == x ? x : -INFINITY;
@@ -31,7 +33,7 @@ __device__ __forceinline__ void wave_topk(const float* z, int E, int top, int la
     float best = -INFINITY;
     int bi = 0x7fffffff;
 #pragma unroll
-    for (int i = 0; i < kMaxExperts / 64; ++i) {
+    for (int i = 0; i < NE; ++i) {
       const int e = lane + 64 * i;
       if (e < E && !(taken >> i & 1) && (bi == 0x7fffffff || v[i] > best)) best = v[i], bi = e;
     }
@@ -51,51 +53,68 @@ __device__ __forceinline__ void wave_topk(const float* z, int E, int top, int la
 
 }  // namespace
 
-// 16 tokens per workgroup, 8 waves split K; experts in groups of 64 (4 MFMA tiles), the waves'
-// partial tiles summed through LDS into z[token][expert]. wr: [rows_w][K] rows (rows_w % 16 == 0,
-// rows past the last used one zero).
-__global__ void __launch_bounds__(512) moe_route_kernel(const bf16_t* __restrict__ h, const bf16_t* __restrict__ wr,
+// 16 tokens per workgroup, 8 waves split K; experts in groups of NT MFMA tiles of 16, the waves'
+// partial tiles summed through LDS into z[token][expert]. wr: [rows_w][K] rows (rows_w % (16 NT)
+// == 0, rows past the last used one zero). NE: experts per lane of the top-k.
+constexpr int kRouteWaves = 8;
+
+template <int NT, int NE>
+__global__ void __launch_bounds__(kRouteWaves * 64) moe_route_kernel(const bf16_t* __restrict__ h, const bf16_t* __restrict__ wr,
                                                         int T, int K, int E, int rows_w, int top, int* __restrict__ ids,
                                                         float* __restrict__ weights, float* __restrict__ gate,
                                                         float* __restrict__ logits) {
+  constexpr int U = NT == 1 ? 16 : NT == 2 ? 8 : 4;   // K steps whose loads are in flight together
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  float* red = sm;                       // [8 waves][4 tiles][256]
-  float* z = sm + 8 * 4 * 256;           // [16][rows_w]
+  float* red = sm;                              // [waves][NT][256]
+  float* z = sm + kRouteWaves * NT * 256;       // [16][rows_w]
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
   const int l15 = lane & 15, lq = lane >> 4;
   const int t0 = blockIdx.x * 16;
   const bf16_t* hp = h + (int64_t)min(t0 + l15, T - 1) * K + 8 * lq;
   const int steps = K / 32;
-  for (int e0 = 0; e0 < rows_w; e0 += 64) {
-    const int nt = min(4, (rows_w - e0) / 16);
-    f32x4 acc[4];
+  for (int e0 = 0; e0 < rows_w; e0 += 16 * NT) {
+    f32x4 acc[NT];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     const bf16_t* wp = wr + (int64_t)(e0 + l15) * K + 8 * lq;
-#pragma unroll 4
-    for (int s = w; s < steps; s += 8) {
+    int s = w;
+    for (; s + (U - 1) * kRouteWaves < steps; s += U * kRouteWaves) {
+      u16x8 b[U], wv[U][NT];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int k = 32 * (s + u * kRouteWaves);
+        b[u] = *reinterpret_cast<const u16x8*>(hp + k);
+#pragma unroll
+        for (int i = 0; i < NT; ++i) wv[u][i] = *reinterpret_cast<const u16x8*>(wp + (int64_t)16 * i * K + k);
+      }
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int i = 0; i < NT; ++i) acc[i] = mfma16(wv[u][i], b[u], acc[i]);
+    }
+    for (; s < steps; s += kRouteWaves) {
       const u16x8 b = *reinterpret_cast<const u16x8*>(hp + 32 * s);
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-        if (i < nt) acc[i] = mfma16(*reinterpret_cast<const u16x8*>(wp + (int64_t)16 * i * K + 32 * s), b, acc[i]);
+      for (int i = 0; i < NT; ++i)
+        acc[i] = mfma16(*reinterpret_cast<const u16x8*>(wp + (int64_t)16 * i * K + 32 * s), b, acc[i]);
     }
     __syncthreads();   // red of the previous expert group is consumed
 #pragma unroll
-    for (int i = 0; i < 4; ++i) *reinterpret_cast<f32x4*>(red + ((w * 4 + i) * 64 + lane) * 4) = acc[i];
+    for (int i = 0; i < NT; ++i) *reinterpret_cast<f32x4*>(red + ((w * NT + i) * 64 + lane) * 4) = acc[i];
     __syncthreads();
-    for (int x = tid; x < nt * 256; x += 512) {   // tile i, lane l, register j: expert 16 i + 4 (l >> 4) + j, token l & 15
+    for (int x = tid; x < NT * 256; x += kRouteWaves * 64) {   // tile i, lane l, register j: expert 16 i + 4 (l >> 4) + j, token l & 15
       const int i = x >> 8, l = (x >> 2) & 63, j = x & 3;
       float v = 0.f;
 #pragma unroll
-      for (int ww = 0; ww < 8; ++ww) v += red[((ww * 4 + i) * 64 + l) * 4 + j];
+      for (int ww = 0; ww < kRouteWaves; ++ww) v += red[((ww * NT + i) * 64 + l) * 4 + j];
       z[(l & 15) * rows_w + e0 + 16 * i + 4 * (l >> 4) + j] = v;
     }
   }
   __syncthreads();
-  for (int i = w; i < 16; i += 8) {
+  for (int i = w; i < 16; i += kRouteWaves) {
     const int t = t0 + i;
     if (t >= T) break;
-    wave_topk(z + i * rows_w, E, top, lane, ids + (int64_t)t * top, weights + (int64_t)t * top);
+    wave_topk<NE>(z + i * rows_w, E, top, lane, ids + (int64_t)t * top, weights + (int64_t)t * top);
     if (gate && lane == 0) gate[t] = z[i * rows_w + E];
     if (logits)
       for (int e = lane; e < E; e += 64) logits[(int64_t)t * E + e] = z[i * rows_w + e];
@@ -106,9 +125,25 @@ int moe_route(const bf16_t* h, const bf16_t* wr, int T, int K, int E, int rows_w
               float* gate, float* logits, hipStream_t stream) {
   if (T == 0) return 0;
   if (K % 32 || rows_w % 16 || E + (gate ? 1 : 0) > rows_w || E < 1 || E > kMaxExperts || top < 1 || top > E) return -1;
-  const size_t lds = (8 * 4 * 256 + 16 * (size_t)rows_w) * sizeof(float);
+  const int NT = rows_w % 64 == 0 ? 4 : rows_w % 32 == 0 ? 2 : 1;
+  const size_t lds = (kRouteWaves * NT * 256 + 16 * (size_t)rows_w) * sizeof(float);
   if (lds > 128 * 1024) return -2;
-  moe_route_kernel<<<(T + 15) / 16, 512, lds, stream>>>(h, wr, T, K, E, rows_w, top, ids, weights, gate, logits);
+  const int grid = (T + 15) / 16, nt = kRouteWaves * 64;
+#define OAMD_ROUTE(NTT, NEE) \
+  moe_route_kernel<NTT, NEE><<<grid, nt, lds, stream>>>(h, wr, T, K, E, rows_w, top, ids, weights, gate, logits)
+#define OAMD_ROUTE_E(NTT)                                             \
+  if (E <= 64) OAMD_ROUTE(NTT, 1);                                    \
+  else if (E <= 128) OAMD_ROUTE(NTT, 2);                              \
+  else OAMD_ROUTE(NTT, kMaxExperts / 64)
+  if (NT == 1) {
+    OAMD_ROUTE_E(1);
+  } else if (NT == 2) {
+    OAMD_ROUTE_E(2);
+  } else {
+    OAMD_ROUTE_E(4);
+  }
+#undef OAMD_ROUTE_E
+#undef OAMD_ROUTE
   OAMD_LAUNCH_CHECK();
   return 0;
 }
@@ -120,7 +155,7 @@ __global__ void __launch_bounds__(256) moe_topk_kernel(const float* __restrict__
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= T) return;
   const float* z = logits + (int64_t)t * ld;
-  wave_topk(z, E, top, lane, ids + (int64_t)t * top, weights + (int64_t)t * top);
+  wave_topk<kMaxExperts / 64>(z, E, top, lane, ids + (int64_t)t * top, weights + (int64_t)t * top);
   if (gate && lane == 0) gate[t] = z[E];
 }
 
@@ -329,7 +364,7 @@ int moe_gemm_skinny(const bf16_t* X, const bf16_t* W, bf16_t* Y, const int* ids,
   if (slots > kMaxSlots || K % 32 || div < 1) return -1;
   if (silu_gu ? N % 128 : N % 16) return -2;
   const dim3 grid(silu_gu ? N / 32 : N / 16, E);
-  const int mt = slots <= 16 * (int64_t)E ? 1 : slots <= 32 * (int64_t)E ? 2 : 4;   // rows an expert gets on average
+  const int mt = slots <= 8 * (int64_t)E ? 1 : slots <= 20 * (int64_t)E ? 2 : 4;   // by the rows an expert gets on average
   if (silu_gu) {
     if (mt == 1) moe_skinny_kernel<2, 1><<<grid, 256, 0, stream>>>(X, W, Y, ids, weights, slots, div, N, K);
     else if (mt == 2) moe_skinny_kernel<2, 2><<<grid, 256, 0, stream>>>(X, W, Y, ids, weights, slots, div, N, K);

@@ -79,8 +79,18 @@ __global__ void __launch_bounds__(NT) stream_step_kernel(const StreamStep a) {
         f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f};
         if (a.yp) {
           const float* p = a.yp + row * a.ld + 4 * v;
-#pragma unroll 4
-          for (int s = 0; s < a.ys; ++s) y += *reinterpret_cast<const f32x4*>(p + s * a.y_slab);
+          int s0 = 0;
+          if constexpr (MAXV == 1) {   // up to 8 slabs requested before the first add: one round trip
+            f32x4 sl[8];
+#pragma unroll
+            for (int s = 0; s < 8; ++s)
+              if (s < a.ys) sl[s] = *reinterpret_cast<const f32x4*>(p + s * a.y_slab);
+#pragma unroll
+            for (int s = 0; s < 8; ++s)
+              if (s < a.ys) y += sl[s];
+            s0 = 8;
+          }
+          for (int s = s0; s < a.ys; ++s) y += *reinterpret_cast<const f32x4*>(p + s * a.y_slab);
         } else if (a.y) {
           y = ld4(a.y, row * a.ld + 4 * v, a.f32);
         }
@@ -110,7 +120,7 @@ __global__ void __launch_bounds__(NT) stream_step_kernel(const StreamStep a) {
     }
   }
   const float tot = block_sum<NT>(ss, scratch);
-  const float rs = 1.f / sqrtf(tot / static_cast<float>(a.width) + a.eps);
+  const float rs = rsqrtf(tot / static_cast<float>(a.width) + a.eps);
 #pragma unroll
   for (int i = 0; i < MAXV; ++i) {
     const int v = tid + i * NT;
@@ -127,6 +137,16 @@ __global__ void __launch_bounds__(NT) stream_step_kernel(const StreamStep a) {
 template <int S>
 static void launch_streams(const StreamStep& a, int n, hipStream_t stream) {
   const int nv = a.ld / 4;
+  if constexpr (S <= 4) {
+    // few rows (decode): a vector per thread, so a row's loads all leave in one round trip
+    if (n <= 512 && nv > 256) {
+      if (nv <= 512) stream_step_kernel<S, 512, 1><<<n, 512, 0, stream>>>(a);
+      else if (nv <= 1024) stream_step_kernel<S, 1024, 1><<<n, 1024, 0, stream>>>(a);
+      else if (nv <= 2048) stream_step_kernel<S, 1024, 2><<<n, 1024, 0, stream>>>(a);
+      else stream_step_kernel<S, 1024, 4><<<n, 1024, 0, stream>>>(a);
+      return;
+    }
+  }
   if (nv <= 64) stream_step_kernel<S, 64, 1><<<n, 64, 0, stream>>>(a);
   else if (nv <= 256) stream_step_kernel<S, 256, 1><<<n, 256, 0, stream>>>(a);
   else if (nv <= 1024) stream_step_kernel<S, 256, 4><<<n, 256, 0, stream>>>(a);

@@ -161,7 +161,7 @@ class SufolixModel(DecoderModel):
             rows.append((m.experts, 0, get(p + "mlp.shared.sg", (1, W))))
             lw.sgu = gu(p + "mlp.shared.", m.shared_ff)
             lw.sd = self._down(get(p + "mlp.shared.down", (W, m.shared_ff)))
-        lw.wr = self._put(dec.pad_to(m.experts + 1, 16), self.ld, rows)
+        lw.wr = self._put(dec.router_rows(m.experts), self.ld, rows)
         return lw
 
     def _build(self, get, has) -> "SufolixModel":

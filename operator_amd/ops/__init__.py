@@ -95,6 +95,16 @@ def interleave_gate_up(g: torch.Tensor, u: torch.Tensor, block: int = GU_BLOCK) 
         2 * inter, H).contiguous()
 
 
+def _gu_splits(M: int, N: int, K: int) -> int:
+    """K slices of a narrow gate|up decode GEMM: one block per 128-column tile leaves most CUs
+    idle below 96 tiles, and the extra SwiGLU pass over the slabs is worth it."""
+    tiles = N // 128 * (M // row_tile(M))
+    S = 1
+    while tiles * S < 96 and S < 8 and K // 64 >= 4 * S:
+        S *= 2
+    return S
+
+
 def gate_up_silu(x: torch.Tensor, wgu: torch.Tensor, block: int | None) -> torch.Tensor:
     """silu(x Wg^T) * (x Wu^T) from the interleaved gate|up weight. Decode buckets run
     one fused gfx950 kernel (GEMM + SwiGLU epilogue, no [M, 2I] intermediate);
@@ -117,6 +127,12 @@ def gate_up_silu(x: torch.Tensor, wgu: torch.Tensor, block: int | None) -> torch
             bm = int(t[2:])
             ws, fl = _pp_sk_workspace(x.device, N // 128) if (bm == 256 and PP_STREAM_K) else (None, None)
             kernels().gemm_pp(x, wgu, y, None, 1, bm, True, True, False, ws, fl)
+            return y
+        if t is None and (S := _gu_splits(M, N, K)) > 1:   # too few column tiles to fill the GPU: split K
+            y = torch.empty(M, N // 2, dtype=x.dtype, device=x.device)
+            slabs = torch.empty(S * M * N, dtype=torch.float32, device=x.device)
+            kernels().gemm_decode(x, wgu, None, slabs, S, 128, row_tile(M), False, False, 3)
+            kernels().splitk_silu(slabs, y, S)
             return y
         if t != "blas":
             bm = t[0] if t else row_tile(M)

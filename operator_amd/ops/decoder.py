@@ -19,9 +19,9 @@ from ._native import kernels
 # general attention work items: 128 query rows whatever the head layout (attn_gd_prefill.hip)
 GD_VARIANT = 5
 GD_BLOCK_Q = 128
-# expert GEMMs: rows per expert from which the 256-row tile kernel beats the weight-streaming one
-MOE_TILE_MIN_ROWS = 64
-MOE_SKINNY_MAX_SLOTS = 4096   # moe.hip kMaxSlots
+# expert GEMMs (expert_plan): most rows per expert, on average, of each form
+MOE_LIST_ROWS, MOE_64_ROWS, MOE_128_ROWS = 7, 44, 220
+MOE_LIST_MAX_SLOTS = 4096   # moe.hip kMaxSlots
 
 
 def pad_to(n: int, m: int) -> int:
@@ -220,10 +220,16 @@ def attn_gd_decode(q: torch.Tensor, cache: tuple, block_tables: torch.Tensor, se
 
 
 # ---------------------------------------------------------------- routed experts
+def router_rows(experts: int) -> int:
+    """Stored rows of a router with a gate row: whole groups of 1, 2 or 4 MFMA tiles."""
+    n = pad_to(experts + 1, 16)
+    return n if n <= 32 else pad_to(n, 64)
+
+
 def route(h: torch.Tensor, wr: torch.Tensor, experts: int, top: int, gated: bool):
     """Router: (ids [T, top] int32, weights [T, top] fp32 sigmoid scores of the largest logits,
     gate [T] fp32 | None). ``wr`` rows: the experts', then (``gated``) the shared expert's gate,
-    then zeros to a multiple of 16; logits in fp32."""
+    then zeros (``router_rows``); logits in fp32."""
     T, dev = h.shape[0], h.device
     if not h.is_cuda:
         return reference.route(h, wr, experts, top, gated)
@@ -244,10 +250,22 @@ def expert_rows_bound(slots: int, experts: int, bm: int) -> int:
     return pad_to(slots + min(experts, slots) * (bm - 1), bm)
 
 
-def experts(h: torch.Tensor, ids: torch.Tensor, wt: torch.Tensor, wgu: torch.Tensor, wd: torch.Tensor):
+def expert_plan(slots: int, E: int) -> int:
+    """How bf16 expert GEMMs run, by the rows an expert gets on average: 0 = weights streamed
+    against the rows of each expert's own list, no sorting (few rows), 64 / 128 = sorted rows in
+    tiles of that many on the decode GEMM, 256 = the prefill tile kernel."""
+    rows = slots / E
+    if rows <= MOE_LIST_ROWS and slots <= MOE_LIST_MAX_SLOTS:
+        return 0
+    return 64 if rows <= MOE_64_ROWS else 128 if rows <= MOE_128_ROWS else 256
+
+
+def experts(h: torch.Tensor, ids: torch.Tensor, wt: torch.Tensor, wgu: torch.Tensor, wd: torch.Tensor,
+            plan: int | None = None):
     """SwiGLU experts on their tokens scaled by the router weight: (rows, epos) such that
     token t's contributions are rows[epos[t, k]] (epos None: row t * top + k).
-    wgu [E, 2 ff, ld] with gate | up interleaved in 64-row blocks, wd [E, ld, ff]."""
+    wgu [E, 2 ff, ld] with gate | up interleaved in 64-row blocks, wd [E, ld, ff];
+    ``plan``: expert_plan's choice (bf16), for tests and tuning."""
     T, top = ids.shape
     E, ld, ff = wd.shape
     slots = T * top
@@ -255,22 +273,28 @@ def experts(h: torch.Tensor, ids: torch.Tensor, wt: torch.Tensor, wgu: torch.Ten
         return reference.experts(h, ids, wt, wgu, wd), None
     C, dev = kernels(), h.device
     bf16 = h.dtype == torch.bfloat16
-    if bf16 and slots <= MOE_SKINNY_MAX_SLOTS and slots < MOE_TILE_MIN_ROWS * E:
+    bm = (expert_plan(slots, E) if plan is None else plan) if bf16 else 64
+    if bm in (64, 128) and bf16 and ld % 128:
+        bm = 256   # the decode GEMM's column tiles
+    if bm == 0:
         m = torch.empty(slots, ff, dtype=h.dtype, device=dev)
         C.moe_gemm_skinny(h, wgu, m, ids, wt, top, True)
         y = torch.empty(slots, ld, dtype=h.dtype, device=dev)
         C.moe_gemm_skinny(m, wd, y, ids, wt, 1, False)
         return y, None
-    bm = 256 if bf16 else 64
     rows = expert_rows_bound(slots, E, bm)
     i32 = dict(dtype=torch.int32, device=dev)
     pos, src, gtab = torch.empty(T, top, **i32), torch.empty(rows, **i32), torch.empty(1 + rows // bm, **i32)
     rs = torch.empty(rows, dtype=torch.float32, device=dev)
     C.moe_sort(ids, wt, E, bm, pos, src, rs, gtab)
-    xp = torch.empty(rows, ld, dtype=h.dtype, device=dev)
-    C.moe_gather(h, src, gtab, bm, xp)
     m = torch.empty(rows, ff, dtype=h.dtype, device=dev)
     y = torch.empty(rows, ld, dtype=h.dtype, device=dev)
+    if bf16 and bm < 256:
+        C.moe_gemm_rows(h, wgu, m, bm, gtab, src, rs, True)
+        C.moe_gemm_rows(m, wd, y, bm, gtab)
+        return y, pos
+    xp = torch.empty(rows, ld, dtype=h.dtype, device=dev)
+    C.moe_gather(h, src, gtab, bm, xp)
     if bf16:
         C.moe_gemm_tile(xp, wgu, m, gtab, rs, True)
         C.moe_gemm_tile(m, wd, y, gtab)

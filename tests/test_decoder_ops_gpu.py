@@ -254,12 +254,14 @@ def _expert_weights(g, E, ff, ld, dtype):
 
 @pytest.mark.parametrize("T,E,top,ff,ld", [(1, 4, 1, 128, 128), (16, 8, 2, 192, 256), (33, 5, 5, 128, 192), (70, 3, 2, 128, 320),
                                            (300, 4, 2, 256, 256), (2100, 6, 3, 128, 128), (64, 200, 4, 128, 128)])
-@pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
-def test_route_and_experts(T, E, top, ff, ld, dtype):
+@pytest.mark.parametrize("dtype,plan", [(torch.bfloat16, p) for p in (None, 0, 64, 128, 256)] + [(torch.float32, None)])
+def test_route_and_experts(T, E, top, ff, ld, dtype, plan):
+    if plan == 0 and T * top > dec.MOE_LIST_MAX_SLOTS:
+        pytest.skip("more rows than an expert's list holds")
     g = _g(T + E)
     gate, up, down, wgu = _expert_weights(g, E, ff, ld, dtype)
     h = _rand(g, T, ld).to(dtype)
-    wr = torch.zeros(dec.pad_to(E + 1, 16), ld)
+    wr = torch.zeros(dec.router_rows(E), ld)
     wr[:E + 1] = _rand(g, E + 1, ld, scale=ld ** -0.5) * 2
     wr = wr.to(dtype)
     ids, wt, gt = dec.route(h.to(DEV), wr.to(DEV), E, top, True)
@@ -272,7 +274,7 @@ def test_route_and_experts(T, E, top, ff, ld, dtype):
     assert torch.equal(i.sort(1)[0][sure], idx.sort(1)[0][sure]) and int(i.min()) >= 0 and int(i.max()) < E
     _close(wt, torch.sigmoid(z.gather(1, i)), 1e-4)
     _close(gt, z[:, E], 1e-4)
-    rows, pos = dec.experts(h.to(DEV), ids, wt, wgu.to(DEV), down.to(DEV))
+    rows, pos = dec.experts(h.to(DEV), ids, wt, wgu.to(DEV), down.to(DEV), plan)
     p = torch.arange(T * top).view(T, top) if pos is None else pos.cpu().long()
     got = rows.double().cpu()[p].sum(1)
     w = wt.cpu().double()
@@ -292,11 +294,11 @@ def test_experts_all_tokens_to_one():
     g = _g(3)
     E, ff, ld = 6, 128, 256
     gate, up, down, wgu = _expert_weights(g, E, ff, ld, torch.bfloat16)
-    for T in (40, 1100):
+    for T, plan in ((40, 0), (40, 64), (200, 128), (1100, 256)):
         h = _rand(g, T, ld).to(torch.bfloat16)
         ids = torch.full((T, 1), 4, dtype=torch.int32, device=DEV)
         wt = torch.full((T, 1), 0.5, device=DEV)
-        rows, pos = dec.experts(h.to(DEV), ids, wt, wgu.to(DEV), down.to(DEV))
+        rows, pos = dec.experts(h.to(DEV), ids, wt, wgu.to(DEV), down.to(DEV), plan)
         p = torch.arange(T) if pos is None else pos.cpu().long().flatten()
         x = 0.5 * h.double()
         a, b = x @ gate[4].double().T, x @ up[4].double().T
@@ -322,3 +324,13 @@ def test_gemm_f32(M, N, K):
         y = ops.gate_up_silu(x.to(DEV), gu.to(DEV), 64)
         a, b = x.double() @ w.double().T, x.double() @ w.flip(0).double().T
         _close(y, a * torch.sigmoid(a) * b, 2e-6 * K ** 0.5)
+
+
+@pytest.mark.parametrize("M,N,K", [(64, 256, 512), (128, 1024, 256), (256, 512, 1024), (192, 128, 256)])
+def test_narrow_gate_up_splits_k(M, N, K):
+    g = _g(M)
+    a, b, x = (_rand(g, *s, scale=K ** -0.25).to(torch.bfloat16) for s in ((N // 2, K), (N // 2, K), (M, K)))
+    assert ops._gu_splits(M, N, K) > 1
+    y = ops.gate_up_silu(x.to(DEV), ops.interleave_gate_up(a, b).to(DEV), 64)
+    u, v = x.double() @ a.double().T, x.double() @ b.double().T
+    _close(y, u * torch.sigmoid(u) * v, 2e-2)
