@@ -1,5 +1,5 @@
-"""The general decoder kernels (streams, QKV heads, any-head-size attention, routed experts, fp32
-products) against plain fp32 / fp64 formulas."""
+"""The general decoder ops (streams, QKV heads, any-head-size attention, routed experts, fp32
+products), each alone, against plain fp64 formulas: the CPU references and the GPU kernels."""
 import pytest
 import torch
 
@@ -7,8 +7,14 @@ import sufolix_oracle as O
 from operator_amd import ops
 from operator_amd.ops import decoder as dec
 
-pytestmark = pytest.mark.gpu
-DEV = "cuda"
+DEV = "cpu"
+
+
+@pytest.fixture(autouse=True, params=["cpu", pytest.param("cuda", marks=pytest.mark.gpu)])
+def device(request):
+    global DEV
+    DEV = request.param
+    return DEV
 
 
 def _g(seed):
@@ -61,7 +67,7 @@ def test_stream_step(S, width, ld, dtype):
     # fp32 slabs and identity routing rows; the last step picks rows and keeps the streams
     slabs = _rand(g, 3, T, ld) * pad
     e = (_rand(g, T * top, ld) * pad).to(dtype)
-    sk = ops.SplitK(c(slabs).reshape(-1), 3, T, ld)
+    sk = slabs.sum(0) if DEV == "cpu" else ops.SplitK(c(slabs).reshape(-1), 3, T, ld)   # split-K is the GPU's
     rows = torch.tensor([4, 1])
     x = c(xr.float())
     h = dec.stream_step(x, dec.SublayerOut(sk, None, c(e), None, top), dec.Stream(c(inp), c(mix), c(out)), None, c(w),
@@ -80,7 +86,7 @@ LAYOUTS = [(8, 2, 48, 32, 48), (6, 3, 40, 24, 32), (4, 4, 128, 128, 128), (5, 1,
 def _cache_rows(cache, kind, dtype):
     """Token-row view [pages, G, P, d] of a layer's cache (bf16 GPU caches are tiled)."""
     c = cache.cpu()
-    if dtype == torch.float32:
+    if dtype == torch.float32 or DEV == "cpu":
         return c
     n, G, P, d = c.shape
     t = c.reshape(n, G, P // 16, 16 * d)
@@ -104,7 +110,8 @@ def test_qkv_heads(H, G, D, Dv, rot, dtype, slabs):
         real[(H + G) * dk + h * dv:(H + G) * dk + h * dv + Dv] = 1
     if slabs:
         sl = _rand(g, slabs, T, L.ncol) * real
-        src, rows = ops.SplitK(sl.reshape(-1).to(DEV), slabs, T, L.ncol), sl.double().sum(0)
+        src = sl.sum(0) if DEV == "cpu" else ops.SplitK(sl.reshape(-1).to(DEV), slabs, T, L.ncol)
+        rows = sl.double().sum(0)
     else:
         r = (_rand(g, T, L.ncol) * real).to(dtype)
         src, rows = r.to(DEV), r.double()
@@ -258,6 +265,8 @@ def _expert_weights(g, E, ff, ld, dtype):
 def test_route_and_experts(T, E, top, ff, ld, dtype, plan):
     if plan == 0 and T * top > dec.MOE_LIST_MAX_SLOTS:
         pytest.skip("more rows than an expert's list holds")
+    if DEV == "cpu" and (plan is not None or T > 300):
+        pytest.skip("kernel choice and tile borders are the GPU's")
     g = _g(T + E)
     gate, up, down, wgu = _expert_weights(g, E, ff, ld, dtype)
     h = _rand(g, T, ld).to(dtype)
