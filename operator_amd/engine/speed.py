@@ -110,7 +110,9 @@ def run(names: list[str], layers: int = 4, prefill=PREFILL, decode=DECODE, emit=
         for b, c in decode:
             from operator_amd import ops
 
-            reqs = [GenRequest([1] * (c - 1), output=[1]) for _ in range(b)]
+            # rows with tokens (and sampling seeds) of their own: equal rows would share their experts
+            reqs = [GenRequest([1] * (c - 1), output=[int(t)], temperature=1.0, seed=i)
+                    for i, t in enumerate(torch.randint(0, cfg.vocab_size, (b,)))]
             for r in reqs:
                 eng._reserve(r)
                 r.pages = r.pages + kv.allocator.alloc(1)   # the steps below pass the page's end

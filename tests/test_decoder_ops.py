@@ -79,7 +79,7 @@ def test_stream_step(S, width, ld, dtype):
 
 
 # ---------------------------------------------------------------- QKV heads
-LAYOUTS = [(8, 2, 48, 32, 48), (6, 3, 40, 24, 32), (4, 4, 128, 128, 128), (5, 1, 96, 64, 20), (2, 1, 16, 40, 16),
+LAYOUTS = [(10, 2, 56, 40, 24), (6, 3, 40, 24, 32), (4, 4, 128, 128, 128), (5, 1, 96, 64, 20), (2, 1, 16, 40, 16),
            (3, 3, 200, 160, 100), (16, 1, 64, 96, 2)]
 
 
@@ -163,7 +163,7 @@ def _spiky(g, T, H, G, D, Dv, dtype):
     return q.to(dtype), k.to(dtype), v.to(dtype)
 
 
-SHAPES = [(8, 2, 48, 32), (6, 3, 40, 24), (4, 4, 128, 128), (5, 1, 96, 64), (2, 1, 16, 40), (3, 3, 200, 160),
+SHAPES = [(10, 2, 56, 40), (6, 3, 40, 24), (4, 4, 128, 128), (5, 1, 96, 64), (2, 1, 16, 40), (3, 3, 200, 160),
           (16, 1, 64, 96), (34, 2, 32, 32), (12, 4, 80, 100), (7, 7, 256, 256)]
 
 
