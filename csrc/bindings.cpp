@@ -102,7 +102,7 @@ void tile_rows(const at::Tensor& x, at::Tensor& xt) {
   RC(oamd::tile_rows(ptr<bf16_t>(x), ptr<bf16_t>(xt), (int)x.size(0), (int)x.size(1), cur_stream()));
 }
 
-void silu_mul(const at::Tensor& gu, at::Tensor& out, int64_t block) {
+void silu_mul(const at::Tensor& gu, at::Tensor& out, int64_t block, int64_t glu) {
   CHECK_DEV(gu); CHECK_BF16(gu); CHECK_BF16(out); ROWMAJOR_VEC(gu); ROWMAJOR_VEC(out);
   const int64_t rows = gu.size(0), inter = out.size(1);
   TORCH_CHECK(gu.size(1) == 2 * inter && out.size(0) == rows && inter % 8 == 0, "silu_mul shape mismatch");
@@ -110,7 +110,7 @@ void silu_mul(const at::Tensor& gu, at::Tensor& out, int64_t block) {
   TORCH_CHECK(block % 8 == 0 && inter % block == 0, "silu_mul: interleave block must divide inter, % 8");
   const c10::hip::HIPGuardMasqueradingAsCUDA g(gu.device());
   RC(oamd::silu_mul(ptr<bf16_t>(gu), ptr<bf16_t>(out), rows, (int)inter, (int)block, gu.stride(0), out.stride(0),
-                    cur_stream()));
+                    (int)glu, cur_stream()));
 }
 
 void embedding(const at::Tensor& ids, const at::Tensor& table, at::Tensor& out) {
@@ -212,9 +212,10 @@ void rope_kv(const at::Tensor& qkv, const at::Tensor& pos, const at::Tensor& cos
                    xp, (int)splits, optr<bf16_t>(bias), fp8, (float)k_scale, (float)v_scale, cur_stream()));
 }
 
+// silu_gu of the GEMMs below: 0 = plain product, 1 / 2 = gated feed-forward epilogue with silu / tanh-gelu
 void gemm_decode(const at::Tensor& x, const at::Tensor& w, const c10::optional<at::Tensor>& y_opt,
                  const c10::optional<at::Tensor>& p,
-                 int64_t splits, int64_t bn, int64_t bm, bool silu_gu, bool w_tiled, int64_t stages) {
+                 int64_t splits, int64_t bn, int64_t bm, int64_t silu_gu, bool w_tiled, int64_t stages) {
   CHECK_DEV(x); CHECK_BF16(x); CHECK_BF16(w); CHECK_CONTIG(x); CHECK_CONTIG(w);
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2, "x [M,K], w [N,K]");
   const int64_t M = x.size(0), K = x.size(1), N = w.size(0);
@@ -243,11 +244,11 @@ void gemm_decode(const at::Tensor& x, const at::Tensor& w, const c10::optional<a
   TORCH_CHECK(K < (1LL << 31) / 64 && M * K < (1LL << 31) && N * K < (1LL << 40), "gemm too large");
   const c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
   RC(oamd::gemm_decode(ptr<bf16_t>(x), ptr<bf16_t>(w), yp, pp, (int)M, (int)N, (int)K, (int)splits,
-                       (int)bn, (int)bm, silu_gu, w_tiled, (int)stages, cur_stream()));
+                       (int)bn, (int)bm, (int)silu_gu, w_tiled, (int)stages, cur_stream()));
 }
 
 void gemm_tile(const at::Tensor& x, const at::Tensor& w, const c10::optional<at::Tensor>& y_opt,
-               const c10::optional<at::Tensor>& bias, bool silu_gu, int64_t variant, int64_t splits,
+               const c10::optional<at::Tensor>& bias, int64_t silu_gu, int64_t variant, int64_t splits,
                const c10::optional<at::Tensor>& partial) {
   CHECK_DEV(x); CHECK_BF16(x); CHECK_BF16(w); CHECK_CONTIG(x); CHECK_CONTIG(w);
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2, "x [M,K], w [N,K]");
@@ -286,11 +287,11 @@ void gemm_tile(const at::Tensor& x, const at::Tensor& w, const c10::optional<at:
   TORCH_CHECK(M * K < (1LL << 40) && N * K < (1LL << 40) && M < (1LL << 31) && N < (1LL << 31), "gemm too large");
   const c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
   RC(oamd::gemm_tile(ptr<bf16_t>(x), ptr<bf16_t>(w), yp, optr<bf16_t>(bias), (int)M, (int)N, (int)K, (int)ldy,
-                     silu_gu, (int)variant, (int)splits, pp, cur_stream()));
+                     (int)silu_gu, (int)variant, (int)splits, pp, cur_stream()));
 }
 
 void gemm_pp(const at::Tensor& x, const at::Tensor& w, const c10::optional<at::Tensor>& y_opt,
-             const c10::optional<at::Tensor>& p, int64_t splits, int64_t bm, bool silu_gu, bool nt, bool one_seg,
+             const c10::optional<at::Tensor>& p, int64_t splits, int64_t bm, int64_t silu_gu, bool nt, bool one_seg,
              const c10::optional<at::Tensor>& sk_ws, const c10::optional<at::Tensor>& sk_flags) {
   CHECK_DEV(x); CHECK_BF16(x); CHECK_BF16(w); CHECK_CONTIG(x); CHECK_CONTIG(w);
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.size(1) == x.size(1), "x [M,K], w [N,K]");
@@ -326,12 +327,12 @@ void gemm_pp(const at::Tensor& x, const at::Tensor& w, const c10::optional<at::T
     wsp = sk_ws->data_ptr<float>();
     flp = sk_flags->data_ptr<int>();
   }
-  RC(oamd::gemm_pp(ptr<bf16_t>(x), ptr<bf16_t>(w), yp, pp, (int)M, (int)N, (int)K, (int)splits, (int)bm, silu_gu, nt,
+  RC(oamd::gemm_pp(ptr<bf16_t>(x), ptr<bf16_t>(w), yp, pp, (int)M, (int)N, (int)K, (int)splits, (int)bm, (int)silu_gu, nt,
                    cur_stream(), one_seg, wsp, flp));
 }
 
 void gemm_skinny(const at::Tensor& x, const at::Tensor& w, const c10::optional<at::Tensor>& y_opt,
-                 const c10::optional<at::Tensor>& p, int64_t splits, bool silu_gu) {
+                 const c10::optional<at::Tensor>& p, int64_t splits, int64_t silu_gu) {
   CHECK_DEV(x); CHECK_BF16(x); CHECK_BF16(w); CHECK_CONTIG(x); CHECK_CONTIG(w);
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.size(1) == x.size(1), "x [M,K], w [N,K]");
   const int64_t M = x.size(0), K = x.size(1), N = w.size(0);
@@ -357,7 +358,7 @@ void gemm_skinny(const at::Tensor& x, const at::Tensor& w, const c10::optional<a
   }
   TORCH_CHECK(N * K < (1LL << 40) && M * K < (1LL << 31), "gemm too large");
   const c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
-  RC(oamd::gemm_skinny(ptr<bf16_t>(x), ptr<bf16_t>(w), yp, pp, (int)M, (int)N, (int)K, (int)splits, silu_gu,
+  RC(oamd::gemm_skinny(ptr<bf16_t>(x), ptr<bf16_t>(w), yp, pp, (int)M, (int)N, (int)K, (int)splits, (int)silu_gu,
                        cur_stream()));
 }
 
@@ -586,7 +587,8 @@ PYBIND11_MODULE(_C, m) {
   m.def("gemm_xr", &gemm_xr, pybind11::arg("xt"), pybind11::arg("w"), pybind11::arg("y") = pybind11::none(),
         pybind11::arg("p") = pybind11::none(), pybind11::arg("splits") = 1, pybind11::arg("epi") = 1);
   m.def("tile_rows", &tile_rows, pybind11::arg("x"), pybind11::arg("xt"));
-  m.def("silu_mul", &silu_mul, pybind11::arg("gu"), pybind11::arg("out"), pybind11::arg("block") = 0);
+  m.def("silu_mul", &silu_mul, pybind11::arg("gu"), pybind11::arg("out"), pybind11::arg("block") = 0,
+        pybind11::arg("glu") = 1);
   m.def("embedding", &embedding);
   m.def("rope_kv", &rope_kv, pybind11::arg("qkv"), pybind11::arg("pos"), pybind11::arg("cos"),
         pybind11::arg("sin"), pybind11::arg("Hq"), pybind11::arg("Hkv"), pybind11::arg("q_out"),
@@ -611,18 +613,18 @@ PYBIND11_MODULE(_C, m) {
         pybind11::arg("bn") = 64, pybind11::arg("bm") = 64, pybind11::arg("reduce") = true);
   m.def("gemm_decode", &gemm_decode, pybind11::arg("x"), pybind11::arg("w"), pybind11::arg("y"),
         pybind11::arg("p") = pybind11::none(), pybind11::arg("splits") = 1, pybind11::arg("bn") = 64,
-        pybind11::arg("bm") = 0, pybind11::arg("silu_gu") = false, pybind11::arg("w_tiled") = false,
+        pybind11::arg("bm") = 0, pybind11::arg("silu_gu") = 0, pybind11::arg("w_tiled") = false,
         pybind11::arg("stages") = 3);
   m.def("gemm_tile", &gemm_tile, pybind11::arg("x"), pybind11::arg("w"), pybind11::arg("y"),
-        pybind11::arg("bias") = pybind11::none(), pybind11::arg("silu_gu") = false, pybind11::arg("variant") = 0,
+        pybind11::arg("bias") = pybind11::none(), pybind11::arg("silu_gu") = 0, pybind11::arg("variant") = 0,
         pybind11::arg("splits") = 1, pybind11::arg("partial") = pybind11::none());
   m.def("gemm_pp", &gemm_pp, pybind11::arg("x"), pybind11::arg("w"), pybind11::arg("y"),
         pybind11::arg("p") = pybind11::none(), pybind11::arg("splits") = 1, pybind11::arg("bm") = 256,
-        pybind11::arg("silu_gu") = false, pybind11::arg("nt") = true, pybind11::arg("one_seg") = false,
+        pybind11::arg("silu_gu") = 0, pybind11::arg("nt") = true, pybind11::arg("one_seg") = false,
         pybind11::arg("sk_ws") = pybind11::none(), pybind11::arg("sk_flags") = pybind11::none());
   m.def("gemm_pp_sk_grid", &oamd::gemm_pp_sk_grid, pybind11::arg("tiles"), pybind11::arg("steps"));
   m.def("gemm_skinny", &gemm_skinny, pybind11::arg("x"), pybind11::arg("w"), pybind11::arg("y"),
-        pybind11::arg("p") = pybind11::none(), pybind11::arg("splits") = 1, pybind11::arg("silu_gu") = false);
+        pybind11::arg("p") = pybind11::none(), pybind11::arg("splits") = 1, pybind11::arg("silu_gu") = 0);
   m.def("attn_prefill", &attn_prefill, pybind11::arg("q"), pybind11::arg("k"), pybind11::arg("v"),
         pybind11::arg("o"), pybind11::arg("cu_seqlens"), pybind11::arg("work_seq"), pybind11::arg("work_q0"),
         pybind11::arg("scale"), pybind11::arg("block_q") = 64, pybind11::arg("pk") = pybind11::none(),

@@ -11,7 +11,7 @@
 //                 S left in the registers; a lane's column is one head, so the softmax
 //                 rescale is lane-local
 // The waves are merged through LDS; sequences cut into several splits leave fp32 partials
-// for the combine kernel.
+// for the combine kernel. With a window only the last `window` tokens are read.
 #include "attn_gd.h"
 
 namespace oamd {
@@ -24,10 +24,14 @@ constexpr int kTok = 32;            // tokens per wave chunk
 constexpr int kChunk = 4 * kTok;    // tokens per workgroup round
 constexpr int kMaxPages = 1024;     // page ids of one split staged in LDS
 
-__device__ __forceinline__ int split_tokens(int len, int num_splits) {
+// tokens of one split of `len`, a multiple of `round`
+__device__ __forceinline__ int split_tokens(int len, int num_splits, int round) {
   const int per = (len + num_splits - 1) / num_splits;
-  return (per + kChunk - 1) / kChunk * kChunk;
+  return (per + round - 1) / round * round;
 }
+
+// first token a windowed query reads, down to a whole cache tile
+__device__ __forceinline__ int window_start(int len, int window) { return max(0, len - window) & ~15; }
 
 template <int NK, int NV>
 struct Frag {
@@ -60,11 +64,13 @@ __global__ void __launch_bounds__(256, (NK + NV <= 8) ? 2 : 1) attn_gd_decode_ke
       for (int e = tid; e < nh * a.dvp; e += 256) orow[e] = 0;
     return;
   }
-  const int per = split_tokens(len, a.num_splits);
-  const int start = s * per;
+  const int first = window_start(len, a.window);   // tokens below len - window share its tile and are masked
+  const int per = split_tokens(len - first, a.num_splits, kChunk);
+  const int start = first + s * per;
   if (start >= len) return;
   const int end = min(len, start + per);
-  const int ns_b = (len + per - 1) / per;
+  const int ns_b = (len - first + per - 1) / per;
+  const int lo = len - a.window;
   const int nch = (end - start + kTok - 1) / kTok;
 
   const int page0 = start >> a.log2_page;
@@ -116,7 +122,8 @@ __global__ void __launch_bounds__(256, (NK + NV <= 8) ? 2 : 1) attn_gd_decode_ke
       for (int st = 0; st < NK; ++st) d = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bf8(r.k[i][st]), bf8(qf[st]), d, 0, 0, 0);
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        sc[i][j] = base + 16 * i + 4 * lg + j < end ? d[j] * a.scale_log2 : -INFINITY;
+        const int t = base + 16 * i + 4 * lg + j;
+        sc[i][j] = t < end && t >= lo ? d[j] * a.scale_log2 : -INFINITY;
         mx = fmaxf(mx, sc[i][j]);
       }
     }
@@ -190,6 +197,7 @@ __global__ void __launch_bounds__(256, (NK + NV <= 8) ? 2 : 1) attn_gd_decode_ke
       L += f * mls[ww][h][1];
     }
     if (ns_b == 1) {
+      if (a.gate) o *= a.gate[(int64_t)b * Hq + kvh * a.G + h0 + h];
       orow[e] = f2bf(L > 0.f ? o / L : 0.f);
     } else {
       const int64_t bh = (int64_t)b * Hq + kvh * a.G + h0 + h;
@@ -202,13 +210,14 @@ __global__ void __launch_bounds__(256, (NK + NV <= 8) ? 2 : 1) attn_gd_decode_ke
   }
 }
 
-// Sum the partials of sequences cut into several splits: grid (B, Hq), 64 threads.
-__global__ void __launch_bounds__(64) attn_gd_combine_kernel(const AttnDecode a) {
+// Sum the partials of sequences cut into several splits: grid (B, Hq).
+__global__ void __launch_bounds__(256) attn_gd_combine_kernel(const AttnDecode a, int round) {
   const int b = blockIdx.x, hq = blockIdx.y, Hq = gridDim.y;
   const int len = min(a.seq_lens[b], a.max_pages * a.page_size);
   if (len <= 0) return;
-  const int per = split_tokens(len, a.num_splits);
-  const int ns = (len + per - 1) / per;
+  const int n = len - window_start(len, a.window);
+  const int per = split_tokens(n, a.num_splits, round);
+  const int ns = (n + per - 1) / per;
   if (ns == 1) return;
   const int64_t bh = (int64_t)b * Hq + hq;
   const float* ml = a.ml_part + bh * a.num_splits * 2;
@@ -216,8 +225,9 @@ __global__ void __launch_bounds__(64) attn_gd_combine_kernel(const AttnDecode a)
   for (int s = 0; s < ns; ++s) M = fmaxf(M, ml[2 * s]);
   float L = 0.f;
   for (int s = 0; s < ns; ++s) L += exp2f(ml[2 * s] - M) * ml[2 * s + 1];
-  const float inv = L > 0.f ? 1.f / L : 0.f;
-  for (int d = threadIdx.x; d < a.dvp; d += 64) {
+  float inv = L > 0.f ? 1.f / L : 0.f;
+  if (a.gate) inv *= a.gate[bh];
+  for (int d = threadIdx.x; d < a.dvp; d += blockDim.x) {
     float o = 0.f;
     for (int s = 0; s < ns; ++s) o += exp2f(ml[2 * s] - M) * a.o_part[(bh * a.num_splits + s) * a.dvp + d];
     a.out[b * (int64_t)a.o_ld + hq * a.dvp + d] = f2bf(o * inv);
@@ -240,7 +250,7 @@ static int launch_nv(const AttnDecode& a, int grid, hipStream_t stream) {
 
 int attn_gd_decode(const AttnDecode& a, int B, hipStream_t stream) {
   if (B == 0) return 0;
-  if (a.dkp % 8 || a.dvp % 32 || a.G < 1 || a.page_size % 16 || a.max_pages > kMaxPages || a.num_splits < 1) return -1;
+  if (a.dkp % 8 || a.dvp % 32 || a.G < 1 || a.page_size % 16 || a.max_pages > kMaxPages || a.num_splits < 1 || a.window < 1) return -1;
   const int grid = B * a.num_splits * a.Hkv * ((a.G + 15) / 16);
   int rc = -2;
   switch (dim_bin(a.dkp)) {
@@ -254,10 +264,12 @@ int attn_gd_decode(const AttnDecode& a, int B, hipStream_t stream) {
   }
   if (rc != 0) return rc;
   OAMD_LAUNCH_CHECK();
-  if (a.num_splits > 1) {
-    attn_gd_combine_kernel<<<dim3(B, a.Hkv * a.G), 64, 0, stream>>>(a);
-    OAMD_LAUNCH_CHECK();
-  }
+  return a.num_splits > 1 ? attn_combine(a, B, kChunk, stream) : 0;
+}
+
+int attn_combine(const AttnDecode& a, int B, int round, hipStream_t stream) {
+  attn_gd_combine_kernel<<<dim3(B, a.Hkv * a.G), a.dvp > 128 ? 256 : 64, 0, stream>>>(a, round);
+  OAMD_LAUNCH_CHECK();
   return 0;
 }
 

@@ -12,6 +12,7 @@
 // transposing LDS read. The rescale is deferred (a running maximum is kept until a tile
 // raises it by more than 8 in log2 units).
 // seq_pfx: keys of a shared prompt prefix (rows of pk / pv) come before a sequence's own.
+// window: tiles that no row of the workgroup sees are never loaded.
 #include "attn_gd.h"
 
 namespace oamd {
@@ -72,6 +73,9 @@ __global__ void __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) attn_gd_prefill
   const int pl = a.seq_pfx != nullptr ? a.seq_pfx[seq] : 0;
   const int npt = (pl + BK - 1) / BK;
   const int ntiles = npt + (kend + BK - 1) / BK;
+  // first tile with a key that the first row sees (keys count from the prefix's start)
+  const int lo = pl + q0 - a.window + 1;
+  const int kt0 = lo <= 0 ? 0 : lo < pl ? lo / BK : npt + (lo - pl) / BK;
   const bool active = wave_used && rbase < slen;
   const int wend = min(slen, rbase + 32);   // own keys this wave can see: < wend
 
@@ -122,8 +126,8 @@ __global__ void __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) attn_gd_prefill
     }
   };
 
-  load_tile(0);
-  for (int kt = 0; kt < ntiles; ++kt) {
+  load_tile(kt0);
+  for (int kt = kt0; kt < ntiles; ++kt) {
     const int kb = (kt - npt) * BK;   // own-key coordinates (negative: a prefix tile)
     __syncthreads();
     store_tile();
@@ -148,7 +152,9 @@ __global__ void __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) attn_gd_prefill
     // register i of block b is key kb + 32b + (i&3) + 8(i>>2) + 4h
     const bool ptile = kb < 0;
     const int pend = pl - kt * BK;
-    const bool mask = ptile ? (pend < BK) : ((kb + BK > rbase + 1) || (kb + BK > slen));
+    const int wlo = qrow - a.window - (ptile ? kt * BK - pl : kb);   // tile keys up to here are out of the row's window
+    const bool mask = (ptile ? (pend < BK) : ((kb + BK > rbase + 1) || (kb + BK > slen))) ||
+                      rbase + 31 - a.window >= (ptile ? kt * BK - pl : kb);
     float mx = -INFINITY;
 #pragma unroll
     for (int b = 0; b < 2; ++b)
@@ -157,7 +163,7 @@ __global__ void __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) attn_gd_prefill
         float sv = sacc[b][i] * a.scale_log2;
         if (mask) {
           const int j = 32 * b + (i & 3) + 8 * (i >> 2) + 4 * h;
-          if (ptile ? (j >= pend) : (kb + j > qrow || kb + j >= slen)) sv = -INFINITY;
+          if ((ptile ? (j >= pend) : (kb + j > qrow || kb + j >= slen)) || j <= wlo) sv = -INFINITY;
         }
         sacc[b][i] = sv;
         mx = fmaxf(mx, sv);
@@ -208,7 +214,8 @@ __global__ void __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) attn_gd_prefill
   if (!active) return;
   const float lsum = lpart + __shfl_xor(lpart, 32, kWave);
   if (qrow >= slen) return;
-  const float inv = lsum > 0.f ? 1.f / lsum : 0.f;
+  float inv = lsum > 0.f ? 1.f / lsum : 0.f;
+  if (a.gate) inv *= a.gate[(int64_t)(s0 + qrow) * Hq + hq];
   bf16_t* dst = a.o + (int64_t)(s0 + qrow) * a.o_ld + hq * a.dvp;
   // register i of block dd is dim 32 dd + (i&3) + 8(i>>2) + 4h
 #pragma unroll
@@ -241,7 +248,7 @@ static int launch_dv(const AttnPrefill& a, dim3 grid, hipStream_t stream) {
 
 int attn_gd_prefill(const AttnPrefill& a, int num_work, hipStream_t stream) {
   if (num_work == 0) return 0;
-  if (a.dkp % 8 || a.dvp % 32 || a.G < 1 || a.gc < 1 || a.gc > 4 || a.G % a.gc) return -1;
+  if (a.dkp % 8 || a.dvp % 32 || a.G < 1 || a.gc < 1 || a.gc > 4 || a.G % a.gc || a.window < 1) return -1;
   const int rg = 4 / a.gc, sub = 4 / rg;   // 32 rg rows per workgroup, 128 per work item
   const dim3 grid(num_work, a.Hkv * (a.G / a.gc), sub);
   switch (dim_bin(a.dkp)) {

@@ -43,6 +43,19 @@ __device__ __forceinline__ void rope_pair(float a, float b, float c, float s, fl
   o2 = __builtin_fmaf(b, c, a * s);
 }
 
+// Activation of a gated feed-forward, as gate * sigmoid(gate * (a + c gate^2)): silu (1, 0) and the
+// tanh form of gelu, 0.5 z (1 + tanh(r (z + 0.044715 z^3))) with r = sqrt(2 / pi), which is
+// z * sigmoid(2 r z + 2 r 0.044715 z^3). A kernel argument, so one kernel serves both.
+struct GluAct {
+  float a = 1.f, c = 0.f;
+};
+enum Glu { kGluNone = 0, kGluSilu = 1, kGluGeluTanh = 2 };
+inline GluAct glu_act(int glu) { return glu == kGluGeluTanh ? GluAct{1.5957691216057308f, 0.07135481282924846f} : GluAct{}; }
+
+__device__ __forceinline__ float glu_gate(float z, const GluAct& g) {
+  return z / (1.f + __expf(-z * __builtin_fmaf(g.c, z * z, g.a)));
+}
+
 __device__ __forceinline__ uint32_t pack_bf2(float lo, float hi) {
   return static_cast<uint32_t>(f2bf(lo)) | (static_cast<uint32_t>(f2bf(hi)) << 16);
 }

@@ -14,7 +14,8 @@ namespace oamd {
 template <bool SILU>
 __global__ void __launch_bounds__(256) gemm_f32_kernel(const float* __restrict__ X, const float* __restrict__ W,
                                                        float* __restrict__ Y, int M, int N, int K, int ldy,
-                                                       const int* __restrict__ gtab, const float* __restrict__ rscale) {
+                                                       const int* __restrict__ gtab, const float* __restrict__ rscale,
+                                                       GluAct act, int64_t ldx, int64_t xh, int64_t yh) {
   constexpr int NB = SILU ? 2 : 1;
   __shared__ float xs[16][64 + 4];
   __shared__ float ws[NB][16][64 + 4];
@@ -23,6 +24,11 @@ __global__ void __launch_bounds__(256) gemm_f32_kernel(const float* __restrict__
     if ((int)blockIdx.x >= gtab[0]) return;
     W += (int64_t)gtab[1 + blockIdx.x] * N * K;
   }
+  if (blockIdx.z) {   // one product per head
+    X += blockIdx.z * xh;
+    W += (int64_t)blockIdx.z * N * K;
+    Y += blockIdx.z * yh;
+  }
   const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
   const int lr = tid >> 2, lk = (tid & 3) * 4;   // loader: row, 4 consecutive k
   float acc[NB][4][4] = {};
@@ -30,7 +36,7 @@ __global__ void __launch_bounds__(256) gemm_f32_kernel(const float* __restrict__
     __syncthreads();
     {
       f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
-      if (m0 + lr < M) v = *reinterpret_cast<const f32x4*>(X + (int64_t)(m0 + lr) * K + k0 + lk);
+      if (m0 + lr < M) v = *reinterpret_cast<const f32x4*>(X + (int64_t)(m0 + lr) * ldx + k0 + lk);
 #pragma unroll
       for (int j = 0; j < 4; ++j) xs[lk + j][lr] = v[j];
     }
@@ -70,34 +76,44 @@ __global__ void __launch_bounds__(256) gemm_f32_kernel(const float* __restrict__
       float y = acc[0][i][j];
       if constexpr (SILU) {
         const float g = c * y, u = c * acc[NB - 1][i][j];
-        y = g / (1.f + expf(-g)) * u;
+        y = g / (1.f + expf(-g * __builtin_fmaf(act.c, g * g, act.a))) * u;
       }
       Y[(int64_t)m * ldy + n] = y;
     }
   }
 }
 
-int gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, int ldy, bool silu_gu, const int* gtab,
+int gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, int ldy, int glu, const int* gtab,
              const float* rscale, hipStream_t stream) {
   if (M == 0) return 0;
-  if (K % 16 || (silu_gu && N % 128)) return -1;
-  const int nf = silu_gu ? N / 2 : N;
+  if (K % 16 || (glu && N % 128)) return -1;
+  const int nf = glu ? N / 2 : N;
   const dim3 grid((M + 63) / 64, (nf + 63) / 64);
-  if (silu_gu) gemm_f32_kernel<true><<<grid, 256, 0, stream>>>(X, W, Y, M, N, K, ldy, gtab, rscale);
-  else gemm_f32_kernel<false><<<grid, 256, 0, stream>>>(X, W, Y, M, N, K, ldy, gtab, rscale);
+  if (glu) gemm_f32_kernel<true><<<grid, 256, 0, stream>>>(X, W, Y, M, N, K, ldy, gtab, rscale, glu_act(glu), K, 0, 0);
+  else gemm_f32_kernel<false><<<grid, 256, 0, stream>>>(X, W, Y, M, N, K, ldy, gtab, rscale, GluAct{}, K, 0, 0);
+  OAMD_LAUNCH_CHECK();
+  return 0;
+}
+
+int head_gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, int H, int64_t ldx, int64_t xh,
+                  int64_t ldy, int64_t yh, hipStream_t stream) {
+  if (M == 0) return 0;
+  if (K % 16 || ldx % 4 || xh % 4 || H < 1 || H > 65535) return -1;
+  const dim3 grid((M + 63) / 64, (N + 63) / 64, H);
+  gemm_f32_kernel<false><<<grid, 256, 0, stream>>>(X, W, Y, M, N, K, (int)ldy, nullptr, nullptr, GluAct{}, ldx, xh, yh);
   OAMD_LAUNCH_CHECK();
   return 0;
 }
 
 // Attention of one query row and head per workgroup; each of the 4 waves takes every fourth
-// 64-key block (a key per lane), then owns output dims lane, lane + 64, ...
+// 64-key block (a key per lane), then owns NE output dims lane, lane + 64, ...
 // PAGED: row b's keys come from the paged cache (token rows); else from packed k / v rows of
 // the sequence holding the row, after the shared-prefix rows.
-template <bool PAGED>
+template <bool PAGED, int NE>
 __global__ void __launch_bounds__(256) attn_f32_kernel(const AttnF32 a) {
-  __shared__ float qs[256];
+  __shared__ float qs[64 * NE];
   __shared__ float ps[4][64];
-  __shared__ float red[4][256];
+  __shared__ float red[4][64 * NE];
   __shared__ float mls[4][2];
   const int t = blockIdx.x, hq = blockIdx.y, kvh = hq / (gridDim.y / a.Hkv);
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
@@ -124,8 +140,8 @@ __global__ void __launch_bounds__(256) attn_f32_kernel(const AttnF32 a) {
   auto key = [&](int j, const float*& kp, const float*& vp) {
     if constexpr (PAGED) {
       const int64_t r = ((int64_t)a.block_tables[(int64_t)t * a.max_pages + j / a.page_size] * a.Hkv + kvh) * a.page_size + j % a.page_size;
-      kp = a.k + r * a.dkp;
-      vp = a.v + r * a.dvp;
+      kp = a.k + r * a.k_ld;
+      vp = a.v + r * a.v_ld;
     } else {
       const int64_t r = j < pl ? j : base + j - pl;
       kp = (j < pl ? a.pk : a.k) + (r * a.Hkv + kvh) * a.dkp;
@@ -133,8 +149,9 @@ __global__ void __launch_bounds__(256) attn_f32_kernel(const AttnF32 a) {
     }
   };
   float m = -1e30f, l = 0.f;
-  float acc[4] = {0.f, 0.f, 0.f, 0.f};
-  for (int j0 = w * 64; j0 < n; j0 += 256) {
+  float acc[NE] = {};
+  const int lo = max(0, n - a.window);   // first key in the window
+  for (int j0 = lo + w * 64; j0 < n; j0 += 256) {
     const int j = j0 + lane;
     float s = -INFINITY;
     if (j < n) {
@@ -158,13 +175,13 @@ __global__ void __launch_bounds__(256) attn_f32_kernel(const AttnF32 a) {
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 #pragma unroll
-    for (int e = 0; e < 4; ++e) acc[e] *= alpha;
+    for (int e = 0; e < NE; ++e) acc[e] *= alpha;
     const int cnt = min(64, n - j0);
     for (int i = 0; i < cnt; ++i) {
       const float *kp, *vp;
       key(j0 + i, kp, vp);
 #pragma unroll
-      for (int e = 0; e < 4; ++e)
+      for (int e = 0; e < NE; ++e)
         if (lane + 64 * e < a.dvp) acc[e] = __builtin_fmaf(ps[w][i], vp[lane + 64 * e], acc[e]);
     }
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
@@ -172,7 +189,7 @@ __global__ void __launch_bounds__(256) attn_f32_kernel(const AttnF32 a) {
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   }
 #pragma unroll
-  for (int e = 0; e < 4; ++e) red[w][lane + 64 * e] = acc[e];
+  for (int e = 0; e < NE; ++e) red[w][lane + 64 * e] = acc[e];
   if (lane == 0) {
     mls[w][0] = m;
     mls[w][1] = l;
@@ -187,15 +204,17 @@ __global__ void __launch_bounds__(256) attn_f32_kernel(const AttnF32 a) {
       o += f * red[ww][d];
       L += f * mls[ww][1];
     }
-    out[d] = o / L;
+    out[d] = a.gate ? o / L * a.gate[(int64_t)t * gridDim.y + hq] : o / L;
   }
 }
 
 int attn_f32(const AttnF32& a, int rows, int Hq, bool paged, hipStream_t stream) {
   if (rows == 0) return 0;
-  if (a.dkp % 4 || a.dkp > 256 || a.dvp > 256 || Hq % a.Hkv) return -1;
-  if (paged) attn_f32_kernel<true><<<dim3(rows, Hq), 256, 0, stream>>>(a);
-  else attn_f32_kernel<false><<<dim3(rows, Hq), 256, 0, stream>>>(a);
+  const int top = a.dkp > a.dvp ? a.dkp : a.dvp;
+  if (a.dkp % 4 || top > (paged ? 640 : 256) || Hq % a.Hkv || a.window < 1) return -1;
+  if (paged && top > 256) attn_f32_kernel<true, 10><<<dim3(rows, Hq), 256, 0, stream>>>(a);
+  else if (paged) attn_f32_kernel<true, 4><<<dim3(rows, Hq), 256, 0, stream>>>(a);
+  else attn_f32_kernel<false, 4><<<dim3(rows, Hq), 256, 0, stream>>>(a);
   OAMD_LAUNCH_CHECK();
   return 0;
 }

@@ -75,7 +75,7 @@ __global__ void __launch_bounds__(kWaves * 64, NS == 2 ? 2 : 1) gemm_tn_kernel(c
                                                                  float* __restrict__ P, int M, int N, int K, int S,
                                                                  int w_tiled, const int* __restrict__ gtab = nullptr,
                                                                  const int* __restrict__ src = nullptr,
-                                                                 const float* __restrict__ rscale = nullptr) {
+                                                                 const float* __restrict__ rscale = nullptr, GluAct act = {}) {
   using C = GemmCfg<BM, BN, NS>;
   __shared__ __attribute__((aligned(1024))) char lds[C::LDS_BYTES];
   const int tid = threadIdx.x, lane = tid & 63;
@@ -224,7 +224,7 @@ __global__ void __launch_bounds__(kWaves * 64, NS == 2 ? 2 : 1) gemm_tn_kernel(c
       for (int e = 0; e < 8; ++e) {
         const float g = bf2f(f2bf(GRP ? c * cr[f0 + e] : cr[f0 + e]));
         const float u = bf2f(f2bf(GRP ? c * cr[64 + f0 + e] : cr[64 + f0 + e]));
-        const float sg = bf2f(f2bf(g / (1.f + __expf(-g))));
+        const float sg = bf2f(f2bf(glu_gate(g, act)));
         o[e] = f2bf(sg * u);
       }
       *reinterpret_cast<u16x8*>(Y + (int64_t)(m0 + row) * NO + nt * 64 + f0) = o;
@@ -285,26 +285,26 @@ int moe_gemm_rows(const bf16_t* X, const bf16_t* W, bf16_t* Y, int max_rows, int
 }
 
 int gemm_decode(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, int BN,
-                int BM, bool silu_gu, bool w_tiled_b, int stages, hipStream_t stream) {
+                int BM, int glu, bool w_tiled_b, int stages, hipStream_t stream) {
   // bit 0: tiled W layout; bit 1: W streams with the non-temporal policy (OAMD_BF16_WNT)
   static const int wnt = [] { const char* e = getenv("OAMD_BF16_WNT"); return e && e[0] == '0' ? 0 : 2; }();
   const int w_tiled = (w_tiled_b ? 1 : 0) | wnt;
   if (w_tiled_b && (N % 64 != 0 || K % 64 != 0)) return -6;
   if ((BM != 64 && BM != 128 && BM != 256) || M % BM != 0) return -1;
-  if (silu_gu) {  // fused SwiGLU: one K slice, 128-column tiles of 64 gate + 64 up rows
+  if (glu) {  // fused SwiGLU: one K slice, 128-column tiles of 64 gate + 64 up rows
     if (BN != 128 || S != 1 || N % 128 != 0 || K % kBK != 0) return -5;
     const dim3 grid(N / 128, M / BM);
     switch (BM) {
       case 64:
-        if (stages == 2) gemm_tn_kernel<64, 128, kEpiSiluGU, 2><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled);
-        else if (stages == 4) gemm_tn_kernel<64, 128, kEpiSiluGU, 4><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled);
-        else gemm_tn_kernel<64, 128, kEpiSiluGU><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled);
+        if (stages == 2) gemm_tn_kernel<64, 128, kEpiSiluGU, 2><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled, nullptr, nullptr, nullptr, glu_act(glu));
+        else if (stages == 4) gemm_tn_kernel<64, 128, kEpiSiluGU, 4><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled, nullptr, nullptr, nullptr, glu_act(glu));
+        else gemm_tn_kernel<64, 128, kEpiSiluGU><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled, nullptr, nullptr, nullptr, glu_act(glu));
         break;
       case 128:
-        if (stages == 4) gemm_tn_kernel<128, 128, kEpiSiluGU, 4><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled);
-        else gemm_tn_kernel<128, 128, kEpiSiluGU><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled);
+        if (stages == 4) gemm_tn_kernel<128, 128, kEpiSiluGU, 4><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled, nullptr, nullptr, nullptr, glu_act(glu));
+        else gemm_tn_kernel<128, 128, kEpiSiluGU><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled, nullptr, nullptr, nullptr, glu_act(glu));
         break;
-      default: gemm_tn_kernel<256, 128, kEpiSiluGU><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled); break;
+      default: gemm_tn_kernel<256, 128, kEpiSiluGU><<<grid, kWaves * 64, 0, stream>>>(X, W, Y, P, M, N, K, 1, w_tiled, nullptr, nullptr, nullptr, glu_act(glu)); break;
     }
     OAMD_LAUNCH_CHECK();
     return 0;

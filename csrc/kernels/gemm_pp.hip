@@ -68,7 +68,8 @@ __device__ __forceinline__ uint2 pack4(f32x4 v) { return make_uint2(pack_bf2(v[0
 template <int XH, int EPI, bool NT, bool ONE = false, bool SK = false>
 __global__ void __launch_bounds__(512) gemm_pp_kernel(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W,
                                                       bf16_t* __restrict__ Y, float* __restrict__ P, int M, int N,
-                                                      int K, float* __restrict__ ws, int* __restrict__ flags) {
+                                                      int K, float* __restrict__ ws, int* __restrict__ flags,
+                                                      GluAct act = {}) {
   constexpr int NR = XH + 1;               // regions per K-tile
   constexpr int BUF = NR * kRegion;
   constexpr int GL = 2;                    // DMA instructions per wave per region
@@ -227,7 +228,7 @@ __global__ void __launch_bounds__(512) gemm_pp_kernel(const bf16_t* __restrict__
           for (int r = 0; r < 4; ++r) {
             const float gg = bf2f(f2bf(gt[r]));
             const float uu = bf2f(f2bf(up[r]));
-            o[r] = bf2f(f2bf(gg / (1.f + __expf(-gg)))) * uu;
+            o[r] = bf2f(f2bf(glu_gate(gg, act))) * uu;
           }
           *reinterpret_cast<uint2*>(Y + (int64_t)tok * (N >> 1) + col) = pack4(o);
         } else {
@@ -418,33 +419,34 @@ int gemm_pp_sk_grid(int tiles, int steps) {
   return G;
 }
 
-int gemm_pp(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, int bm, bool silu_gu,
+int gemm_pp(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, int bm, int glu,
             bool nt, hipStream_t stream, bool one_seg, float* ws, int* flags) {
   if (M < 1 || N % 128 != 0 || S < 1 || S > 32 || K % (kBK * S) != 0) return -1;
   if (bm != 128 && bm != 256) return -2;
-  if (silu_gu && S != 1) return -3;
+  if (glu && S != 1) return -3;
   if (S > 1 && P == nullptr) return -4;
   if (S == 1 && Y == nullptr) return -5;
   const dim3 grid(N / 128, S, (M + bm - 1) / bm);
-  const int epi = silu_gu ? kSilu : (S > 1 ? kPartial : kStore);
+  const GluAct act = glu_act(glu);
+  const int epi = glu ? kSilu : (S > 1 ? kPartial : kStore);
   // stream-K: 256-row tile (M <= 256), one K slice, workspace ((N / 128) x 128 KiB fp32) and
   // zeroed flags (N / 128 ints; the kernel leaves them zero) given
   const int skg = (ws != nullptr && flags != nullptr && bm == 256 && M <= 256 && S == 1 && !one_seg && nt)
                       ? gemm_pp_sk_grid(N / 128, K / kBK) : 0;
   if (skg > 0) {
     if (epi == kSilu)
-      gemm_pp_kernel<2, kSilu, true, false, true><<<skg, 512, 0, stream>>>(X, W, Y, P, M, N, K, ws, flags);
+      gemm_pp_kernel<2, kSilu, true, false, true><<<skg, 512, 0, stream>>>(X, W, Y, P, M, N, K, ws, flags, act);
     else
-      gemm_pp_kernel<2, kStore, true, false, true><<<skg, 512, 0, stream>>>(X, W, Y, P, M, N, K, ws, flags);
+      gemm_pp_kernel<2, kStore, true, false, true><<<skg, 512, 0, stream>>>(X, W, Y, P, M, N, K, ws, flags, act);
     OAMD_LAUNCH_CHECK();
     return 0;
   }
-#define OAMD_PP(XH, E, NTB) gemm_pp_kernel<XH, E, NTB><<<grid, 512, 0, stream>>>(X, W, Y, P, M, N, K, nullptr, nullptr)
+#define OAMD_PP(XH, E, NTB) gemm_pp_kernel<XH, E, NTB><<<grid, 512, 0, stream>>>(X, W, Y, P, M, N, K, nullptr, nullptr, act)
 #define OAMD_PP_E(XH, NTB)                  \
   if (epi == kSilu) OAMD_PP(XH, kSilu, NTB); \
   else if (epi == kPartial) OAMD_PP(XH, kPartial, NTB); \
   else OAMD_PP(XH, kStore, NTB)
-#define OAMD_PP1(E) gemm_pp_kernel<2, E, true, true><<<grid, 512, 0, stream>>>(X, W, Y, P, M, N, K, nullptr, nullptr)
+#define OAMD_PP1(E) gemm_pp_kernel<2, E, true, true><<<grid, 512, 0, stream>>>(X, W, Y, P, M, N, K, nullptr, nullptr, act)
   if (bm == 256 && one_seg) {   // one barrier segment per K-tile (nt weights)
     if (epi == kSilu) OAMD_PP1(kSilu);
     else if (epi == kPartial) OAMD_PP1(kPartial);

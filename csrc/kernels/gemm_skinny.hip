@@ -38,7 +38,7 @@ template <int NT, int MT, int EPI>
 __global__ void __launch_bounds__(sk::kThreads) gemm_skinny_kernel(const bf16_t* __restrict__ X,
                                                                  const bf16_t* __restrict__ W,
                                                                  bf16_t* __restrict__ Y, float* __restrict__ P,
-                                                                 int M, int N, int K, int S) {
+                                                                 int M, int N, int K, int S, GluAct act = {}) {
   __shared__ float red[sk::kWaves][NT * MT][64 * 4];
   const int tid = threadIdx.x, lane = tid & 63;
   const int w = tid >> 6;
@@ -134,7 +134,7 @@ __global__ void __launch_bounds__(sk::kThreads) gemm_skinny_kernel(const bf16_t*
     if constexpr (EPI == sk::kSilu) {
       const float g = bf2f(f2bf(v[0]));
       const float u = bf2f(f2bf(v[NT - 1]));
-      const float sg = bf2f(f2bf(g / (1.f + __expf(-g))));
+      const float sg = bf2f(f2bf(glu_gate(g, act)));
       const int f = (blockIdx.x >> 2) * 64 + (blockIdx.x & 3) * 16 + rr;
       Y[(int64_t)m * (N / 2) + f] = f2bf(sg * u);
     } else if constexpr (EPI == sk::kPartial) {
@@ -145,18 +145,18 @@ __global__ void __launch_bounds__(sk::kThreads) gemm_skinny_kernel(const bf16_t*
   }
 }
 
-int gemm_skinny(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, bool silu_gu,
+int gemm_skinny(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, int glu,
                 hipStream_t stream) {
   if (M < 1 || M > 32) return -1;
   if (S < 1 || S > 8 || K % (S * sk::kWaves * 32) != 0) return -2;
-  if (silu_gu && (S != 1 || N % 128 != 0)) return -3;
+  if (glu && (S != 1 || N % 128 != 0)) return -3;
   if (N % 16 != 0) return -4;
   if (S > 1 && P == nullptr) return -5;
   const int MT = M <= 16 ? 1 : 2;
-  if (silu_gu) {
+  if (glu) {
     const dim3 grid(N / 32, 1);  // one block per (16 gate rows, 16 up rows)
-    if (MT == 1) gemm_skinny_kernel<2, 1, sk::kSilu><<<grid, sk::kThreads, 0, stream>>>(X, W, Y, P, M, N, K, 1);
-    else gemm_skinny_kernel<2, 2, sk::kSilu><<<grid, sk::kThreads, 0, stream>>>(X, W, Y, P, M, N, K, 1);
+    if (MT == 1) gemm_skinny_kernel<2, 1, sk::kSilu><<<grid, sk::kThreads, 0, stream>>>(X, W, Y, P, M, N, K, 1, glu_act(glu));
+    else gemm_skinny_kernel<2, 2, sk::kSilu><<<grid, sk::kThreads, 0, stream>>>(X, W, Y, P, M, N, K, 1, glu_act(glu));
   } else {
     const dim3 grid(N / 16, S);
     if (S > 1) {

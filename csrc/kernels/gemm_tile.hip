@@ -68,7 +68,8 @@ __device__ __forceinline__ uint2 pack4(f32x4 v) {
 template <int EPI, bool PH2 = false>
 __global__ void __launch_bounds__(512) gemm_tile256_kernel(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W,
                                                            bf16_t* __restrict__ Y, const bf16_t* __restrict__ bias,
-                                                           int M, int N, int K, int ldy, float* __restrict__ P) {
+                                                           int M, int N, int K, int ldy, float* __restrict__ P,
+                                                           GluAct act = {}) {
   __shared__ __attribute__((aligned(1024))) char lds[2 * kBuf];
   const int tid = threadIdx.x, lane = tid & 63;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -269,7 +270,7 @@ __global__ void __launch_bounds__(512) gemm_tile256_kernel(const bf16_t* __restr
           for (int r = 0; r < 4; ++r) {
             const float gg = bf2f(f2bf(gt[r]));
             const float uu = bf2f(f2bf(up[r]));
-            const float sg = bf2f(f2bf(gg / (1.f + __expf(-gg))));
+            const float sg = bf2f(f2bf(glu_gate(gg, act)));
             o[r] = sg * uu;
           }
           *reinterpret_cast<uint2*>(yrow + col) = pack4(o);
@@ -327,7 +328,7 @@ template <int EPI, int AUX = 16, bool COLS = false>
 __global__ void __launch_bounds__(256) gemm_tile256_h4_kernel(const bf16_t* __restrict__ X,
                                                               const bf16_t* __restrict__ W, bf16_t* __restrict__ Y,
                                                               const bf16_t* __restrict__ bias, int M, int N, int K,
-                                                              int ldy) {
+                                                              int ldy, GluAct act = {}) {
   constexpr int kHalf = 32768;       // one operand of a tile: 256 rows x 128 B
   constexpr int kTile = 2 * kHalf;   // X then W
   __shared__ __attribute__((aligned(1024))) char lds[2 * kTile];
@@ -501,7 +502,7 @@ __global__ void __launch_bounds__(256) gemm_tile256_h4_kernel(const bf16_t* __re
           for (int r = 0; r < 4; ++r) {
             const float gg = bf2f(f2bf(gt[r]));
             const float uu = bf2f(f2bf(up[r]));
-            const float sg = bf2f(f2bf(gg / (1.f + __expf(-gg))));
+            const float sg = bf2f(f2bf(glu_gate(gg, act)));
             o[r] = sg * uu;
           }
           *reinterpret_cast<uint2*>(yrow + col) = pack4(o);
@@ -565,7 +566,7 @@ __global__ void __launch_bounds__(256) gemm_tile256_p5_kernel(const bf16_t* __re
                                                               const bf16_t* __restrict__ bias, int M, int N, int K,
                                                               int ldy, int group_m,
                                                               const int* __restrict__ gtab = nullptr,
-                                                              const float* __restrict__ rscale = nullptr) {
+                                                              const float* __restrict__ rscale = nullptr, GluAct act = {}) {
   constexpr int AUX = 16;
   constexpr int kHalf = 32768;   // one operand of a K-step: 256 rows x 128 B
   __shared__ __attribute__((aligned(1024))) char lds[DEEP ? 5 * kHalf : 4 * kHalf];
@@ -854,7 +855,7 @@ __global__ void __launch_bounds__(256) gemm_tile256_p5_kernel(const bf16_t* __re
             for (int rr = 0; rr < 4; ++rr) {
               const float gg = bf2f(f2bf(gt[rr]));
               const float uu = bf2f(f2bf(up[rr]));
-              const float sg = bf2f(f2bf(gg / (1.f + __expf(-gg))));
+              const float sg = bf2f(f2bf(glu_gate(gg, act)));
               o[jj][rr] = sg * uu;
             }
           }
@@ -890,7 +891,7 @@ __global__ void __launch_bounds__(256) gemm_tile256_p5_kernel(const bf16_t* __re
 // blocks): g = bf16(sum_s P[s][m][128 b + j]), u = bf16(sum_s P[s][m][128 b + 64 + j]),
 // y = bf16(bf16(silu(g)) * u) — the numerics of the fused epilogue. 4 features per thread.
 __global__ void splitk_silu_reduce_kernel(const float* __restrict__ P, bf16_t* __restrict__ Y, int M, int N, int S,
-                                          int ldy) {
+                                          int ldy, GluAct act) {
   const int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * 4;
   const int NO = N / 2;
   if (i >= (int64_t)M * NO) return;
@@ -908,23 +909,23 @@ __global__ void splitk_silu_reduce_kernel(const float* __restrict__ P, bf16_t* _
   for (int r = 0; r < 4; ++r) {
     const float gg = bf2f(f2bf(g[r]));
     const float uu = bf2f(f2bf(u[r]));
-    o[r] = bf2f(f2bf(gg / (1.f + __expf(-gg)))) * uu;
+    o[r] = bf2f(f2bf(glu_gate(gg, act))) * uu;
   }
   *reinterpret_cast<uint2*>(Y + (int64_t)m * ldy + f) = pack4(o);
 }
 
-int splitk_silu(const float* P, bf16_t* Y, int M, int N, int S, hipStream_t stream) {
+int splitk_silu(const float* P, bf16_t* Y, int M, int N, int S, int glu, hipStream_t stream) {
   if (M < 1 || N % 128 != 0 || S < 1) return -1;
   const int64_t threads = (int64_t)M * (N / 2) / 4;
-  splitk_silu_reduce_kernel<<<(threads + 255) / 256, 256, 0, stream>>>(P, Y, M, N, S, N / 2);
+  splitk_silu_reduce_kernel<<<(threads + 255) / 256, 256, 0, stream>>>(P, Y, M, N, S, N / 2, glu_act(glu));
   OAMD_LAUNCH_CHECK();
   return 0;
 }
 
 template <int DEEP>
 static void launch_p5(const bf16_t* X, const bf16_t* W, bf16_t* Y, const bf16_t* bias, int M, int N, int K, int ldy,
-                      bool silu_gu, int grid, hipStream_t stream, int gm = kGroupM) {
-  if (silu_gu) gemm_tile256_p5_kernel<kEpiSilu, DEEP><<<grid, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, gm);
+                      int glu, int grid, hipStream_t stream, int gm = kGroupM) {
+  if (glu) gemm_tile256_p5_kernel<kEpiSilu, DEEP><<<grid, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, gm, nullptr, nullptr, glu_act(glu));
   else if (bias) gemm_tile256_p5_kernel<kEpiBias, DEEP><<<grid, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, gm);
   else gemm_tile256_p5_kernel<kEpiStore, DEEP><<<grid, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, gm);
 }
@@ -957,20 +958,20 @@ int moe_gemm_tile(const bf16_t* X, const bf16_t* W, bf16_t* Y, int max_rows, int
 }
 
 int gemm_tile(const bf16_t* X, const bf16_t* W, bf16_t* Y, const bf16_t* bias, int M, int N, int K, int ldy,
-              bool silu_gu, int variant, int S, float* P, hipStream_t stream) {
+              int glu, int variant, int S, float* P, hipStream_t stream) {
   if (M < 1 || N < 16 || N % 16 != 0 || K < kBK || K % kBK != 0) return -1;
-  if (silu_gu && (N % 128 != 0 || bias != nullptr)) return -2;
-  if (Y != nullptr && ldy < (silu_gu ? N / 2 : N)) return -3;
+  if (glu && (N % 128 != 0 || bias != nullptr)) return -2;
+  if (Y != nullptr && ldy < (glu ? N / 2 : N)) return -3;
   if (S < 1 || S > 64 || K % (kBK * S) != 0 || (S > 1 && (P == nullptr || bias != nullptr))) return -5;
-  if (Y == nullptr && (S == 1 || silu_gu)) return -6;
+  if (Y == nullptr && (S == 1 || glu)) return -6;
   const int nwg = ((M + kT - 1) / kT) * ((N + kT - 1) / kT);
   if (S > 1) {   // fp32 slabs, then (unless the consumer sums them) one reduce pass
     gemm_tile256_kernel<kEpiPartial><<<dim3(nwg, S), 512, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, P);
     OAMD_LAUNCH_CHECK();
     if (Y == nullptr) return 0;
-    if (silu_gu) {
+    if (glu) {
       const int64_t threads = (int64_t)M * (N / 2) / 4;
-      splitk_silu_reduce_kernel<<<(threads + 255) / 256, 256, 0, stream>>>(P, Y, M, N, S, ldy);
+      splitk_silu_reduce_kernel<<<(threads + 255) / 256, 256, 0, stream>>>(P, Y, M, N, S, ldy, glu_act(glu));
       OAMD_LAUNCH_CHECK();
       return 0;
     }
@@ -987,36 +988,36 @@ int gemm_tile(const bf16_t* X, const bf16_t* W, bf16_t* Y, const bf16_t* bias, i
     const int grid = min(nwg, device_cus());
     // GROUP_M 4 for the narrow projections (M = 32k, N = 6144: 1106 vs 1145 us at GROUP_M 8; N = 4096
     // equal; 16 / 32 slower: profiles/gemm_tile_p5_vs_hipblaslt_r6.jsonl)
-    if (N >= 16384) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 4);   // GROUP_M 4: -1.1 / -1.4 % at M = 12k / 32k
-    else launch_p5<0>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 4);
+    if (N >= 16384) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 4);   // GROUP_M 4: -1.1 / -1.4 % at M = 12k / 32k
+    else launch_p5<0>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 4);
   } else if (variant >= 6 && variant <= 14 && K >= 2 * kBK && st16) {   // p5 A/B arms (timing, same numerics)
     const int grid = min(nwg, device_cus());
-    if (variant == 6) launch_p5<0>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 4);         // GROUP_M 4
-    else if (variant == 7) launch_p5<0>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 16);   // GROUP_M 16
-    else if (variant == 8) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream);       // W third buffer
-    else if (variant == 10) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 4);   // W third, GROUP_M 4
-    else if (variant == 11) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 16);  // W third, GROUP_M 16
-    else if (variant == 12) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 2);   // W third, GROUP_M 2
-    else if (variant == 13) launch_p5<1>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 4);   // X third, GROUP_M 4
-    else if (variant == 14) launch_p5<0>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 2);   // GROUP_M 2
-    else launch_p5<0>(X, W, Y, bias, M, N, K, ldy, silu_gu, grid, stream, 32);                      // GROUP_M 32
+    if (variant == 6) launch_p5<0>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 4);         // GROUP_M 4
+    else if (variant == 7) launch_p5<0>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 16);   // GROUP_M 16
+    else if (variant == 8) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream);       // W third buffer
+    else if (variant == 10) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 4);   // W third, GROUP_M 4
+    else if (variant == 11) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 16);  // W third, GROUP_M 16
+    else if (variant == 12) launch_p5<2>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 2);   // W third, GROUP_M 2
+    else if (variant == 13) launch_p5<1>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 4);   // X third, GROUP_M 4
+    else if (variant == 14) launch_p5<0>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 2);   // GROUP_M 2
+    else launch_p5<0>(X, W, Y, bias, M, N, K, ldy, glu, grid, stream, 32);                      // GROUP_M 32
   } else if ((variant == 0 || variant == 1) && off32) {   // 4-wave, two 64 KiB buffers, four phases per K-tile
-    if (silu_gu) gemm_tile256_h4_kernel<kEpiSilu><<<nwg, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy);
+    if (glu) gemm_tile256_h4_kernel<kEpiSilu><<<nwg, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, glu_act(glu));
     else if (bias) gemm_tile256_h4_kernel<kEpiBias><<<nwg, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy);
     else gemm_tile256_h4_kernel<kEpiStore><<<nwg, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy);
   } else if (variant == 4 && off32) {   // h4 with W-fragment MFMA groups (timing)
-    if (silu_gu) gemm_tile256_h4_kernel<kEpiSilu, 16, true><<<nwg, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy);
+    if (glu) gemm_tile256_h4_kernel<kEpiSilu, 16, true><<<nwg, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, glu_act(glu));
     else if (bias) gemm_tile256_h4_kernel<kEpiBias, 16, true><<<nwg, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy);
     else gemm_tile256_h4_kernel<kEpiStore, 16, true><<<nwg, 256, 0, stream>>>(X, W, Y, bias, M, N, K, ldy);
   } else if (variant == 2 || (variant == 0 && M > 256)) {
     // 8-wave ping-pong, two barrier segments per K-tile (the round-3 default; 2-8 % behind
     // variant 1 on the prefill shapes, profiles/gemm_tile_h4_vs_ph2_m32k.jsonl); also the
     // fallback for operands past 32-bit offsets
-    if (silu_gu) gemm_tile256_kernel<kEpiSilu, true><<<nwg, 512, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, nullptr);
+    if (glu) gemm_tile256_kernel<kEpiSilu, true><<<nwg, 512, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, nullptr, glu_act(glu));
     else if (bias) gemm_tile256_kernel<kEpiBias, true><<<nwg, 512, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, nullptr);
     else gemm_tile256_kernel<kEpiStore, true><<<nwg, 512, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, nullptr);
   } else {   // 8-wave ping-pong, four segments per K-tile (variant 3, or 0 at M <= 256 past 32-bit offsets)
-    if (silu_gu) gemm_tile256_kernel<kEpiSilu><<<nwg, 512, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, nullptr);
+    if (glu) gemm_tile256_kernel<kEpiSilu><<<nwg, 512, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, nullptr, glu_act(glu));
     else if (bias) gemm_tile256_kernel<kEpiBias><<<nwg, 512, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, nullptr);
     else gemm_tile256_kernel<kEpiStore><<<nwg, 512, 0, stream>>>(X, W, Y, bias, M, N, K, ldy, nullptr);
   }

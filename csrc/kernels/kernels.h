@@ -14,7 +14,7 @@ int rmsnorm(const bf16_t* x, bf16_t* residual, const bf16_t* w, bf16_t* y, int r
             int64_t x_stride, int64_t r_stride, int64_t y_stride, float eps, const float* xp, int S,
             hipStream_t stream);
 int silu_mul(const bf16_t* gu, bf16_t* out, int64_t rows, int inter, int block, int64_t in_stride,
-             int64_t out_stride, hipStream_t stream);
+             int64_t out_stride, int glu, hipStream_t stream);   // glu: Glu of common.h
 // Decode-step bookkeeping (norm_act.hip): cache slots + sampler positions of the step's tokens,
 // then the state advance after sampling (B <= 1024 rows, one workgroup each).
 int decode_slots(const int* bt, const int64_t* pos, const int* ctx, int64_t* slots, int64_t* spos, int B,
@@ -31,21 +31,21 @@ int rope_kv(const bf16_t* qkv, int64_t qkv_stride, const int64_t* pos, const flo
 // Y[M,N] = X[M,K] W[N,K]^T for decode buckets (M a multiple of the BM-row tile, BM in {64,128,256}); S-way split-K
 // (S | 8) with fp32 slabs P[S][M][N] reduced into Y; BN in {64, 128} columns per tile.
 int gemm_decode(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, int BN,
-                int BM, bool silu_gu, bool w_tiled, int stages, hipStream_t stream);
+                int BM, int glu, bool w_tiled, int stages, hipStream_t stream);
 
 // Compute-bound 256x256-tile GEMM (prefill projections, lm_head; gemm_tile.hip): Y[M, N] = X[M,K] W[N,K]^T
-// (+ bias[N]) for any M >= 1, N % 16 == 0, K % 64 == 0; silu_gu: fused SwiGLU over the 64-row interleaved
+// (+ bias[N]) for any M >= 1, N % 16 == 0, K % 64 == 0; glu: fused SwiGLU over the 64-row interleaved
 // gate|up weight (N % 128 == 0), Y [M, N/2]. ldy = Y's row stride in elements.
-// S > 1: S-way split-K into fp32 slabs P[S][M][N], then reduced into Y (SwiGLU applied when silu_gu);
+// S > 1: S-way split-K into fp32 slabs P[S][M][N], then reduced into Y (SwiGLU applied when glu);
 // Y == nullptr leaves the slabs to the consumer (rmsnorm / rope_kv sum them).
 int gemm_tile(const bf16_t* X, const bf16_t* W, bf16_t* Y, const bf16_t* bias, int M, int N, int K, int ldy,
-              bool silu_gu, int variant, int S, float* P, hipStream_t stream);
+              int glu, int variant, int S, float* P, hipStream_t stream);
 // Decode-bucket GEMM on the ping-pong schedule (gemm_pp.hip): Y[M,N] = X[M,K] W[N,K]^T, bm-row tiles
 // (128 / 256), 128-column tiles (N % 128 == 0), S-way split-K slabs P (S > 1; reduced into Y unless Y is
-// nullptr); silu_gu: fused SwiGLU (S == 1), Y [M, N/2]; nt: non-temporal weight loads.
+// nullptr); glu: fused SwiGLU (S == 1), Y [M, N/2]; nt: non-temporal weight loads.
 // ws / flags (both given): the stream-K form for bm 256, S 1, nt (gemm_pp.hip SK): ws >= (N / 128) x 32768
 // floats, flags >= N / 128 ints, zero (left zero). gemm_pp_sk_grid: its block count, 0 = plain launch.
-int gemm_pp(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, int bm, bool silu_gu,
+int gemm_pp(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, int bm, int glu,
             bool nt, hipStream_t stream, bool one_seg = false, float* ws = nullptr, int* flags = nullptr);
 int gemm_pp_sk_grid(int tiles, int steps);
 // 256-row decode GEMM with register-streamed activations (gemm_xr.hip): Xt = X [256, K] in the tiled
@@ -57,12 +57,12 @@ int gemm_xr(const bf16_t* Xt, const bf16_t* W, bf16_t* Y, float* P, int M, int N
 int tile_rows(const bf16_t* x, bf16_t* xt, int rows, int K, hipStream_t stream);
 // Y[M, N] = bf16(sum_s P[s][M][N]) (fp32 split-K slabs).
 int splitk_reduce(const float* P, bf16_t* Y, int64_t MN, int S, hipStream_t stream);
-// Y [M, N/2] = SwiGLU of the summed fp32 slabs [S][M][N] of a 64-row interleaved gate|up projection.
-int splitk_silu(const float* P, bf16_t* Y, int M, int N, int S, hipStream_t stream);
+// Y [M, N/2] = act(gate) * up (glu) of the summed fp32 slabs [S][M][N] of a 64-row interleaved gate|up projection.
+int splitk_silu(const float* P, bf16_t* Y, int M, int N, int S, int glu, hipStream_t stream);
 // Skinny-M decode GEMM (M <= 32, gemm_skinny.hip): N % 16 == 0, K % (128 S) == 0; S-way split-K slabs P
-// reduced into Y (Y == nullptr: left for the consumer); silu_gu: fused SwiGLU over the 64-row
+// reduced into Y (Y == nullptr: left for the consumer); glu: fused SwiGLU over the 64-row
 // interleaved gate|up weight, Y [M, N/2].
-int gemm_skinny(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, bool silu_gu,
+int gemm_skinny(const bf16_t* X, const bf16_t* W, bf16_t* Y, float* P, int M, int N, int K, int S, int glu,
                 hipStream_t stream);
 
 // FP8 e4m3fn W8A8: Y = (X8 . W8^T) * sx[m] * sw[n]; any M (BM-row tiles), S | 8 split-K.
@@ -167,6 +167,7 @@ struct StreamStep {
   int top;                  // 0: none
   const float *mix, *out;   // [S][S], [S] (fp32)
   const float* in;          // [S]
+  const float* post_w;      // [ld] norm weight of the sublayer's own output before it joins (one stream), or nullptr
   const float* w;           // [ld] norm weight (fp32, zero past width)
   void* h;                  // [rows][ld] bf16 or fp32
   float eps;
@@ -212,7 +213,10 @@ struct AttnPrefill {
   float scale_log2;
   const bf16_t *pk, *pv;        // shared-prefix rows and per-sequence prefix lengths, or nullptr
   const int* seq_pfx;
+  int window;                   // a query sees keys less than this far back (kNoWindow: all)
+  const float* gate;            // [T][Hq]: every head's output times its gate, or nullptr
 };
+constexpr int kNoWindow = 1 << 30;
 int attn_gd_prefill(const AttnPrefill& a, int num_work, hipStream_t stream);
 struct AttnDecode {
   const bf16_t* q;              // [B][Hq][dkp]
@@ -223,12 +227,92 @@ struct AttnDecode {
   float *o_part, *ml_part;      // [B][Hq][num_splits][dvp], [..][2] when num_splits > 1
   int Hkv, G, dkp, dvp, page_size, log2_page, max_pages, num_splits;
   float scale_log2;
+  int window;                   // as in AttnPrefill
+  const float* gate;            // [B][Hq] or nullptr
 };
 int attn_gd_decode(const AttnDecode& a, int B, hipStream_t stream);
+// Sums the partials of split sequences (split length a multiple of `round` tokens).
+int attn_combine(const AttnDecode& a, int B, int round, hipStream_t stream);
+// Latent rows (attn_latent_decode.hip): k_cache [pages][P][dkp], values are a row's first rp dims, Hkv = 1,
+// G heads, dvp = rp (out and partials rows), dkp % 64 == 0 in 128..640.
+int attn_latent_decode(const AttnDecode& a, int B, int rp, hipStream_t stream);
+
+// Short-convolution heads (conv_heads.hip)
+struct ConvHeads {
+  const float* xp;          // S fp32 slabs [S][T][ncol], slab elements apart, or nullptr
+  int S;
+  int64_t slab;
+  const void* row;          // [T][ncol] rows (bf16 / fp32): q | k | gate logits
+  int ncol;
+  int taps;                 // 1..8
+  const float* conv;        // [taps][(Hq + Hkv) dkp], last row: the current token's weight
+  const float *qw, *kw;     // [dkp] norm weights, zero past dk
+  const int64_t* pos;
+  int Hq, Hkv, dk, dkp, dvp;
+  float eps;
+  const int* cu_seqlens;    // prefill: [num_seqs + 1], else nullptr
+  int num_seqs;
+  const int* prev_page;     // [num_seqs] page of the tokens before a sequence's first row (-1: none), or nullptr
+  const int* block_tables;  // decode: [T][max_pages], else nullptr
+  int max_pages;
+  void* tails;              // [pages][taps - 1][(Hq + Hkv) dkp]
+  int64_t pages;
+  void *q_out, *k_out, *v_out;   // [T][Hq][dkp], [T][Hkv][dkp], [T][Hkv][dvp] (k_out / v_out may be nullptr)
+  void *k_cache, *v_cache;
+  const int64_t* slots;     // < 0: not kept
+  int log2_page;
+  float* gate;              // [T][Hq] sigmoid gates
+};
+int conv_heads(const ConvHeads& a, int tokens, bool f32, hipStream_t stream);
+
+// Latent attention (latent.hip)
+struct LatentRows {
+  const float* xp;          // as in ConvHeads; columns: query latent qp | latent rp | rotated part rotp | gates
+  int S;
+  int64_t slab;
+  const void* row;
+  int ncol;
+  int q_rank, qp, kv_rank, rp, rot, rotp, ck, H;   // true sizes (the norms' means) and stored ones
+  const float *qw, *cw;     // [qp], [rp] norm weights, zero past the true size
+  float eps;
+  const int64_t* pos;
+  const float *cos_t, *sin_t;   // [max_pos][rot_ld]
+  int rot_ld;
+  int64_t max_pos;
+  void* cq;                 // [T][qp]
+  void* lat;                // [T][ck] c | rotated part | zeros; nullptr: the layer has none of its own
+  void* cache;              // [pages][P][ck] token rows
+  const int64_t* slots;
+  float* gate;              // [T][H]
+};
+int latent_rows(const LatentRows& a, int tokens, bool f32, hipStream_t stream);
+struct RotateHeads {
+  const float* xp;          // S slabs [S][T][H dp] summed into q, or nullptr: q in place
+  int S;
+  int64_t slab;
+  void* q;                  // [T][H][dp]
+  const int64_t* pos;
+  const float *cos_t, *sin_t;
+  int rot_ld;
+  int64_t max_pos;
+  int H, dp, d, rot;        // rotated: columns d .. d + rot of a head
+};
+int rotate_heads(const RotateHeads& a, int tokens, bool f32, hipStream_t stream);
+struct HeadGemm {
+  const bf16_t *X, *W;      // X row m head h at m ldx + h xh; W [H][N][K]
+  bf16_t* Y;
+  int M, N, K, H;
+  int64_t ldx, xh, ldy, yh;
+  int pad, x0, nx;          // pad more columns of Y: X's columns x0 .. x0 + nx, then zeros (pad % 16 == 0)
+};
+int head_gemm(const HeadGemm& a, hipStream_t stream);
 
 // fp32 forms (f32.hip)
-int gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, int ldy, bool silu_gu, const int* gtab,
+int gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, int ldy, int glu, const int* gtab,
              const float* rscale, hipStream_t stream);
+// One product per head: as HeadGemm, without the extra columns.
+int head_gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, int H, int64_t ldx, int64_t xh,
+                  int64_t ldy, int64_t yh, hipStream_t stream);
 struct AttnF32 {
   const float *q, *k, *v;       // k / v: packed rows, or the paged cache (token rows)
   float* o;
@@ -237,9 +321,12 @@ struct AttnF32 {
   int num_seqs;
   const int *block_tables, *seq_lens;   // paged
   int Hkv, dkp, dvp, page_size, max_pages;
+  int64_t k_ld, v_ld;           // elements between the rows of one head's keys / values in k, v
   float scale;
   const float *pk, *pv;
   const int* seq_pfx;
+  int window;                   // as in AttnPrefill
+  const float* gate;            // [rows][Hq] or nullptr
 };
 int attn_f32(const AttnF32& a, int rows, int Hq, bool paged, hipStream_t stream);
 
@@ -257,7 +344,7 @@ int moe_sort(const int* ids, const float* weights, int slots, int top, int E, in
 // xp[row] = h[src[row]] (zeros for padding) for the rows of gtab's tiles; row_bytes % 16 == 0
 int moe_gather(const void* h, const int* src, const int* gtab, int bm, int max_rows, void* xp, int row_bytes,
                hipStream_t stream);
-// Decode: row slot of Y = X row (slot / div) . W[ids[slot]]^T; silu_gu: SwiGLU of weights[slot] * the
+// Decode: row slot of Y = X row (slot / div) . W[ids[slot]]^T; glu: SwiGLU of weights[slot] * the
 // products over the 64-row interleaved gate|up weight. W [E][N][K], K % 64 == 0, N % 16 == 0 (silu: 128).
 int moe_gemm_skinny(const bf16_t* X, const bf16_t* W, bf16_t* Y, const int* ids, const float* weights, int slots,
                     int div, int E, int N, int K, bool silu_gu, hipStream_t stream);

@@ -162,12 +162,12 @@ int rmsnorm(const bf16_t* x, bf16_t* residual, const bf16_t* w, bf16_t* y,
   return 0;
 }
 
-// out[m, i] = silu(gate) * up; grid-stride over 8-element vectors. gate|up
+// out[m, i] = act(gate) * up; grid-stride over 8-element vectors. gate|up
 // columns are interleaved in blocks of `block` features (block == inter: the
 // plain [gate | up] concatenation): gate of feature i at (i / block) * 2 * block
 // + i % block, up `block` columns later.
 __global__ void silu_mul_kernel(const bf16_t* __restrict__ gu, bf16_t* __restrict__ out,
-                                int64_t rows, int inter, int block, int64_t in_stride, int64_t out_stride) {
+                                int64_t rows, int inter, int block, int64_t in_stride, int64_t out_stride, GluAct act) {
   const int vpr = inter >> 3;
   const int64_t total = rows * vpr;
   for (int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; idx < total;
@@ -182,7 +182,7 @@ __global__ void silu_mul_kernel(const bf16_t* __restrict__ gu, bf16_t* __restric
     for (int j = 0; j < 8; ++j) {
       const float gf = bf2f(g[j]);
       // HF: act(gate) rounded to bf16, then multiplied by up in bf16
-      const float s = bf2f(f2bf(gf / (1.f + __expf(-gf))));
+      const float s = bf2f(f2bf(glu_gate(gf, act)));
       o[j] = f2bf(s * bf2f(u[j]));
     }
     *reinterpret_cast<u16x8*>(out + m * out_stride + c) = o;
@@ -190,7 +190,7 @@ __global__ void silu_mul_kernel(const bf16_t* __restrict__ gu, bf16_t* __restric
 }
 
 int silu_mul(const bf16_t* gu, bf16_t* out, int64_t rows, int inter, int block,
-             int64_t in_stride, int64_t out_stride, hipStream_t stream) {
+             int64_t in_stride, int64_t out_stride, int glu, hipStream_t stream) {
   if (rows == 0) return 0;
   if (block <= 0 || block % 8 != 0 || inter % block != 0) return -1;
   const int64_t total = rows * (inter / 8);
@@ -198,7 +198,7 @@ int silu_mul(const bf16_t* gu, bf16_t* out, int64_t rows, int inter, int block,
   int64_t blocks = (total + nt - 1) / nt;
   if (blocks > 256 * 16) blocks = 256 * 16;
   silu_mul_kernel<<<static_cast<int>(blocks), nt, 0, stream>>>(gu, out, rows, inter, block, in_stride,
-                                                               out_stride);
+                                                               out_stride, glu_act(glu));
   OAMD_LAUNCH_CHECK();
   return 0;
 }

@@ -11,42 +11,9 @@
 // [8 dims]; V tile [dvp/32][4 token group][16 dims][2 half][4 token] (dim d = 32 b + 16 half
 // + i). Every MFMA fragment of the decode kernel is then one contiguous 1 KiB wave access.
 // fp32 cache: token rows.
-#include "common.h"
-#include "kernels.h"
+#include "rows.h"
 
 namespace oamd {
-
-namespace {
-
-template <typename T>
-__device__ __forceinline__ void st8(T* p, const float (&v)[8]);
-template <>
-__device__ __forceinline__ void st8<float>(float* p, const float (&v)[8]) {
-  *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
-  *reinterpret_cast<f32x4*>(p + 4) = f32x4{v[4], v[5], v[6], v[7]};
-}
-template <>
-__device__ __forceinline__ void st8<bf16_t>(bf16_t* p, const float (&v)[8]) {
-  *reinterpret_cast<uint4*>(p) =
-      make_uint4(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]), pack_bf2(v[4], v[5]), pack_bf2(v[6], v[7]));
-}
-
-template <typename T>
-__device__ __forceinline__ void ld8(const T* p, float (&v)[8]);
-template <>
-__device__ __forceinline__ void ld8<float>(const float* p, float (&v)[8]) {
-  const f32x4 a = *reinterpret_cast<const f32x4*>(p), b = *reinterpret_cast<const f32x4*>(p + 4);
-#pragma unroll
-  for (int j = 0; j < 4; ++j) v[j] = a[j], v[4 + j] = b[j];
-}
-template <>
-__device__ __forceinline__ void ld8<bf16_t>(const bf16_t* p, float (&v)[8]) {
-  const u16x8 a = *reinterpret_cast<const u16x8*>(p);
-#pragma unroll
-  for (int j = 0; j < 8; ++j) v[j] = bf2f(a[j]);
-}
-
-}  // namespace
 
 // GW lanes (a power of two) share a q / k head, each with CPT chunks of 8 dims (GW * CPT * 8 >= dkp);
 // v is copied in 8-dim items. Grid (tokens, items / 256); consecutive tokens run on one XCD, so
@@ -98,7 +65,6 @@ __global__ void __launch_bounds__(256) qkv_heads_kernel(const QkvHeads a) {
   const int64_t slot = a.slots ? a.slots[t] : -1;
   const int64_t page = slot >= 0 ? slot >> a.log2_page : 0;
   const int off = static_cast<int>(slot & ((1 << a.log2_page) - 1));
-  constexpr bool kF32 = sizeof(T) == 4;
 
   if (it < rot_items) {
     const int h = it / GW, c0 = it % GW;   // head; chunks c0, c0 + GW, ...
@@ -155,10 +121,7 @@ __global__ void __launch_bounds__(256) qkv_heads_kernel(const QkvHeads a) {
         if (a.k_out) st8<T>(static_cast<T*>(a.k_out) + ((int64_t)t * a.Hkv + kh) * a.dkp + 8 * c, x[i]);
         if (slot >= 0 && a.k_cache) {
           const int64_t head = (page * a.Hkv + kh) << a.log2_page;
-          T* dst = static_cast<T*>(a.k_cache);
-          if constexpr (kF32) dst += (head + off) * a.dkp + 8 * c;
-          else dst += (head + (off & ~15)) * a.dkp + (c * 16 + (off & 15)) * 8;
-          st8<T>(dst, x[i]);
+          cache_k8<T>(static_cast<T*>(a.k_cache), head, off, a.dkp, c, x[i]);
         }
       }
     }
@@ -180,15 +143,7 @@ __global__ void __launch_bounds__(256) qkv_heads_kernel(const QkvHeads a) {
     if (a.v_out) st8<T>(static_cast<T*>(a.v_out) + at, x);
     if (slot >= 0 && a.v_cache) {
       const int64_t head = (page * a.Hkv + kh) << a.log2_page;
-      T* dst = static_cast<T*>(a.v_cache);
-      if constexpr (kF32) {
-        st8<T>(dst + (head + off) * a.dvp + 8 * c, x);
-      } else {
-        const int d0 = 8 * c, t16 = off & 15;
-        dst += (head + (off & ~15)) * a.dvp + (((d0 >> 5) * 4 + (t16 >> 2)) * 16 + (d0 & 15)) * 8 + ((d0 >> 4) & 1) * 4 + (t16 & 3);
-#pragma unroll
-        for (int j = 0; j < 8; ++j) dst[8 * j] = f2bf(x[j]);
-      }
+      cache_v8<T>(static_cast<T*>(a.v_cache), head, off, a.dvp, c, x);
     }
   }
 }

@@ -9,6 +9,7 @@
 // fp32 split-K slabs of the projection that made it, scaled by a per-token sigmoid gate,
 // and / or as the rows of the experts a token was routed to.
 // The first step (ids != nullptr) writes every stream from the scaled embedding row; the
+// With post_w (one stream) y is itself divided by its root mean square and scaled before it joins. The
 // last one (sum) normalises the plain sum of the streams and needs only the rows whose
 // logits are wanted (rows). HBM-bound: 8 S bytes per feature per token plus y and h.
 #include "common.h"
@@ -27,8 +28,8 @@ __device__ __forceinline__ f32x4 ld4(const void* p, int64_t i, bool f32) {
 }  // namespace
 
 // One workgroup per row; thread t owns 4-feature vectors t, t + NT, ... (MAXV of them).
-// S: compile-time bound of the stream count a.S.
-template <int S, int NT, int MAXV>
+// S: compile-time bound of the stream count a.S. POST: y is normalised first (post_w).
+template <int S, int NT, int MAXV, bool POST>
 __global__ void __launch_bounds__(NT) stream_step_kernel(const StreamStep a) {
   __shared__ float scratch[NT / 64];
   __shared__ float coef[S * S + 2 * S];   // mix[from][to], out, in
@@ -57,6 +58,50 @@ __global__ void __launch_bounds__(NT) stream_step_kernel(const StreamStep a) {
 
   const int nv = a.ld >> 2;
   float* xr = a.x + row * (int64_t)a.S * a.ld;
+  auto output = [&](int v) {   // 4 features of the sublayer's output
+    f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (a.yp) {
+      const float* p = a.yp + row * a.ld + 4 * v;
+      int s0 = 0;
+      if constexpr (MAXV == 1) {   // up to 8 slabs requested before the first add: one round trip
+        f32x4 sl[8];
+#pragma unroll
+        for (int s = 0; s < 8; ++s)
+          if (s < a.ys) sl[s] = *reinterpret_cast<const f32x4*>(p + s * a.y_slab);
+#pragma unroll
+        for (int s = 0; s < 8; ++s)
+          if (s < a.ys) y += sl[s];
+        s0 = 8;
+      }
+      for (int s = s0; s < a.ys; ++s) y += *reinterpret_cast<const f32x4*>(p + s * a.y_slab);
+    } else if (a.y) {
+      y = ld4(a.y, row * a.ld + 4 * v, a.f32);
+    }
+    if (a.gate) y *= gate;
+    for (int k = 0; k < a.top; ++k) {
+      const int64_t sl = row * a.top + k;
+      const int64_t er = a.epos ? (int64_t)a.epos[sl] : sl;
+      y += ld4(a.e, er * a.ld + 4 * v, a.f32);
+    }
+    return y;
+  };
+  f32x4 yn[POST ? MAXV : 1];
+  if constexpr (POST) {
+    float ys = 0.f;
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i) {
+      const int v = tid + i * NT;
+      yn[i] = v < nv ? output(v) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ys += yn[i][j] * yn[i][j];
+    }
+    const float rs = 1.f / sqrtf(block_sum<NT>(ys, scratch) / static_cast<float>(a.width) + a.eps);
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i) {
+      const int v = tid + i * NT;
+      if (v < nv) yn[i] *= rs * *reinterpret_cast<const f32x4*>(a.post_w + 4 * v);
+    }
+  }
   f32x4 u[MAXV];
   float ss = 0.f;
 #pragma unroll
@@ -76,30 +121,9 @@ __global__ void __launch_bounds__(NT) stream_step_kernel(const StreamStep a) {
 #pragma unroll
         for (int s = 0; s < S; ++s)
           xo[s] = s < a.S ? *reinterpret_cast<const f32x4*>(xr + (int64_t)s * a.ld + 4 * v) : f32x4{0.f, 0.f, 0.f, 0.f};
-        f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (a.yp) {
-          const float* p = a.yp + row * a.ld + 4 * v;
-          int s0 = 0;
-          if constexpr (MAXV == 1) {   // up to 8 slabs requested before the first add: one round trip
-            f32x4 sl[8];
-#pragma unroll
-            for (int s = 0; s < 8; ++s)
-              if (s < a.ys) sl[s] = *reinterpret_cast<const f32x4*>(p + s * a.y_slab);
-#pragma unroll
-            for (int s = 0; s < 8; ++s)
-              if (s < a.ys) y += sl[s];
-            s0 = 8;
-          }
-          for (int s = s0; s < a.ys; ++s) y += *reinterpret_cast<const f32x4*>(p + s * a.y_slab);
-        } else if (a.y) {
-          y = ld4(a.y, row * a.ld + 4 * v, a.f32);
-        }
-        if (a.gate) y *= gate;
-        for (int k = 0; k < a.top; ++k) {
-          const int64_t sl = row * a.top + k;
-          const int64_t er = a.epos ? (int64_t)a.epos[sl] : sl;
-          y += ld4(a.e, er * a.ld + 4 * v, a.f32);
-        }
+        f32x4 y;
+        if constexpr (POST) y = yn[i];
+        else y = output(v);
 #pragma unroll
         for (int t = 0; t < S; ++t) {
           f32x4 n = y * coef[S * S + t];
@@ -134,30 +158,32 @@ __global__ void __launch_bounds__(NT) stream_step_kernel(const StreamStep a) {
   }
 }
 
-template <int S>
+template <int S, bool POST = false>
 static void launch_streams(const StreamStep& a, int n, hipStream_t stream) {
   const int nv = a.ld / 4;
   if constexpr (S <= 4) {
     // few rows (decode): a vector per thread, so a row's loads all leave in one round trip
     if (n <= 512 && nv > 256) {
-      if (nv <= 512) stream_step_kernel<S, 512, 1><<<n, 512, 0, stream>>>(a);
-      else if (nv <= 1024) stream_step_kernel<S, 1024, 1><<<n, 1024, 0, stream>>>(a);
-      else if (nv <= 2048) stream_step_kernel<S, 1024, 2><<<n, 1024, 0, stream>>>(a);
-      else stream_step_kernel<S, 1024, 4><<<n, 1024, 0, stream>>>(a);
+      if (nv <= 512) stream_step_kernel<S, 512, 1, POST><<<n, 512, 0, stream>>>(a);
+      else if (nv <= 1024) stream_step_kernel<S, 1024, 1, POST><<<n, 1024, 0, stream>>>(a);
+      else if (nv <= 2048) stream_step_kernel<S, 1024, 2, POST><<<n, 1024, 0, stream>>>(a);
+      else stream_step_kernel<S, 1024, 4, POST><<<n, 1024, 0, stream>>>(a);
       return;
     }
   }
-  if (nv <= 64) stream_step_kernel<S, 64, 1><<<n, 64, 0, stream>>>(a);
-  else if (nv <= 256) stream_step_kernel<S, 256, 1><<<n, 256, 0, stream>>>(a);
-  else if (nv <= 1024) stream_step_kernel<S, 256, 4><<<n, 256, 0, stream>>>(a);
-  else if (nv <= 2048) stream_step_kernel<S, 256, 8><<<n, 256, 0, stream>>>(a);
-  else stream_step_kernel<S, 256, 16><<<n, 256, 0, stream>>>(a);
+  if (nv <= 64) stream_step_kernel<S, 64, 1, POST><<<n, 64, 0, stream>>>(a);
+  else if (nv <= 256) stream_step_kernel<S, 256, 1, POST><<<n, 256, 0, stream>>>(a);
+  else if (nv <= 1024) stream_step_kernel<S, 256, 4, POST><<<n, 256, 0, stream>>>(a);
+  else if (nv <= 2048) stream_step_kernel<S, 256, 8, POST><<<n, 256, 0, stream>>>(a);
+  else stream_step_kernel<S, 256, 16, POST><<<n, 256, 0, stream>>>(a);
 }
 
 int stream_step(const StreamStep& a, int n_rows, hipStream_t stream) {
   if (n_rows == 0) return 0;
   if (a.S < 1 || a.S > 8 || a.ld % 8 != 0 || a.ld > 16384 || a.width < 1 || a.width > a.ld) return -1;
-  if (a.S == 1) launch_streams<1>(a, n_rows, stream);
+  if (a.post_w && a.S != 1) return -2;
+  if (a.post_w) launch_streams<1, true>(a, n_rows, stream);
+  else if (a.S == 1) launch_streams<1>(a, n_rows, stream);
   else if (a.S == 2) launch_streams<2>(a, n_rows, stream);
   else if (a.S <= 4) launch_streams<4>(a, n_rows, stream);
   else launch_streams<8>(a, n_rows, stream);

@@ -47,13 +47,14 @@ def build_engine(s: Settings, device: str | torch.device | None = None, tp=None,
 
     from operator_amd.engine.llm import LLMEngine
     from operator_amd.models import weight_cache
+    from operator_amd.models.config import ARCHS
     from operator_amd.models.kv_cache import PagedKVCache
     from operator_amd.models.registry import build_model, load_config
 
     e = s.engine
     dev = torch.device(device or e.device)
     cfg = load_config(e.model, e.model_path)
-    if cfg.arch == "sufolix" and cfg.max_position < e.max_context:
+    if cfg.arch not in ARCHS and cfg.max_position < e.max_context:
         cfg = replace(cfg, max_position=e.max_context)   # a table length there, not a property of the model
     dtype = getattr(torch, e.dtype)
     if tp is not None and tp.world > 1 and dev.type == "cuda" and e.oneshot_allreduce_mb > 0 \
@@ -66,11 +67,11 @@ def build_engine(s: Settings, device: str | torch.device | None = None, tp=None,
     # KV cache: the compute dtype, or OCP fp8 (e4m3fn, per-tensor scales) with engine.kv_dtype=fp8
     if e.kv_dtype not in ("auto", "fp8"):
         raise ValueError(f"engine.kv_dtype must be auto or fp8, not {e.kv_dtype!r}")
-    if e.kv_dtype == "fp8" and cfg.arch == "sufolix":
-        raise ValueError("engine.kv_dtype=fp8: sufolix models keep keys and values in the compute dtype")
+    if e.kv_dtype == "fp8" and cfg.arch not in ARCHS:
+        raise ValueError(f"engine.kv_dtype=fp8: {cfg.arch} models keep keys and values in the compute dtype")
     kv_dtype = torch.float8_e4m3fn if e.kv_dtype == "fp8" else dtype
     pages = kv_pages or PagedKVCache.pages_for_shapes(int(e.kv_cache_gb * 1e9), model.kv_shapes(), e.page_size,
-                                                      torch.finfo(kv_dtype).bits // 8)
+                                                      torch.finfo(kv_dtype).bits // 8, model.page_rows())
     kv = PagedKVCache.for_model(model, pages, e.page_size, dtype=kv_dtype, k_scale=e.kv_scale, v_scale=e.kv_scale)
     kw = dict(max_batch=e.max_batch, max_prefill_tokens=e.max_prefill_tokens, max_context=e.max_context,
               use_graphs=e.use_graphs, multi_step=e.multi_step, admit_wait_s=e.admit_wait_ms / 1e3,

@@ -316,7 +316,7 @@ class _PrefillGraph:
         # profiles/bench_r4_flagship_idle.jsonl "copyBuffer -> copyBuffer")
         spec = (("ids", T, i64), ("pos", T, i64), ("slots", T, i64), ("last", S, i64), ("seeds", S, i64),
                 ("spos", S, i64), ("cu", S + 1, i32), ("ws", self.W, i32), ("wq", self.W, i32),
-                ("temp", S, torch.float32), ("pfx", S, i32))
+                ("temp", S, torch.float32), ("pfx", S, i32), ("prev", S, i32))
         self._layout, off = [], 0
         for n, k, dt in spec:
             isz = torch.empty((), dtype=dt).element_size()
@@ -348,7 +348,8 @@ class _PrefillGraph:
         e, d = self.eng, self.dev
         pre = (e._pk, e._pv, d["pfx"], None) if e.prefix_sharing else None
         fb = ForwardBatch(d["ids"], d["pos"], d["slots"], True, d["last"], seq_lens=[],
-                          prefill_work=(d["cu"], d["ws"], d["wq"], self.variant), prefix=pre)
+                          prefill_work=(d["cu"], d["ws"], d["wq"], self.variant), prefix=pre,
+                          prev_pages=d["prev"] if pre is not None else None)
         logits = e.model.forward(fb, e.kv)
         self.tok = e.model.sample(logits, d["temp"], d["seeds"], d["spos"])
 
@@ -367,7 +368,7 @@ class _PrefillGraph:
             self._run()
         self.graph = g
 
-    def launch(self, ids, pos, slots, cu, ws, wq, last, temp, seeds, spos, pfx=None):
+    def launch(self, ids, pos, slots, cu, ws, wq, last, temp, seeds, spos, pfx=None, prev=None):
         """Queue one replay for the real batch (numpy inputs, <= T tokens, <= S
         sequences); returns (pinned token buffer, event): ``event`` completes when the
         batch's sampled first tokens are in the buffer."""
@@ -379,7 +380,8 @@ class _PrefillGraph:
         b = len(last)
         for name, arr, fill in (("ids", ids, 0), ("pos", pos, 0), ("slots", slots, -1), ("last", last, 0),
                                 ("seeds", seeds, 0), ("spos", spos, 0), ("temp", temp, 0.0), ("ws", ws, -1),
-                                ("wq", wq, 0), ("cu", cu, int(cu[-1])), ("pfx", pfx if pfx is not None else [], 0)):
+                                ("wq", wq, 0), ("cu", cu, int(cu[-1])), ("pfx", pfx if pfx is not None else [], 0),
+                                ("prev", prev if prev is not None else [], -1)):
             v = h[name].numpy()
             v[:len(arr)] = arr
             v[len(arr):] = fill
@@ -507,8 +509,8 @@ class LLMEngine:
         if self.prefix_sharing:
             n = self._pfx_cap
             new = lambda h, d: torch.zeros(n, h, d, dtype=self._pfx_dtype, device=self.device)  # noqa: E731
-            self._pk = [new(h, dk) for h, dk, _ in model.kv_shapes()]
-            self._pv = [new(h, dv) for h, _, dv in model.kv_shapes()]
+            self._pk = [new(h, dk) for h, dk, _ in model.prefix_shapes()]
+            self._pv = [new(h, dv) for h, _, dv in model.prefix_shapes()]
 
     # ------------------------------------------------------------------ API
     def submit(self, req: GenRequest) -> GenRequest:
@@ -834,7 +836,8 @@ class LLMEngine:
         return dict(ids=np.concatenate([np.asarray(r.prompt[n:], dtype=np.int64) for r, n in zip(batch, skip)]),
                     pos=np.concatenate(ar),
                     slots=np.concatenate([np.asarray(r.pages, dtype=np.int64)[a // P] * P + a % P for r, a in zip(batch, ar)]),
-                    cu=cu, ws=ws, wq=wq, var=var, lens=lens, skip=skip, full=full)
+                    cu=cu, ws=ws, wq=wq, var=var, lens=lens, skip=skip, full=full,
+                    prev=[r.pages[(n - 1) // P] if n else -1 for r, n in zip(batch, skip)])
 
     def _to_device(self, x, dt=torch.long) -> torch.Tensor:
         return torch.as_tensor(np.asarray(x)).to(dtype=dt).to(self.device, non_blocking=True)
@@ -846,7 +849,7 @@ class LLMEngine:
             if self.device.type == "cuda" else None
         pre = (self._pk, self._pv, t(p["skip"], torch.int32), p["skip"]) if any(p["skip"]) else None
         fb = ForwardBatch(t(p["ids"]), t(p["pos"]), t(p["slots"]), True, t(last), seq_lens=p["lens"], prefill_work=work,
-                          prefix=pre)
+                          prefix=pre, prev_pages=None if pre is None else t(p["prev"], torch.int32))
         return self.model.forward(fb, self.kv)
 
     def _prefill_impl(self, batch: list[GenRequest]) -> _PendingPrefill:
@@ -859,7 +862,7 @@ class LLMEngine:
         g = self._prefill_graph_for(n, len(batch))
         if g is not None:
             toks, ev = g.launch(p["ids"], p["pos"], p["slots"], p["cu"], p["ws"], p["wq"], last, temps, seeds, p["full"],
-                                p["skip"])
+                                p["skip"], p["prev"])
             self.stats.prefill_graph_replays += 1
             self.stats.prefill_padded_tokens += g.T - n
         else:

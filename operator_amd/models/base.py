@@ -2,7 +2,7 @@
 
 ``LLMEngine`` drives any class with this surface: ``cfg`` (layers, max_position, eos_ids),
 ``device`` / ``dtype``, ``forward(ForwardBatch, PagedKVCache)``, ``sample``, the per-layer
-cache shapes (``kv_shapes``) and the prefill attention's work granularity (``prefill_plan``).
+cache shapes (``kv_shapes``, ``page_rows``) and the prefill attention's work granularity (``prefill_plan``).
 """
 from __future__ import annotations
 
@@ -31,6 +31,9 @@ class ForwardBatch:
     # cached post-RoPE K/V per layer ([P, Hkv, D] each); sequence s's tokens follow pfx_lens[s] of them
     prefix: tuple | None = None
     kv_sink: object = None   # called (layer, k, v) with each prefill layer's K/V (prefix capture)
+    # per sequence the page of the tokens before its first row, -1: none ([S] int32; state that
+    # lives in the pages continues from there)
+    prev_pages: torch.Tensor | None = None
     residual_sink: object = None   # called (layer, x [T, hidden] fp32) with the residual after each layer
     # decode
     block_tables: torch.Tensor | None = None   # [B, max_pages] int32
@@ -59,6 +62,16 @@ class DecoderModel:
     def kv_shapes(self) -> list[tuple[int, int, int]]:
         """(kv heads, key size, value size) each layer keeps in the cache."""
         raise NotImplementedError
+
+    def prefix_shapes(self) -> list[tuple[int, int, int]]:
+        """(heads, key size, value size) of the rows each layer's prefill attention reads of a shared
+        prompt prefix."""
+        return self.kv_shapes()
+
+    def page_rows(self) -> list[tuple[int, int] | None]:
+        """(rows, columns) of recurrent state each layer keeps per cache page (None: none), for layers that
+        need the last few tokens' projections; a page holds that of its own tokens."""
+        return []
 
     def prefill_plan(self) -> tuple[int, int]:
         """(attention variant, query rows per work item) of the prefill work list."""

@@ -17,6 +17,9 @@ exact architecture, or loaded from a local HF safetensors directory whose
   sufolix  Sufolix (``config_from_dir``): hyper-connected residual streams, attention layers
            with their own head sizes, per-head q/k norm and value mixing, dense or
            routed-expert feed-forwards; ``SufolixConfig``
+  relurax  Relurax (``config_from_dir``): sliding-window attention whose values are its convolved
+           keys, latent attention that may read another layer's cached rows, norms before and
+           after every sublayer; ``ReluraxConfig``
 """
 from __future__ import annotations
 
@@ -108,7 +111,9 @@ PRESETS: dict[str, LlamaConfig] = {
 @dataclass(frozen=True)
 class AttentionSpec:
     """One attention mixer: head counts and sizes, rotary positions on the first ``rot_dims``
-    dimensions, the score scale, and whether its values mix with the first mixing layer's."""
+    dimensions, the score scale, and whether its values mix with the first mixing layer's.
+    ``conv``: taps of a short causal convolution on q and k (0: none), ``window``: how far back a
+    query sees, itself included (0: everything)."""
     heads: int
     kv_heads: int
     dim: int
@@ -117,6 +122,24 @@ class AttentionSpec:
     rot_base: float = 10000.0
     rot_dims: int = 0
     v_mix: bool = False
+    conv: int = 0
+    window: int = 0
+
+
+@dataclass(frozen=True)
+class LatentSpec:
+    """One latent-attention mixer: queries from a latent of ``q_rank``, keys and values from one of
+    ``kv_rank``; per head ``dim`` unrotated and ``rot_dim`` rotated query / key dimensions (all of the
+    latter rotate) and ``vdim`` value ones. ``kv_from``: the layer whose cached rows it reads (-1: its own)."""
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rot_base: float = 10000.0
+    kv_from: int = -1
 
 
 @dataclass(frozen=True)
@@ -131,7 +154,7 @@ class FeedForwardSpec:
 
 @dataclass(frozen=True)
 class DecoderLayerSpec:
-    mixer: AttentionSpec
+    mixer: AttentionSpec | LatentSpec
     mlp: FeedForwardSpec | None = None
 
 
@@ -173,13 +196,63 @@ class SufolixConfig:
         return asdict(self)
 
 
+@dataclass(frozen=True)
+class ReluraxConfig:
+    name: str = "relurax"
+    vocab_size: int = 32000
+    hidden: int = 1024
+    rms_eps: float = 1e-6
+    layer_specs: tuple[DecoderLayerSpec, ...] = ()
+    max_position: int = 32768        # rotary table length, not a limit of the design
+    bos_id: int = -1
+    eos_ids: tuple[int, ...] = (-1,)
+    arch: str = "relurax"
+    add_bos: bool = False
+
+    @property
+    def layers(self) -> int:
+        return len(self.layer_specs)
+
+    def param_count(self) -> int:
+        h = self.hidden
+        n = 2 * self.vocab_size * h + h
+        for sp in self.layer_specs:
+            m = sp.mixer
+            n += 2 * h + m.heads * h + m.heads * m.vdim * h
+            if isinstance(m, LatentSpec):
+                n += m.q_rank * (h + 1) + m.heads * (m.dim + m.rot_dim) * m.q_rank + m.heads * (m.dim + m.vdim) * m.kv_rank
+                n += (m.kv_rank + m.rot_dim) * h + m.kv_rank if m.kv_from < 0 else 0
+            else:
+                n += (m.heads + m.kv_heads) * m.dim * (h + m.conv) + 2 * m.dim
+            n += 3 * h * sp.mlp.ff + 2 * h if sp.mlp is not None else 0
+        return n
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
+        n = 0
+        for m in (sp.mixer for sp in self.layer_specs):
+            if isinstance(m, LatentSpec):
+                n += m.kv_rank + m.rot_dim if m.kv_from < 0 else 0
+            else:
+                n += m.kv_heads * (m.dim + m.vdim)
+        return n * dtype_bytes
+
+    def to_dict(self) -> dict:
+        return asdict(self)
+
+
+def _relurax(name: str, layers: int, attn: AttentionSpec, latent: LatentSpec, ff: int, **kw) -> ReluraxConfig:
+    """Alternating window / latent layers; every second latent layer reads the one before it."""
+    mix = [attn if i % 2 == 0 else latent if i % 4 == 1 else replace(latent, kv_from=i - 2) for i in range(layers)]
+    return ReluraxConfig(name=name, layer_specs=tuple(DecoderLayerSpec(m, FeedForwardSpec(ff)) for m in mix), **kw)
+
+
 def _sufolix(name: str, layers: int, mixer: AttentionSpec, dense: FeedForwardSpec, moe: FeedForwardSpec, **kw) -> SufolixConfig:
     """Alternating dense / expert layers of one mixer."""
     return SufolixConfig(name=name, layer_specs=tuple(DecoderLayerSpec(mixer, moe if i % 2 else dense)
                                                       for i in range(layers)), **kw)
 
 
-DESIGN_PRESETS: dict[str, SufolixConfig] = {
+DESIGN_PRESETS: dict[str, SufolixConfig | ReluraxConfig] = {
     "tiny-sufolix": _sufolix("tiny-sufolix", 4, AttentionSpec(6, 3, 40, 24, 0.2, 20000.0, 32, True),
                              FeedForwardSpec(160), FeedForwardSpec(72, experts=5, top=2, shared_ff=96),
                              vocab_size=1000, hidden=192, streams=3, embed_scale=8.0, bos_id=990, eos_ids=(991,)),
@@ -192,10 +265,21 @@ DESIGN_PRESETS: dict[str, SufolixConfig] = {
     "sufolix-1b": _sufolix("sufolix-1b", 16, AttentionSpec(16, 4, 128, 96, 0.1, 100000.0, 64, True),
                            FeedForwardSpec(8192), FeedForwardSpec(1024, experts=32, top=4, shared_ff=2048),
                            vocab_size=32000, hidden=2048, streams=4, bos_id=1, eos_ids=(2,)),
+    "tiny-relurax": _relurax("tiny-relurax", 4, AttentionSpec(6, 2, 40, 40, 0.2, conv=4, window=24),
+                             LatentSpec(5, 24, 8, 40, 72, 48, 0.25, 20000.0), 160,
+                             vocab_size=1000, hidden=192, bos_id=990, eos_ids=(991,)),
+    # Llama-3-8B's width, heads and feed-forward; latents of the usual large-model sizes
+    "relurax-8b": _relurax("relurax-8b", 32, AttentionSpec(32, 8, 128, 128, 0.088388, conv=4, window=1024),
+                           LatentSpec(32, 128, 64, 128, 1536, 512, 0.072169, 500000.0), 14336,
+                           vocab_size=128256, hidden=4096, bos_id=128000, eos_ids=(128001, 128009)),
+    # the width of a ~1B model, fewer and smaller heads
+    "relurax-1b": _relurax("relurax-1b", 16, AttentionSpec(16, 4, 128, 128, 0.088388, conv=4, window=512),
+                           LatentSpec(16, 96, 32, 96, 768, 256, 0.088388, 100000.0), 8192,
+                           vocab_size=32000, hidden=2048, bos_id=1, eos_ids=(2,)),
 }
 
 
-def get_config(name: str, **overrides) -> "LlamaConfig | SufolixConfig":
+def get_config(name: str, **overrides) -> "LlamaConfig | SufolixConfig | ReluraxConfig":
     if name in DESIGN_PRESETS:
         c = DESIGN_PRESETS[name]
     elif name in PRESETS:
@@ -298,7 +382,59 @@ def sufolix_from_dict(hc: dict, name: str = "sufolix") -> SufolixConfig:
                          rms_eps=float(hc["norm"]["eps"]), layer_specs=tuple(specs))
 
 
-def config_from_dir(path: str, name: str | None = None) -> "LlamaConfig | SufolixConfig":
+def _heads(i: int, m: dict, dim: int) -> None:
+    if int(m["heads"]) < 1 or max(dim, int(m["vdim"])) > 256:
+        raise ValueError(f"layer {i}: head sizes {dim}/{m['vdim']}; the attention kernels go up to 256")
+
+
+def relurax_from_dict(hc: dict, name: str = "relurax") -> ReluraxConfig:
+    """ReluraxConfig from a checkpoint's config.json contents."""
+    specs: list[DecoderLayerSpec] = []
+    for i, lay in enumerate(hc["layers"]):
+        m, f, kind = lay["mixer"], lay.get("mlp"), lay["type"]
+        if kind == "attention":
+            _heads(i, m, int(m["dim"]))
+            mixer = AttentionSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                                  scale=float(m["scale"]), conv=int(m["conv"]), window=int((m.get("mask") or {}).get("size", 0)))
+            if mixer.kv_heads < 1 or mixer.heads % mixer.kv_heads:
+                raise ValueError(f"layer {i}: {mixer.heads} query heads over {mixer.kv_heads} kv heads")
+            if mixer.vdim != mixer.dim:
+                raise ValueError(f"layer {i}: values are the keys, but their sizes are {mixer.vdim} and {mixer.dim}")
+            if not 1 <= mixer.conv <= 8:
+                raise ValueError(f"layer {i}: a convolution of {mixer.conv} taps (1..8 supported)")
+            if "mask" in m and mixer.window < 1:
+                raise ValueError(f"layer {i}: a window of {mixer.window} tokens")
+        elif kind == "latent_attention":
+            _heads(i, m, int(m["dim"]) + int(m["rot_dim"]))
+            mixer = LatentSpec(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                               q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]), scale=float(m["scale"]),
+                               rot_base=float(m["rot"]["base"]), kv_from=-1 if m.get("kv_from") is None else int(m["kv_from"]))
+            if mixer.rot_dim % 2 or int(m["rot"]["dims"]) != mixer.rot_dim:
+                raise ValueError(f"layer {i}: {m['rot']['dims']} rotated dimensions of a part of {mixer.rot_dim}")
+            if -(-mixer.kv_rank // 32) * 32 + mixer.rot_dim > 640 or mixer.q_rank > 4096:
+                raise ValueError(f"layer {i}: latent sizes {mixer.q_rank} and {mixer.kv_rank} + {mixer.rot_dim}; "
+                                 "the latent kernels go up to 4096 and 640")
+            if mixer.kv_from >= 0:
+                src = specs[mixer.kv_from].mixer if mixer.kv_from < i else None
+                if not isinstance(src, LatentSpec) or src.kv_from >= 0 or (src.kv_rank, src.rot_dim, src.rot_base) != (
+                        mixer.kv_rank, mixer.rot_dim, mixer.rot_base):
+                    raise ValueError(f"layer {i}: layer {mixer.kv_from} keeps no latent rows of its kind")
+        else:
+            raise ValueError(f"layer {i}: mixer type {kind!r} not supported")
+        if f is not None and f["kind"] != "dense":
+            raise ValueError(f"layer {i}: feed-forward kind {f['kind']!r} not supported")
+        specs.append(DecoderLayerSpec(mixer, None if f is None else FeedForwardSpec(int(f["ff"]))))
+    if not specs:
+        raise ValueError("no layers")
+    return ReluraxConfig(name=name, vocab_size=int(hc["vocab"]), hidden=int(hc["width"]), rms_eps=float(hc["norm"]["eps"]),
+                         layer_specs=tuple(specs))
+
+
+# config.json "architecture" -> reader
+DESIGNS = {"sufolix": sufolix_from_dict, "relurax": relurax_from_dict}
+
+
+def config_from_dir(path: str, name: str | None = None) -> "LlamaConfig | SufolixConfig | ReluraxConfig":
     """The configuration a checkpoint directory's config.json describes, whichever of the
     supported architectures it is (``architecture``: a design of its own; ``model_type``: a
     HuggingFace Llama-architecture checkpoint)."""
@@ -307,6 +443,6 @@ def config_from_dir(path: str, name: str | None = None) -> "LlamaConfig | Sufoli
     arch = hc.get("architecture")
     if arch is None:
         return config_from_hf(path, name)
-    if str(arch).lower() != "sufolix":
+    if str(arch).lower() not in DESIGNS:
         raise ValueError(f"{path}: architecture {arch!r} not supported")
-    return sufolix_from_dict(hc, name or os.path.basename(os.path.normpath(path)))
+    return DESIGNS[str(arch).lower()](hc, name or os.path.basename(os.path.normpath(path)))

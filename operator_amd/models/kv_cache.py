@@ -17,7 +17,12 @@ bf16 / fp32). Not the default.
 
 ``shapes`` gives every layer its own (kv heads, key size, value size): one K and one V
 tensor per layer instead of the two stacked ones. How a layer arranges a page's bytes is its
-kernels' business (attn_decode.hip's K tiles, qkv_heads.hip's K / V tiles).
+kernels' business (attn_decode.hip's K tiles, qkv_heads.hip's K / V tiles). A layer that keeps
+latent rows has one head and no values; one that reads another layer's rows has no heads.
+
+``page_rows`` adds per layer a few rows of recurrent state to every page (``state``): the last
+projections a short convolution asks for belong to the page of their tokens, so they are
+allocated, shared with a common prefix and freed with it.
 """
 from __future__ import annotations
 
@@ -54,7 +59,8 @@ class PageAllocator:
 class PagedKVCache:
     def __init__(self, layers: int, num_pages: int, kv_heads: int, head_dim: int, page_size: int = 64,
                  device: str | torch.device = "cuda", dtype: torch.dtype = torch.bfloat16,
-                 k_scale: float = 1.0, v_scale: float = 1.0, shapes: list[tuple[int, int, int]] | None = None):
+                 k_scale: float = 1.0, v_scale: float = 1.0, shapes: list[tuple[int, int, int]] | None = None,
+                 page_rows: list[tuple[int, int] | None] = ()):
         if page_size & (page_size - 1):
             raise ValueError("page_size must be a power of two")
         if k_scale <= 0 or v_scale <= 0:
@@ -70,6 +76,7 @@ class PagedKVCache:
             new = lambda h, d: torch.zeros(num_pages, h, page_size, d, dtype=dtype, device=device)  # noqa: E731
             self.k = [new(h, dk) for h, dk, _ in shapes]
             self.v = [new(h, dv) for h, _, dv in shapes]
+        self.state = [None if r is None else torch.zeros(num_pages, *r, dtype=dtype, device=device) for r in page_rows]
         self.allocator = PageAllocator(num_pages)
 
     @classmethod
@@ -78,13 +85,17 @@ class PagedKVCache:
         """The cache ``model`` needs (its ``kv_shapes``), in its compute dtype unless given."""
         shapes = model.kv_shapes()
         h, dk, dv = shapes[0]
+        rows = model.page_rows()
+        if any(r is not None and r[0] > page_size for r in rows):
+            raise ValueError(f"pages of {page_size} tokens cannot hold the state rows of {rows}")
         alike = dk == dv and all(s == shapes[0] for s in shapes)
         return cls(len(shapes), num_pages, h, dk, page_size, device=model.device, dtype=dtype or model.dtype,
-                   k_scale=k_scale, v_scale=v_scale, shapes=None if alike else shapes)
+                   k_scale=k_scale, v_scale=v_scale, shapes=None if alike else shapes, page_rows=rows)
 
     @staticmethod
-    def pages_for_shapes(budget_bytes: int, shapes: list[tuple[int, int, int]], page_size: int, dtype_bytes: int = 2) -> int:
-        per_page = sum(h * (dk + dv) for h, dk, dv in shapes) * page_size * dtype_bytes
+    def pages_for_shapes(budget_bytes: int, shapes: list[tuple[int, int, int]], page_size: int, dtype_bytes: int = 2,
+                         page_rows: list[tuple[int, int] | None] = ()) -> int:
+        per_page = (sum(h * (dk + dv) for h, dk, dv in shapes) * page_size + sum(r * c for r, c in filter(None, page_rows))) * dtype_bytes
         return max(1, int(budget_bytes // per_page))
 
     @staticmethod

@@ -7,9 +7,10 @@ from __future__ import annotations
 
 from .config import ARCHS, config_from_dir, get_config
 from .llama import LlamaModel
+from .relurax import ReluraxModel
 from .sufolix import SufolixModel
 
-MODELS = {**{a: LlamaModel for a in ARCHS}, "sufolix": SufolixModel}
+MODELS = {**{a: LlamaModel for a in ARCHS}, "sufolix": SufolixModel, "relurax": ReluraxModel}
 
 
 def load_config(name: str, model_path: str | None = None):

@@ -21,7 +21,6 @@ residual streams, norms, router, rotation and softmax are fp32 in both.
 from __future__ import annotations
 
 import math
-import os
 from dataclasses import dataclass
 
 import torch
@@ -30,9 +29,10 @@ from operator_amd import ops
 from operator_amd.ops import decoder as dec
 from operator_amd.parallel.comm import Group
 
-from .base import DecoderModel, ForwardBatch
+from .base import ForwardBatch
 from .config import SufolixConfig
 from .kv_cache import PagedKVCache
+from .padded import PaddedModel
 
 
 @dataclass
@@ -57,22 +57,13 @@ class SufolixLayer:
     sd: torch.Tensor | None = None
 
 
-class SufolixModel(DecoderModel):
+class SufolixModel(PaddedModel):
     LAYER = SufolixLayer
-    LAYOUT_FUNCS = ("init_random", "load_checkpoint", "_build", "_layer", "_gate_up", "_down", "_put")
+    LAYOUT_FUNCS = PaddedModel.LAYOUT_FUNCS + ("init_random", "_layer")
 
     def __init__(self, cfg: SufolixConfig, device: str | torch.device = "cuda", tp: Group | None = None,
                  dtype: torch.dtype = torch.bfloat16, weight_dtype: str = "bfloat16"):
-        self.tp = tp or Group.single()
-        if self.tp.world != 1:
-            raise ValueError("sufolix models run on one GPU (tensor parallel degree 1)")
-        if weight_dtype != "bfloat16":
-            raise ValueError(f"sufolix weights are stored in the compute dtype, not {weight_dtype!r}")
-        if dtype not in (torch.bfloat16, torch.float32):
-            raise ValueError(f"sufolix computes in bfloat16 or float32, not {dtype}")
-        self.cfg, self.device, self.dtype = cfg, torch.device(device), dtype
-        self.ld = max(128, dec.pad_to(cfg.hidden, 64))
-        self.gu_block = ops.GU_BLOCK
+        super().__init__(cfg, device, tp, dtype, weight_dtype)
         self.heads = [dec.HeadLayout(a.heads, a.kv_heads, a.dim, a.vdim, a.rot_dims, True, cfg.rms_eps)
                       for a in (sp.mixer for sp in cfg.layer_specs)]
         self.hq = max(L.heads for L in self.heads)
@@ -86,31 +77,12 @@ class SufolixModel(DecoderModel):
             self.rot.append(tabs[key])
         mixing = [i for i, sp in enumerate(cfg.layer_specs) if sp.mixer.v_mix]
         self.first_mix = mixing[0] if mixing else -1
-        self.layers: list[SufolixLayer] = []
-        self.embed = self.final_norm = self.lm_head = None
 
     # ------------------------------------------------------------------ engine surface
     def kv_shapes(self) -> list[tuple[int, int, int]]:
         return [(L.kv_heads, *L.pads) for L in self.heads]
 
-    def prefill_plan(self) -> tuple[int, int]:
-        return dec.GD_VARIANT, dec.GD_BLOCK_Q
-
     # ------------------------------------------------------------------ weights
-    def _put(self, rows: int, cols: int, parts, dtype=None) -> torch.Tensor:
-        """Zero [rows, cols] with each (row, col, tensor) of ``parts`` placed in it."""
-        t = torch.zeros(rows, cols, dtype=dtype or self.dtype, device=self.device)
-        for r, c, p in parts:
-            t[r:r + p.shape[0], c:c + p.shape[1]] = p
-        return t
-
-    def _gate_up(self, gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
-        n = max(128, dec.pad_to(gate.shape[0], 64))
-        return ops.interleave_gate_up(self._put(n, self.ld, [(0, 0, gate)]), self._put(n, self.ld, [(0, 0, up)]))
-
-    def _down(self, w: torch.Tensor) -> torch.Tensor:
-        return self._put(self.ld, max(128, dec.pad_to(w.shape[1], 64)), [(0, 0, w)])
-
     def _layer(self, i: int, get, has) -> SufolixLayer:
         c, sp, L, W = self.cfg, self.cfg.layer_specs[i], self.heads[i], self.cfg.hidden
         a, p = sp.mixer, f"l{i}."
@@ -122,9 +94,7 @@ class SufolixModel(DecoderModel):
             return get(name, shape).float().reshape(shape).contiguous()
 
         def norm(name):
-            w = torch.zeros(self.ld, device=self.device)
-            w[:W] = f32(name, (W,))
-            return w
+            return self._padded(f32(name, (W,)), self.ld)
 
         def hc(q):   # a single stream without stored coefficients is the plain residual
             one = torch.ones(S) if S == 1 else None
@@ -164,18 +134,6 @@ class SufolixModel(DecoderModel):
         lw.wr = self._put(dec.router_rows(m.experts), self.ld, rows)
         return lw
 
-    def _build(self, get, has) -> "SufolixModel":
-        """Packed, padded weights from ``get(name, shape)`` (checkpoint tensor names)."""
-        c, V = self.cfg, self.cfg.vocab_size
-        self.embed = self._put(V, self.ld, [(0, 0, get("embed", (V, c.hidden)))])
-        self.layers = [self._layer(i, get, has) for i in range(c.layers)]
-        self.final_norm = torch.zeros(self.ld, device=self.device)
-        self.final_norm[:c.hidden] = get("final.norm", (c.hidden,)).float()
-        self.lm_head = self._put(dec.pad_to(V, 64), self.ld, [(0, 0, get("head", (V, c.hidden)))])
-        if self.device.type == "cuda":
-            torch.cuda.synchronize(self.device)
-        return self
-
     def init_random(self, seed: int = 0) -> "SufolixModel":
         """Random weights of the exact architecture: O(1) activations, streams that mix mildly."""
         def get(name, shape):
@@ -194,25 +152,6 @@ class SufolixModel(DecoderModel):
             return t if leaf == "embed" else t * (1.0 / math.sqrt(shape[-1]))
 
         return self._build(get, lambda name: True)
-
-    def load_checkpoint(self, path: str) -> "SufolixModel":
-        """Weights of a checkpoint directory (safetensors), checked against ``cfg``'s shapes."""
-        from safetensors import safe_open
-
-        names: dict = {}
-        for f in sorted(f for f in os.listdir(path) if f.endswith(".safetensors")):
-            sf = safe_open(os.path.join(path, f), framework="pt", device="cpu")
-            names.update({k: sf for k in sf.keys()})
-        if not names:
-            raise FileNotFoundError(f"no *.safetensors in {path}")
-
-        def get(name, shape):
-            t = names[name].get_tensor(name)
-            if t.numel() != math.prod(shape) or (t.dim() > 1 and tuple(t.shape) != tuple(shape)):
-                raise ValueError(f"{path}: {name} is {tuple(t.shape)}, {tuple(shape)} expected")
-            return t.reshape(shape).to(self.device, self.dtype)
-
-        return self._build(get, lambda name: name in names)
 
     # ------------------------------------------------------------------ forward
     def forward(self, fb: ForwardBatch, kv: PagedKVCache) -> torch.Tensor:
@@ -239,18 +178,6 @@ class SufolixModel(DecoderModel):
             if fb.residual_sink is not None:
                 fb.residual_sink(i, x[:, :, :c.hidden].sum(1))
         return ops.linear(h, self.lm_head)[:, :c.vocab_size]
-
-    def _step(self, x, y: dec.SublayerOut, hc: dec.Stream, after: tuple | None, fb: ForwardBatch) -> torch.Tensor:
-        """Finish a sublayer; ``after`` = (stream coefficients, norm weight) of the next one, None
-        at the end of the model (only the rows whose logits are wanted, streams left as they are)."""
-        c = self.cfg
-        if after is not None:
-            return dec.stream_step(x, y, hc, after[0], after[1], c.hidden, c.rms_eps, self.dtype)
-        if fb.residual_sink is None:
-            return dec.stream_step(x, y, hc, None, self.final_norm, c.hidden, c.rms_eps, self.dtype,
-                                   rows=fb.logits_index, write_x=False)
-        h = dec.stream_step(x, y, hc, None, self.final_norm, c.hidden, c.rms_eps, self.dtype)
-        return h if fb.logits_index is None else h.index_select(0, fb.logits_index)
 
     def _mixer(self, i: int, lw: SufolixLayer, h, v_first, fb: ForwardBatch, kv: PagedKVCache, ws):
         """(o-projection output, the first mixing layer's values)."""

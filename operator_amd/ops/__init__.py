@@ -71,17 +71,21 @@ def rmsnorm(x, w: torch.Tensor, eps: float, residual: torch.Tensor | None = None
     return y
 
 
-def silu_mul(gu: torch.Tensor, out: torch.Tensor | None = None, block: int | None = None) -> torch.Tensor:
-    """silu(gate) * up for gate|up interleaved in ``block``-feature blocks (None: [gate | up])."""
+# activation of a gated feed-forward (common.h Glu): act(gate) * up
+SILU, GELU_TANH = 1, 2
+
+
+def silu_mul(gu: torch.Tensor, out: torch.Tensor | None = None, block: int | None = None, act: int = SILU) -> torch.Tensor:
+    """act(gate) * up for gate|up interleaved in ``block``-feature blocks (None: [gate | up])."""
     if not gu.is_cuda:
-        r = reference.silu_mul(gu, block)
+        r = reference.silu_mul(gu, block, act == GELU_TANH)
         if out is not None:
             out.copy_(r)
             return out
         return r
     inter = gu.shape[1] // 2
     o = out if out is not None else torch.empty(gu.shape[0], inter, dtype=gu.dtype, device=gu.device)
-    kernels().silu_mul(gu, o, block or 0)
+    kernels().silu_mul(gu, o, block or 0, act)
     return o
 
 
@@ -105,19 +109,19 @@ def _gu_splits(M: int, N: int, K: int) -> int:
     return S
 
 
-def gate_up_silu(x: torch.Tensor, wgu: torch.Tensor, block: int | None) -> torch.Tensor:
-    """silu(x Wg^T) * (x Wu^T) from the interleaved gate|up weight. Decode buckets run
-    one fused gfx950 kernel (GEMM + SwiGLU epilogue, no [M, 2I] intermediate);
+def gate_up_silu(x: torch.Tensor, wgu: torch.Tensor, block: int | None, act: int = SILU) -> torch.Tensor:
+    """act(x Wg^T) * (x Wu^T) from the interleaved gate|up weight (``act``: SILU or GELU_TANH). Decode
+    buckets run one fused gfx950 kernel (GEMM + gated epilogue, no [M, 2I] intermediate);
     other shapes run the GEMM then the silu_mul kernel."""
     M, K = x.shape
     N = wgu.shape[0]
     if x.is_cuda and block == 64 and f32_ok(x, wgu):
-        return linear_f32(x, wgu, silu_gu=True)
+        return linear_f32(x, wgu, glu=act)
     if (x.is_cuda and block == 64 and x.dtype == torch.bfloat16 and M <= SKINNY_MAX_M and N % 128 == 0
             and K % 128 == 0 and x.is_contiguous() and wgu.is_contiguous()
             and skinny_plan(M, N, K) is not None and _gemm_table_get().get(("silu", M, N, K)) != "blas"):
         y = torch.empty(M, N // 2, dtype=x.dtype, device=x.device)
-        kernels().gemm_skinny(x, wgu, y, None, 1, True)
+        kernels().gemm_skinny(x, wgu, y, None, 1, act)
         return y
     if (x.is_cuda and block == 64 and x.dtype == torch.bfloat16 and M % 64 == 0 and M <= 256 and N % 128 == 0
             and K % 64 == 0 and x.is_contiguous() and wgu.is_contiguous()):
@@ -126,23 +130,23 @@ def gate_up_silu(x: torch.Tensor, wgu: torch.Tensor, block: int | None) -> torch
             y = torch.empty(M, N // 2, dtype=x.dtype, device=x.device)
             bm = int(t[2:])
             ws, fl = _pp_sk_workspace(x.device, N // 128) if (bm == 256 and PP_STREAM_K) else (None, None)
-            kernels().gemm_pp(x, wgu, y, None, 1, bm, True, True, False, ws, fl)
+            kernels().gemm_pp(x, wgu, y, None, 1, bm, act, True, False, ws, fl)
             return y
         if t is None and (S := _gu_splits(M, N, K)) > 1:   # too few column tiles to fill the GPU: split K
             y = torch.empty(M, N // 2, dtype=x.dtype, device=x.device)
             slabs = torch.empty(S * M * N, dtype=torch.float32, device=x.device)
             kernels().gemm_decode(x, wgu, None, slabs, S, 128, row_tile(M), False, False, 3)
-            kernels().splitk_silu(slabs, y, S)
+            kernels().splitk_silu(slabs, y, S, act)
             return y
         if t != "blas":
             bm = t[0] if t else row_tile(M)
             ns = t[1] if t and len(t) > 1 else 3
             y = torch.empty(M, N // 2, dtype=x.dtype, device=x.device)
-            kernels().gemm_decode(x, wgu, y, None, 1, 128, bm, True, False, ns)
+            kernels().gemm_decode(x, wgu, y, None, 1, 128, bm, act, False, ns)
             return y
     if block == 64 and tile_ok(x, wgu) and N % 128 == 0:
-        return linear_tile(x, wgu, silu_gu=True)   # prefill: SwiGLU fused into the tile epilogue
-    return silu_mul(linear(x, wgu), block=block)
+        return linear_tile(x, wgu, glu=act)   # prefill: gating fused into the tile epilogue
+    return silu_mul(linear(x, wgu), block=block, act=act)
 
 
 # Stream-K form of the 256-row gate|up+SwiGLU decode GEMM (csrc/kernels/gemm_pp.hip SK): one block per
@@ -421,13 +425,13 @@ def tile_out_ok(out: torch.Tensor | None) -> bool:
 
 
 def linear_tile(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None,
-                bias: torch.Tensor | None = None, silu_gu: bool = False) -> torch.Tensor:
+                bias: torch.Tensor | None = None, glu: int = 0) -> torch.Tensor:
     """Prefill / lm_head GEMM on the compute-bound gfx950 tile kernel (256 x 256 tiles,
-    LDS-DMA ping-pong pipeline; fused bias or SwiGLU epilogue)."""
+    LDS-DMA ping-pong pipeline; fused bias or gated (``glu``: SILU / GELU_TANH) epilogue)."""
     M = x.shape[0]
     N = w.shape[0]
-    y = out if out is not None else torch.empty(M, N // 2 if silu_gu else N, dtype=x.dtype, device=x.device)
-    kernels().gemm_tile(x, w, y, bias, silu_gu)
+    y = out if out is not None else torch.empty(M, N // 2 if glu else N, dtype=x.dtype, device=x.device)
+    kernels().gemm_tile(x, w, y, bias, glu)
     return y
 
 
@@ -437,11 +441,11 @@ def f32_ok(x: torch.Tensor, w: torch.Tensor) -> bool:
             and w.is_contiguous() and x.shape[1] % 16 == 0)
 
 
-def linear_f32(x: torch.Tensor, w: torch.Tensor, silu_gu: bool = False) -> torch.Tensor:
-    """True 32-bit x @ w^T (fp32 FMA), optionally with the SwiGLU epilogue over a 64-row
+def linear_f32(x: torch.Tensor, w: torch.Tensor, glu: int = 0) -> torch.Tensor:
+    """True 32-bit x @ w^T (fp32 FMA), optionally with the gated epilogue (SILU / GELU_TANH) over a 64-row
     interleaved gate|up weight."""
-    y = torch.empty(x.shape[0], w.shape[0] // 2 if silu_gu else w.shape[0], dtype=x.dtype, device=x.device)
-    kernels().gemm_f32(x, w, y, silu_gu)
+    y = torch.empty(x.shape[0], w.shape[0] // 2 if glu else w.shape[0], dtype=x.dtype, device=x.device)
+    kernels().gemm_f32(x, w, y, glu)
     return y
 
 

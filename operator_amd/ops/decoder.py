@@ -1,9 +1,10 @@
 """Ops of decoders beyond the Llama block: hyper-connection residual streams, QKV heads of any
-size with rotary positions and per-head norm, attention over them, routed experts, and the
-fp32 forms of all of them.
+size with rotary positions and per-head norm, heads behind short convolutions, attention over
+them (full or sliding window, with per-head output gates), latent attention, routed experts, and
+the fp32 forms of all of them.
 
 As in :mod:`operator_amd.ops`: GPU tensors go to the gfx950 kernels (csrc/kernels/streams.hip,
-qkv_heads.hip, attn_gd_*.hip, moe.hip, f32.hip), CPU tensors to the fp32 references. Widths,
+qkv_heads.hip, conv_heads.hip, latent.hip, attn_gd_*.hip, attn_latent_decode.hip, moe.hip, f32.hip), CPU tensors to the fp32 references. Widths,
 head sizes and feature counts are stored padded (``pad_to``) with zero weights, so every GEMM
 meets the tile kernels' alignment whatever the model's sizes.
 """
@@ -70,15 +71,19 @@ def stream_init(ids: torch.Tensor, table: torch.Tensor, scale: float, streams: i
 
 
 def stream_step(x: torch.Tensor, o: SublayerOut, hc: Stream, nxt: torch.Tensor | None, w: torch.Tensor, width: int,
-                eps: float, dtype: torch.dtype, rows: torch.Tensor | None = None, write_x: bool = True) -> torch.Tensor:
+                eps: float, dtype: torch.dtype, rows: torch.Tensor | None = None, write_x: bool = True,
+                post_w: torch.Tensor | None = None) -> torch.Tensor:
     """Finish a sublayer (``hc`` with its output ``o``) and return the next one's normalised
     input: ``nxt`` are its stream coefficients, None the plain sum at the model's end, where
-    ``rows`` picks the rows wanted and ``write_x`` False leaves the streams alone."""
+    ``rows`` picks the rows wanted and ``write_x`` False leaves the streams alone. ``post_w``: weight
+    of an RMS norm of the output itself before it joins (one stream)."""
     from . import SplitK
 
     n = x.shape[0] if rows is None else rows.numel()
     if not x.is_cuda:
         y = reference.sublayer_out(o.y, o.gate, o.e, o.epos, o.top, x.shape[0], x.shape[2])
+        if post_w is not None:
+            y = reference.rms_rows(y, post_w, width, eps)
         xn = reference.stream_mix(x, y, hc.mix, hc.out)
         if write_x:
             x.copy_(xn)
@@ -89,7 +94,7 @@ def stream_step(x: torch.Tensor, o: SublayerOut, hc: Stream, nxt: torch.Tensor |
     slab = isinstance(o.y, SplitK)
     kernels().stream_step(x, h, width, w, eps, in_=nxt, y=None if slab else o.y, slabs=o.y.p if slab else None,
                           splits=o.y.S if slab else 1, gate=o.gate, e=o.e, epos=o.epos, top=o.top, mix=hc.mix,
-                          out=hc.out, rows=rows, write_x=write_x)
+                          out=hc.out, rows=rows, write_x=write_x, post_w=post_w)
     return h
 
 
@@ -167,14 +172,18 @@ def _o_rows(T: int, L: HeadLayout, dtype, dev) -> torch.Tensor:
 
 
 def attn_gd_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, seq_lens: list[int], L: HeadLayout, scale: float,
-                    work: tuple | None = None, prefix: tuple | None = None) -> torch.Tensor:
-    """Causal attention over packed sequences -> [T, ocol] rows for the o-projection.
+                    work: tuple | None = None, prefix: tuple | None = None, window: int = 0,
+                    gate: torch.Tensor | None = None) -> torch.Tensor:
+    """Causal attention over packed sequences -> [T, ocol] rows for the o-projection. ``window``: a
+    query sees keys less than that far back (0: all); ``gate`` [T, H] fp32 scales every head's output.
     ``work`` = (cu_seqlens, work_seq, work_q0, GD_VARIANT); ``prefix`` as in ``attn_prefill``."""
     if not q.is_cuda:
         cu = [0]
         for n in seq_lens:
             cu.append(cu[-1] + int(n))
-        r = reference.attn_prefill(q, k, v, cu, scale, prefix=None if prefix is None else (prefix[0], prefix[1], prefix[3]))
+        r = reference.attn_prefill(q, k, v, cu, scale, prefix=None if prefix is None else (prefix[0], prefix[1], prefix[3]),
+                                   window=window)
+        r = r if gate is None else (r.float() * gate[..., None]).to(r.dtype)
         o = torch.zeros(q.shape[0], L.ocol, dtype=q.dtype)
         o[:, :L.heads * L.pads[1]] = r.reshape(q.shape[0], -1)
         return o
@@ -190,7 +199,7 @@ def attn_gd_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, seq_lens:
         raise ValueError("attn_gd_prefill needs a work list cut at GD_BLOCK_Q rows")
     o = _o_rows(q.shape[0], L, q.dtype, q.device)
     pk, pv, sp = (None, None, None) if prefix is None else prefix[:3]
-    kernels().attn_gd_prefill(q, k, v, o, work[0], work[1], work[2], scale, pk, pv, sp)
+    kernels().attn_gd_prefill(q, k, v, o, work[0], work[1], work[2], scale, pk, pv, sp, window, gate)
     return o
 
 
@@ -198,16 +207,19 @@ def attn_gd_workspace(B: int, layouts, num_splits: int, device):
     """fp32 partials of split decode attention, shared by a model's layers (None: one split)."""
     if num_splits <= 1:
         return None
-    n = max(B * L.heads * num_splits * L.pads[1] for L in layouts)
+    n = max(B * L.heads * num_splits * (L.rp if isinstance(L, LatentLayout) else L.pads[1]) for L in layouts)
     m = max(B * L.heads * num_splits * 2 for L in layouts)
     return (torch.empty(n, dtype=torch.float32, device=device), torch.empty(m, dtype=torch.float32, device=device))
 
 
 def attn_gd_decode(q: torch.Tensor, cache: tuple, block_tables: torch.Tensor, seq_lens: torch.Tensor, L: HeadLayout,
-                   scale: float, num_splits: int = 1, workspace: tuple | None = None) -> torch.Tensor:
-    """One query token per sequence over the paged cache -> [B, ocol] rows."""
+                   scale: float, num_splits: int = 1, workspace: tuple | None = None, window: int = 0,
+                   gate: torch.Tensor | None = None) -> torch.Tensor:
+    """One query token per sequence over the paged cache -> [B, ocol] rows (``window``, ``gate``: as in
+    ``attn_gd_prefill``)."""
     if not q.is_cuda:
-        r = reference.attn_decode_rows(q, cache[0], cache[1], block_tables, seq_lens, scale)
+        r = reference.attn_decode_rows(q, cache[0], cache[1], block_tables, seq_lens, scale, window)
+        r = r if gate is None else (r.float() * gate[..., None]).to(r.dtype)
         o = torch.zeros(q.shape[0], L.ocol, dtype=q.dtype)
         o[:, :L.heads * L.pads[1]] = r.reshape(q.shape[0], -1)
         return o
@@ -215,7 +227,175 @@ def attn_gd_decode(q: torch.Tensor, cache: tuple, block_tables: torch.Tensor, se
     if num_splits > 1 and workspace is None:
         workspace = attn_gd_workspace(q.shape[0], [L], num_splits, q.device)
     ws = workspace if num_splits > 1 else (None, None)
-    kernels().attn_gd_decode(q, cache[0], cache[1], block_tables, seq_lens, o, ws[0], ws[1], num_splits, scale)
+    kernels().attn_gd_decode(q, cache[0], cache[1], block_tables, seq_lens, o, ws[0], ws[1], num_splits, scale, window, gate)
+    return o
+
+
+# ---------------------------------------------------------------- heads behind short convolutions
+@dataclass
+class SequenceEdges:
+    """Where a step's rows stand in their sequences. A prefill has ``cu`` (device, the GPU) /
+    ``lens`` (host, the CPU) of its packed sequences and ``prev_pages`` [S] int32, the page of the
+    tokens before a sequence's first row (-1 or None: there are none); a decode step ``block_tables``."""
+    cu: torch.Tensor | None = None
+    lens: list | None = None
+    prev_pages: torch.Tensor | None = None
+    block_tables: torch.Tensor | None = None
+
+
+def conv_ncol(L: HeadLayout) -> int:
+    """Columns of a packed query | key | gate projection."""
+    return pad_to((L.heads + L.kv_heads) * L.pads[0] + L.heads, 64)
+
+
+def conv_heads(x, pos: torch.Tensor, L: HeadLayout, dtype: torch.dtype, conv: torch.Tensor, qw: torch.Tensor, kw: torch.Tensor,
+               cache: tuple, tails: torch.Tensor | None, slots: torch.Tensor, edges: SequenceEdges):
+    """Packed q | k | gate rows (or SplitK slabs) -> (q [T, H, dk], k [T, G, dk], v [T, G, dv], gate [T, H]
+    fp32): q and k through the short causal convolution ``conv`` [taps, (H + G) dk] and a weighted
+    per-head RMS norm, v the convolved key without the norm, gate the sigmoid. k / v (None at decode)
+    also go to the paged ``cache``, and the last taps - 1 projected rows to ``tails`` [pages, taps - 1, C]."""
+    from . import SplitK
+
+    T, dev = pos.numel(), pos.device
+    dk, dv = L.pads
+    if not pos.is_cuda:
+        q, k, v, gate = reference.conv_heads(x, pos, L, conv, qw, kw, tails, slots, edges, cache[0].shape[2])
+        q, k, v = q.to(dtype), k.to(dtype), v.to(dtype)
+        reference.cache_rows(cache[0], cache[1], k, v, slots)
+        return q, k, v, gate
+    prefill = edges.block_tables is None
+    q = torch.empty(T, L.heads, dk, dtype=dtype, device=dev)
+    k = torch.empty(T, L.kv_heads, dk, dtype=dtype, device=dev) if prefill else None
+    v = torch.empty(T, L.kv_heads, dv, dtype=dtype, device=dev) if prefill else None
+    gate = torch.empty(T, L.heads, dtype=torch.float32, device=dev)
+    slab = isinstance(x, SplitK)
+    kernels().conv_heads(q if slab else x, x.p if slab else None, x.S if slab else 1, conv, qw, kw, pos, L.dim, L.eps, q, k, v,
+                         cache[0], cache[1], slots, tails, gate, conv_ncol(L), edges.cu if prefill else None,
+                         edges.prev_pages if prefill else None, edges.block_tables)
+    return q, k, v, gate
+
+
+# ---------------------------------------------------------------- latent attention
+@dataclass(frozen=True)
+class LatentLayout:
+    """Shapes of one latent-attention layer (true sizes): ``heads`` of ``dim`` unrotated and ``rot``
+    rotated query / key dimensions and ``vdim`` value ones, queries from a latent of ``q_rank``, keys
+    and values from one of ``kv_rank``; ``own`` False: it reads another layer's latent rows."""
+    heads: int
+    dim: int
+    rot: int
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    own: bool = True
+    eps: float = 1e-6
+
+    @property
+    def pads(self) -> tuple[int, int]:
+        """Stored sizes of an expanded query / key head and a value head."""
+        return head_pads(self.dim + self.rot, self.vdim)
+
+    @property
+    def qp(self) -> int:
+        return max(128, pad_to(self.q_rank, 64))
+
+    @property
+    def rp(self) -> int:
+        return pad_to(self.kv_rank, 32)
+
+    @property
+    def rotp(self) -> int:
+        return pad_to(self.rot, 8)
+
+    @property
+    def ck(self) -> int:
+        """Columns of a cached row: latent (rp), rotated part, zeros."""
+        return max(128, pad_to(self.rp + self.rot, 64))
+
+    @property
+    def ncol(self) -> int:
+        """Columns of the packed projection: query latent, latent, rotated part, gates."""
+        return pad_to(self.qp + (self.rp + self.rotp if self.own else 0) + self.heads, 64)
+
+    @property
+    def ocol(self) -> int:
+        return pad_to(self.heads * self.pads[1], 64)
+
+
+def latent_rows(x, pos: torch.Tensor, rot: tuple, L: LatentLayout, dtype: torch.dtype, qw: torch.Tensor, cw: torch.Tensor | None,
+                cache: torch.Tensor | None, slots: torch.Tensor):
+    """Packed projection -> (normed query latent [T, qp], gate [T, H] fp32, latent rows [T, ck] | None); the
+    rows also go to the paged ``cache`` [pages, 1, P, ck]."""
+    from . import SplitK
+
+    T, dev = pos.numel(), pos.device
+    if not pos.is_cuda:
+        return reference.latent_rows(x, pos, rot, L, dtype, qw, cw, cache, slots)
+    cq = torch.empty(T, L.qp, dtype=dtype, device=dev)
+    gate = torch.empty(T, L.heads, dtype=torch.float32, device=dev)
+    lat = torch.empty(T, L.ck, dtype=dtype, device=dev) if L.own else None
+    slab = isinstance(x, SplitK)
+    kernels().latent_rows(cq if slab else x, x.p if slab else None, x.S if slab else 1, L.ncol, L.q_rank, L.kv_rank, L.rp, L.rot,
+                          L.rotp, qw, cw, L.eps, pos, rot[0], rot[1], cq, lat, cache if L.own else None, slots if L.own else None, gate)
+    return cq, gate, lat
+
+
+def rotate_heads(q, pos: torch.Tensor, rot: tuple, L: LatentLayout, dtype: torch.dtype) -> torch.Tensor:
+    """Query heads [T, H dk] (rows, rotated in place, or SplitK slabs) -> [T, H, dk] with the columns dim ..
+    dim + rot of every head rotated (first half paired with the second)."""
+    from . import SplitK
+
+    T, dk = pos.numel(), L.pads[0]
+    if not pos.is_cuda:
+        return reference.rotate_heads(q.view(T, L.heads, dk), pos, rot, L.dim, L.rot).to(dtype)
+    slab = isinstance(q, SplitK)
+    out = torch.empty(T, L.heads, dk, dtype=dtype, device=pos.device) if slab else q.view(T, L.heads, dk)
+    kernels().rotate_heads(out, q.p if slab else None, q.S if slab else 1, L.dim, L.rot, pos, rot[0], rot[1])
+    return out
+
+
+def to_latent(q: torch.Tensor, w: torch.Tensor, L: LatentLayout) -> torch.Tensor:
+    """Decode queries in the space of the cached rows: [B, H, dk] -> [B, H, ck], ``w`` [H, rp, pad16(dim)] the
+    transposed key expansion of every head."""
+    if not q.is_cuda:
+        y = torch.zeros(q.shape[0], L.heads, L.ck, dtype=q.dtype)
+        y[..., :L.rp] = reference.head_gemm(q[..., :w.shape[2]], w)
+        y[..., L.rp:L.rp + L.rot] = q[..., L.dim:L.dim + L.rot]
+        return y
+    if q.dtype == torch.float32:
+        y = torch.zeros(q.shape[0], L.heads, L.ck, dtype=q.dtype, device=q.device)
+        kernels().head_gemm(q, w, y)
+        y[..., L.rp:L.rp + L.rot] = q[..., L.dim:L.dim + L.rot]
+        return y
+    y = torch.empty(q.shape[0], L.heads, L.ck, dtype=q.dtype, device=q.device)
+    kernels().head_gemm(q, w, y, L.dim, L.rot)
+    return y
+
+
+def from_latent(o: torch.Tensor, w: torch.Tensor, L: LatentLayout) -> torch.Tensor:
+    """Attention outputs in the latent space [B, H, rp] -> [B, ocol] rows of values (``w`` [H, dv, rp])."""
+    y = _o_rows(o.shape[0], L, o.dtype, o.device)
+    if not o.is_cuda:
+        y[:, :L.heads * L.pads[1]] = reference.head_gemm(o, w).reshape(o.shape[0], -1)
+        return y
+    kernels().head_gemm(o, w, y)
+    return y
+
+
+def attn_latent_decode(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, seq_lens: torch.Tensor, L: LatentLayout,
+                       scale: float, num_splits: int = 1, workspace: tuple | None = None,
+                       gate: torch.Tensor | None = None) -> torch.Tensor:
+    """One query token per sequence over cached latent rows: [B, H, rp] sums of the latents, gated."""
+    if not q.is_cuda:
+        r = reference.attn_decode_rows(q, cache, cache[..., :L.rp], block_tables, seq_lens, scale)
+        return r if gate is None else (r.float() * gate[..., None]).to(r.dtype)
+    o = torch.empty(q.shape[0], L.heads, L.rp, dtype=q.dtype, device=q.device)
+    if num_splits > 1 and workspace is None:
+        n = q.shape[0] * L.heads * num_splits
+        workspace = (torch.empty(n * L.rp, dtype=torch.float32, device=q.device),
+                     torch.empty(2 * n, dtype=torch.float32, device=q.device))
+    ws = workspace if num_splits > 1 else (None, None)
+    kernels().attn_latent_decode(q, cache, block_tables, seq_lens, o.view(q.shape[0], -1), L.rp, ws[0], ws[1], num_splits, scale, gate)
     return o
 
 

@@ -24,8 +24,8 @@ def rmsnorm(x: torch.Tensor, w: torch.Tensor, eps: float, residual: torch.Tensor
     return (y.float() * w.float()).to(x.dtype), new_res
 
 
-def silu_mul(gu: torch.Tensor, block: int | None = None) -> torch.Tensor:
-    """silu(gate) * up; gate|up columns interleaved in blocks of ``block`` features
+def silu_mul(gu: torch.Tensor, block: int | None = None, gelu: bool = False) -> torch.Tensor:
+    """silu(gate) * up (``gelu``: tanh-gelu instead); gate|up columns interleaved in blocks of ``block`` features
     (None: the plain [gate | up] concatenation)."""
     inter = gu.shape[-1] // 2
     if block and block != inter:
@@ -33,7 +33,8 @@ def silu_mul(gu: torch.Tensor, block: int | None = None) -> torch.Tensor:
         g, u = v[..., 0, :].reshape(*gu.shape[:-1], inter), v[..., 1, :].reshape(*gu.shape[:-1], inter)
     else:
         g, u = gu[..., :inter], gu[..., inter:]
-    s = torch.nn.functional.silu(g.float()).to(gu.dtype)
+    F = torch.nn.functional
+    s = (F.gelu(g.float(), approximate="tanh") if gelu else F.silu(g.float())).to(gu.dtype)
     return (s.float() * u.float()).to(gu.dtype)
 
 
@@ -143,10 +144,11 @@ def rope_kv(qkv: torch.Tensor, pos: torch.Tensor, cos: torch.Tensor, sin: torch.
 
 
 def attn_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, cu_seqlens: list[int] | torch.Tensor,
-                 scale: float, prefix: tuple | None = None) -> torch.Tensor:
+                 scale: float, prefix: tuple | None = None, window: int = 0) -> torch.Tensor:
     """Causal GQA attention over packed variable-length sequences. q [T,Hq,D], k/v [T,Hkv,D].
     ``prefix`` = (pk, pv, lens): sequence i's keys start with the rows pk[:lens[i]] /
-    pv[:lens[i]] (a cached shared prompt prefix), visible to all of its query rows."""
+    pv[:lens[i]] (a cached shared prompt prefix), visible to all of its query rows. ``window``: only
+    keys less than that far back (0: all)."""
     cu = [int(x) for x in cu_seqlens]
     Hq, Hkv = q.shape[1], k.shape[1]
     G = Hq // Hkv
@@ -167,6 +169,9 @@ def attn_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, cu_seqlens: 
         mask = torch.ones(L, L, dtype=torch.bool, device=q.device).triu(1)
         if pl:
             mask = torch.cat([torch.zeros(L, pl, dtype=torch.bool, device=q.device), mask], 1)
+        if window:
+            i, j = torch.arange(L, device=q.device)[:, None] + pl, torch.arange(L + pl, device=q.device)[None]
+            mask |= i - j >= window
         s.masked_fill_(mask, float("-inf"))
         p = torch.softmax(s, -1)
         out[a:b] = torch.matmul(p, vs).transpose(0, 1).to(q.dtype)
@@ -309,8 +314,9 @@ def cache_rows(k_cache: torch.Tensor, v_cache: torch.Tensor, k: torch.Tensor, v:
 
 
 def attn_decode_rows(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
-                     seq_lens: torch.Tensor, scale: float) -> torch.Tensor:
-    """One query token per sequence over a token-row paged cache; keys and values of any size."""
+                     seq_lens: torch.Tensor, scale: float, window: int = 0) -> torch.Tensor:
+    """One query token per sequence over a token-row paged cache; keys and values of any size
+    (``window``: the last that many tokens only)."""
     B, Hq, _ = q.shape
     Hkv, P = k_cache.shape[1], k_cache.shape[2]
     out = torch.zeros(B, Hq, v_cache.shape[3], dtype=q.dtype, device=q.device)
@@ -321,9 +327,83 @@ def attn_decode_rows(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         pages = block_tables[b, :(n + P - 1) // P].long()
         k = k_cache[pages].permute(1, 0, 2, 3).reshape(Hkv, -1, k_cache.shape[3])[:, :n].float()
         v = v_cache[pages].permute(1, 0, 2, 3).reshape(Hkv, -1, v_cache.shape[3])[:, :n].float()
+        a = max(0, n - window) if window else 0
+        k, v = k[:, a:], v[:, a:]
         s = torch.matmul(q[b].float().view(Hkv, Hq // Hkv, -1), k.transpose(1, 2)) * scale
         out[b] = torch.matmul(torch.softmax(s, -1), v).reshape(Hq, -1).to(q.dtype)
     return out
+
+
+def rms_rows(x: torch.Tensor, w: torch.Tensor, width: int, eps: float) -> torch.Tensor:
+    """Weighted RMS norm of zero-padded rows whose true width is ``width``; fp32."""
+    x = x.float()
+    return x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) / width + eps) * w
+
+
+def conv_heads(x: torch.Tensor, pos: torch.Tensor, L, conv: torch.Tensor, qw: torch.Tensor, kw: torch.Tensor, tails,
+               slots: torch.Tensor, edges, P: int):
+    """fp32 (q, k, v, gate) of packed q | k | gate rows; ``tails`` (the last projected rows of every page's
+    tokens, entry position % (taps - 1)) is read before and written after."""
+    dk, dv = L.pads
+    H, G, R = L.heads, L.kv_heads, conv.shape[0] - 1
+    C = (H + G) * dk
+    u = x[:, :C].float()
+    y = torch.zeros_like(u)
+    T = u.shape[0]
+    start, pages, ends = list(range(T)), [-1] * T, list(range(1, T + 1))
+    if edges.block_tables is None:
+        t = 0
+        for s, n in enumerate(edges.lens):
+            pg = -1 if edges.prev_pages is None else int(edges.prev_pages[s])
+            start[t:t + n], pages[t:t + n], ends[t:t + n] = [t] * n, [pg] * n, [t + n] * n
+            t += n
+    for t in range(T):
+        p = int(pos[t])
+        for d in range(min(R, p) + 1):
+            if t - d >= start[t]:
+                v = u[t - d]
+            else:
+                pg = pages[t] if edges.block_tables is None else int(edges.block_tables[t, (p - d) // P])
+                if pg < 0:
+                    continue
+                v = tails[pg, (p - d) % R].float()
+            y[t] += conv[R - d] * v
+    for t in range(T):
+        if R and int(slots[t]) >= 0 and t + R >= ends[t]:
+            tails[int(slots[t]) // P, int(pos[t]) % R] = u[t].to(tails.dtype)
+    q, k = y[:, :H * dk].view(T, H, dk), y[:, H * dk:].view(T, G, dk)
+    v = torch.zeros(T, G, dv)
+    v[..., :dk] = k
+    return rms_rows(q, qw, L.dim, L.eps), rms_rows(k, kw, L.dim, L.eps), v, torch.sigmoid(x[:, C:C + H].float())
+
+
+def rotate_heads(x: torch.Tensor, pos: torch.Tensor, rot: tuple, at: int, dims: int) -> torch.Tensor:
+    """fp32 x [T, H, d] with columns at .. at + dims rotated, i paired with i + dims / 2."""
+    y, n = x.float().clone(), dims // 2
+    c, s = rot[0][pos][:, None, :n], rot[1][pos][:, None, :n]
+    a, b = x[..., at:at + n].float(), x[..., at + n:at + 2 * n].float()
+    y[..., at:at + n], y[..., at + n:at + 2 * n] = a * c - b * s, b * c + a * s
+    return y
+
+
+def latent_rows(x: torch.Tensor, pos: torch.Tensor, rot: tuple, L, dtype, qw, cw, cache, slots):
+    T = x.shape[0]
+    cq = rms_rows(x[:, :L.qp], qw, L.q_rank, L.eps).to(dtype)
+    at, lat = L.qp, None
+    if L.own:
+        lat = torch.zeros(T, L.ck, dtype=dtype)
+        lat[:, :L.rp] = rms_rows(x[:, at:at + L.rp], cw, L.kv_rank, L.eps).to(dtype)
+        at += L.rp
+        lat[:, L.rp:L.rp + L.rot] = rotate_heads(x[:, None, at:at + L.rot], pos, rot, 0, L.rot)[:, 0].to(dtype)
+        at += L.rotp
+        P, ok = cache.shape[2], slots >= 0
+        cache[slots[ok] // P, 0, slots[ok] % P] = lat[ok]
+    return cq, torch.sigmoid(x[:, at:at + L.heads].float()), lat
+
+
+def head_gemm(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """y[m, h] = x[m, h] w[h]^T."""
+    return torch.matmul(x.float().transpose(0, 1), w.float().transpose(1, 2)).transpose(0, 1).to(x.dtype)
 
 
 def route(h: torch.Tensor, wr: torch.Tensor, experts: int, top: int, gated: bool):
