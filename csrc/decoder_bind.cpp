@@ -413,19 +413,20 @@ void conv_heads(const at::Tensor& x, const OptT& slabs, int64_t splits, const at
   const int64_t taps = conv.size(0), C = (Hq + Hkv) * dkp, pages = k_cache.size(0), P = k_cache.size(2);
   need(pos, at::kLong, T, "pos");
   need(q_out, dt, T * Hq * dkp, "q_out");
-  need(conv, at::kFloat, taps * C, "conv");
-  need(qw, at::kFloat, dkp, "q norm weight");
-  need(kw, at::kFloat, dkp, "k norm weight");
+  need(conv, dt, taps * C, "conv");
+  need(qw, dt, dkp, "q norm weight");
+  need(kw, dt, dkp, "k norm weight");
   need(gate, at::kFloat, T * Hq, "gate");
   need(slots, at::kLong, T, "slots");
   need(k_cache, dt, pages * Hkv * P * dkp, "k_cache");
   need(v_cache, dt, pages * Hkv * P * dvp, "v_cache");
   TORCH_CHECK(dk >= 1 && dk <= dkp && dvp >= dkp && ncol >= C + Hq && ncol % 8 == 0 && P >= taps - 1, "conv_heads: sizes");
   oamd::ConvHeads a{};
+  a.T = (int)T;
   set_rows(a, x, slabs, splits, T, ncol, dt);
   a.ncol = (int)ncol;
   a.taps = (int)taps;
-  a.conv = p<float>(conv); a.qw = p<float>(qw); a.kw = p<float>(kw);
+  a.conv = conv.data_ptr(); a.qw = qw.data_ptr(); a.kw = kw.data_ptr();
   a.pos = p<int64_t>(pos);
   a.Hq = (int)Hq; a.Hkv = (int)Hkv; a.dk = (int)dk; a.dkp = (int)dkp; a.dvp = (int)dvp;
   a.eps = (float)eps;
@@ -462,7 +463,7 @@ void conv_heads(const at::Tensor& x, const OptT& slabs, int64_t splits, const at
   a.log2_page = page_log2(P);
   a.gate = p<float>(gate);
   const c10::hip::HIPGuardMasqueradingAsCUDA g(pos.device());
-  RC(oamd::conv_heads(a, (int)T, f32, cur_stream()));
+  RC(oamd::conv_heads(a, f32, cur_stream()));
 }
 
 // lat / cache absent: the layer reads another layer's latent rows

@@ -29,7 +29,7 @@ __device__ __forceinline__ s16x4 tr16(const char* p) {
 
 // DK, DV: instantiated sizes >= the stored sizes dkp, dvp (the rest is zero in LDS)
 template <int DK, int DV>
-__global__ void __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) attn_gd_prefill_kernel(const AttnPrefill a) {
+__global__ void __launch_bounds__(256, (DK + DV <= 320) ? 2 : 1) attn_gd_prefill_kernel(const AttnPrefill a) {
   constexpr int BK = 64, RK = 2 * DK + 16;       // K rows padded by 16 B: conflict-free row reads
   constexpr int RV = DV <= 128 ? 256 : 512;      // V rows: the 16-chunk swizzle below needs 256-B rows
   constexpr int CK = DK / 8, CV = DV / 8;
@@ -38,15 +38,22 @@ __global__ void __launch_bounds__(256, (DK + DV <= 256) ? 2 : 1) attn_gd_prefill
   __shared__ __attribute__((aligned(16))) char Ks[BK * RK];
   __shared__ __attribute__((aligned(16))) char Vs[BK * RV];
 
-  const int wi = blockIdx.x;
+  int wi = blockIdx.x, by = blockIdx.y, bz = blockIdx.z;
+  if (gridDim.y % 8 == 0) {   // a head's workgroups on one XCD, an item's sub-blocks next to each other
+    const int L = blockIdx.x + gridDim.x * (blockIdx.y + gridDim.y * blockIdx.z);
+    const int j = L >> 3;
+    bz = j % gridDim.z;
+    wi = j / gridDim.z % gridDim.x;
+    by = j / gridDim.z / gridDim.x * 8 + (L & 7);
+  }
   const int seq = a.work_seq[wi];
   if (seq < 0) return;   // padding item of a graph-captured prefill (fixed grid)
   const int GC = a.gc, nch = a.G / GC;
-  const int kvh = blockIdx.y / nch, hc = blockIdx.y % nch;
+  const int kvh = by / nch, hc = by % nch;
   const int RG = 4 / GC, BQ = 32 * RG;
   const int s0 = a.cu_seqlens[seq];
   const int slen = a.cu_seqlens[seq + 1] - s0;
-  const int q0 = a.work_q0[wi] + (int)blockIdx.z * BQ;
+  const int q0 = a.work_q0[wi] + bz * BQ;
   if (q0 >= slen) return;
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r32 = lane & 31, h = lane >> 5;

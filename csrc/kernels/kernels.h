@@ -239,14 +239,15 @@ int attn_latent_decode(const AttnDecode& a, int B, int rp, hipStream_t stream);
 
 // Short-convolution heads (conv_heads.hip)
 struct ConvHeads {
+  int T;                    // tokens
   const float* xp;          // S fp32 slabs [S][T][ncol], slab elements apart, or nullptr
   int S;
   int64_t slab;
   const void* row;          // [T][ncol] rows (bf16 / fp32): q | k | gate logits
   int ncol;
   int taps;                 // 1..8
-  const float* conv;        // [taps][(Hq + Hkv) dkp], last row: the current token's weight
-  const float *qw, *kw;     // [dkp] norm weights, zero past dk
+  const void* conv;         // [taps][(Hq + Hkv) dkp], last row: the current token's weight (row type)
+  const void *qw, *kw;      // [dkp] norm weights, zero past dk (row type)
   const int64_t* pos;
   int Hq, Hkv, dk, dkp, dvp;
   float eps;
@@ -263,7 +264,7 @@ struct ConvHeads {
   int log2_page;
   float* gate;              // [T][Hq] sigmoid gates
 };
-int conv_heads(const ConvHeads& a, int tokens, bool f32, hipStream_t stream);
+int conv_heads(const ConvHeads& a, bool f32, hipStream_t stream);
 
 // Latent attention (latent.hip)
 struct LatentRows {

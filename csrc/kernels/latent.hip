@@ -16,18 +16,20 @@ typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
 }  // namespace
 
-// One workgroup of 256 per token; a segment of n padded columns is 8-column chunks tid, tid + 256, ...
-template <typename T, int MAXC>
-__global__ void __launch_bounds__(256) latent_rows_kernel(const LatentRows a) {
-  __shared__ float scratch[4];
-  const int t = xcd_remap(blockIdx.x, gridDim.x), tid = threadIdx.x;
+// NT threads per token (256: a workgroup, for few tokens; 64: a wave); a segment of n padded columns is
+// 8-column chunks tid, tid + NT, ...
+template <typename T, int NT, int MAXC>
+__global__ void __launch_bounds__(256) latent_rows_kernel(const LatentRows a, int tokens) {
+  __shared__ float scratch[8];
+  const int t = xcd_remap(blockIdx.x, gridDim.x) * (256 / NT) + threadIdx.x / NT, tid = threadIdx.x % NT;
+  if (NT == 64 && t >= tokens) return;   // whole waves, and no barrier follows
   const int64_t row = (int64_t)t * a.ncol;
   const int nq = a.qp >> 3, nc = a.lat ? a.rp >> 3 : 0;
   float x[MAXC][8];
   float sq = 0.f, sc = 0.f;
 #pragma unroll
   for (int i = 0; i < MAXC; ++i) {
-    const int ch = tid + 256 * i;   // query latent chunks, then latent chunks
+    const int ch = tid + NT * i;   // query latent chunks, then latent chunks
     if (ch >= nq + nc) continue;
     load_row8<T>(a.xp, a.row, a.S, a.slab, row + 8 * ch, x[i]);
     float s = 0.f;
@@ -36,20 +38,50 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(const LatentRows a) {
     if (ch < nq) sq += s;
     else sc += s;
   }
-  sq = block_sum<256>(sq, scratch);
-  const float rq = 1.f / sqrtf(sq / static_cast<float>(a.q_rank) + a.eps);
-  float rc = 0.f;
-  if (nc) {
-    sc = block_sum<256>(sc, scratch);
-    rc = 1.f / sqrtf(sc / static_cast<float>(a.kv_rank) + a.eps);
-  }
   const int64_t slot = nc && a.slots ? a.slots[t] : -1;
   T* cq = static_cast<T*>(a.cq) + (int64_t)t * a.qp;
   T* lat = nc ? static_cast<T*>(a.lat) + (int64_t)t * a.ck : nullptr;
   T* kept = slot >= 0 ? static_cast<T*>(a.cache) + slot * a.ck : nullptr;   // page rows are contiguous: slot = page * P + token
+  const int after = a.qp + (nc ? a.rp + a.rotp : 0);
+  if (nc) {
+    const int half = a.rot >> 1;
+    int64_t p = a.pos[t];
+    p = p < 0 ? 0 : (p >= a.max_pos ? a.max_pos - 1 : p);
+    for (int i = tid; i < half; i += NT) {
+      const int64_t at = row + a.qp + a.rp + i;
+      const float u = load_row1<T>(a.xp, a.row, a.S, a.slab, at), v = load_row1<T>(a.xp, a.row, a.S, a.slab, at + half);
+      float o1, o2;
+      rope_pair(u, v, a.cos_t[p * a.rot_ld + i], a.sin_t[p * a.rot_ld + i], o1, o2);
+      st1<T>(lat + a.rp + i, o1);
+      st1<T>(lat + a.rp + half + i, o2);
+      if (kept) {
+        st1<T>(kept + a.rp + i, o1);
+        st1<T>(kept + a.rp + half + i, o2);
+      }
+    }
+    for (int i = a.rp + a.rot + tid; i < a.ck; i += NT) {
+      st1<T>(lat + i, 0.f);
+      if (kept) st1<T>(kept + i, 0.f);
+    }
+  }
+  for (int h = tid; h < a.H; h += NT)
+    a.gate[(int64_t)t * a.H + h] = 1.f / (1.f + expf(-load_row1<T>(a.xp, a.row, a.S, a.slab, row + after + h)));
+  sq = wave_sum(sq);   // both sums in one exchange
+  sc = wave_sum(sc);
+  if constexpr (NT == 256) {
+    if ((tid & 63) == 0) {
+      scratch[tid >> 6] = sq;
+      scratch[4 + (tid >> 6)] = sc;
+    }
+    __syncthreads();
+    sq = scratch[0] + scratch[1] + scratch[2] + scratch[3];
+    sc = scratch[4] + scratch[5] + scratch[6] + scratch[7];
+  }
+  const float rq = 1.f / sqrtf(sq / static_cast<float>(a.q_rank) + a.eps);
+  const float rc = nc ? 1.f / sqrtf(sc / static_cast<float>(a.kv_rank) + a.eps) : 0.f;
 #pragma unroll
   for (int i = 0; i < MAXC; ++i) {
-    const int ch = tid + 256 * i;
+    const int ch = tid + NT * i;
     if (ch >= nq + nc) continue;
     float w[8];
     ld8<float>(ch < nq ? a.qw + 8 * ch : a.cw + 8 * (ch - nq), w);
@@ -63,30 +95,6 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(const LatentRows a) {
       if (kept) st8<T>(kept + 8 * (ch - nq), x[i]);
     }
   }
-  const int after = a.qp + (nc ? a.rp + a.rotp : 0);
-  if (nc) {
-    const int half = a.rot >> 1;
-    int64_t p = a.pos[t];
-    p = p < 0 ? 0 : (p >= a.max_pos ? a.max_pos - 1 : p);
-    for (int i = tid; i < half; i += 256) {
-      const int64_t at = row + a.qp + a.rp + i;
-      const float u = load_row1<T>(a.xp, a.row, a.S, a.slab, at), v = load_row1<T>(a.xp, a.row, a.S, a.slab, at + half);
-      float o1, o2;
-      rope_pair(u, v, a.cos_t[p * a.rot_ld + i], a.sin_t[p * a.rot_ld + i], o1, o2);
-      st1<T>(lat + a.rp + i, o1);
-      st1<T>(lat + a.rp + half + i, o2);
-      if (kept) {
-        st1<T>(kept + a.rp + i, o1);
-        st1<T>(kept + a.rp + half + i, o2);
-      }
-    }
-    for (int i = a.rp + a.rot + tid; i < a.ck; i += 256) {
-      st1<T>(lat + i, 0.f);
-      if (kept) st1<T>(kept + i, 0.f);
-    }
-  }
-  for (int h = tid; h < a.H; h += 256)
-    a.gate[(int64_t)t * a.H + h] = 1.f / (1.f + expf(-load_row1<T>(a.xp, a.row, a.S, a.slab, row + after + h)));
 }
 
 int latent_rows(const LatentRows& a, int tokens, bool f32, hipStream_t stream) {
@@ -94,13 +102,13 @@ int latent_rows(const LatentRows& a, int tokens, bool f32, hipStream_t stream) {
   if (a.qp % 8 || a.rp % 8 || a.rot % 2 || a.rot > a.rotp || a.rp + a.rot > a.ck || a.H < 1) return -1;
   const int chunks = a.qp / 8 + (a.lat ? a.rp / 8 : 0);
   if (chunks > 1024) return -2;
-  if (f32) {
-    if (chunks <= 256) latent_rows_kernel<float, 1><<<tokens, 256, 0, stream>>>(a);
-    else latent_rows_kernel<float, 4><<<tokens, 256, 0, stream>>>(a);
-  } else {
-    if (chunks <= 256) latent_rows_kernel<bf16_t, 1><<<tokens, 256, 0, stream>>>(a);
-    else latent_rows_kernel<bf16_t, 4><<<tokens, 256, 0, stream>>>(a);
-  }
+  const bool wave = tokens >= 1024;
+#define OAMD_LATENT(T)                                                                                  \
+  if (wave && chunks <= 256) latent_rows_kernel<T, 64, 4><<<(tokens + 3) / 4, 256, 0, stream>>>(a, tokens);  \
+  else if (chunks <= 256) latent_rows_kernel<T, 256, 1><<<tokens, 256, 0, stream>>>(a, tokens);         \
+  else latent_rows_kernel<T, 256, 4><<<tokens, 256, 0, stream>>>(a, tokens)
+  if (f32) { OAMD_LATENT(float); } else { OAMD_LATENT(bf16_t); }
+#undef OAMD_LATENT
   OAMD_LAUNCH_CHECK();
   return 0;
 }

@@ -34,6 +34,39 @@ __device__ __forceinline__ void ld8<bf16_t>(const bf16_t* p, float (&v)[8]) {
   for (int j = 0; j < 8; ++j) v[j] = bf2f(a[j]);
 }
 
+// eight elements kept as they are stored
+template <typename T>
+struct Raw8;
+template <>
+struct Raw8<float> {
+  float v[8];
+};
+template <>
+struct Raw8<bf16_t> {
+  u16x8 v;
+};
+__device__ __forceinline__ float raw_at(const Raw8<float>& r, int j) { return r.v[j]; }
+__device__ __forceinline__ float raw_at(const Raw8<bf16_t>& r, int j) { return bf2f(r.v[j]); }
+template <typename T>
+__device__ __forceinline__ Raw8<T> raw_zero() {
+  Raw8<T> r;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) r.v[j] = 0;
+  return r;
+}
+template <typename T>
+__device__ __forceinline__ Raw8<T> raw_ld(const T* p) {
+  Raw8<T> r;
+  if constexpr (sizeof(T) == 4) ld8<float>(p, r.v);
+  else r.v = *reinterpret_cast<const u16x8*>(p);
+  return r;
+}
+template <typename T>
+__device__ __forceinline__ void raw_st(T* p, const Raw8<T>& r) {
+  if constexpr (sizeof(T) == 4) st8<float>(p, r.v);
+  else *reinterpret_cast<u16x8*>(p) = r.v;
+}
+
 // columns col..col+7 of row t of a projection: rows [T][ncol], or the sum of S fp32 slabs
 template <typename T>
 __device__ __forceinline__ void load_row8(const float* xp, const void* row, int S, int64_t slab, int64_t at, float (&v)[8]) {
@@ -60,12 +93,32 @@ __device__ __forceinline__ void load_row8(const float* xp, const void* row, int 
   }
 }
 
+// the same in the row type (slabs are summed, then rounded)
+template <typename T>
+__device__ __forceinline__ Raw8<T> raw_row8(const float* xp, const void* row, int S, int64_t slab, int64_t at) {
+  if (!xp) return raw_ld<T>(static_cast<const T*>(row) + at);
+  float v[8];
+  load_row8<T>(xp, row, S, slab, at, v);
+  Raw8<T> r;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    if constexpr (sizeof(T) == 4) r.v[j] = v[j];
+    else r.v[j] = f2bf(v[j]);
+  }
+  return r;
+}
+
 // one element of the same
 template <typename T>
 __device__ __forceinline__ float load_row1(const float* xp, const void* row, int S, int64_t slab, int64_t at) {
   if (xp) {
-    float v = xp[at];
-    for (int s = 1; s < S; ++s) v += xp[at + s * slab];
+    float w[8];
+#pragma unroll
+    for (int s = 0; s < 8; ++s) w[s] = s < S ? xp[at + s * slab] : 0.f;
+    float v = w[0];
+#pragma unroll
+    for (int s = 1; s < 8; ++s) v += w[s];
+    for (int s = 8; s < S; ++s) v += xp[at + s * slab];
     return v;
   }
   if constexpr (sizeof(T) == 4) return static_cast<const float*>(row)[at];

@@ -905,8 +905,11 @@ class LLMEngine:
             st = self._states[bp] = _BucketState(self, bp)
         return st
 
+    def _splits(self, context: int, bp: int) -> int:
+        return ops.decode_splits(context, bp, self.hkv, self.model.split_tokens)
+
     def split_options(self, bp: int) -> list[int]:
-        top = ops.decode_splits(self.max_context, bp, self.hkv)
+        top = self._splits(self.max_context, bp)
         return [1 << i for i in range(top.bit_length())]
 
     def _graph(self, bp: int, splits: int) -> _DecodeGraph:
@@ -958,7 +961,7 @@ class LLMEngine:
             part = order[a:a + self.max_batch]
             rows = [reqs[i] for i in part]
             bp = self._bucket(len(rows))
-            g = self._graph(bp, ops.decode_splits(rows[0].length, bp, self.hkv))
+            g = self._graph(bp, self._splits(rows[0].length, bp))
             g.st.load(rows, self.max_pages)
             g.run(self.use_graphs)
             out[torch.tensor(part, device=self.device)] = g.logits[:len(rows)].float()
@@ -978,7 +981,7 @@ class LLMEngine:
         bp = self._bucket(B)
         k = max(1, min(self.multi_step, min(r.max_tokens - len(r.output) - ahead for r in reqs)))
         # decode-attention split count for the longest context reached in this window
-        splits = ops.decode_splits(max(r.length for r in reqs) + ahead + k - 1, bp, self.hkv)
+        splits = self._splits(max(r.length for r in reqs) + ahead + k - 1, bp)
         g = self._graph(bp, splits)
         st = g.st
         if self._active is not st:

@@ -14,6 +14,8 @@ from dataclasses import replace
 
 import torch
 
+from operator_amd.models.config import LatentSpec
+
 PEAK_FLOPS, PEAK_BYTES = 2.5e15, 8.0e12
 PREFILL = ((1, 1024), (8, 1024), (4, 4096))      # sequences, tokens each
 DECODE = ((1, 1024), (64, 1024), (256, 1024), (64, 4096))   # rows, context
@@ -21,20 +23,38 @@ DECODE = ((1, 1024), (64, 1024), (256, 1024), (64, 4096))   # rows, context
 
 def cut(cfg, layers: int):
     """``cfg`` with its first ``layers`` layers."""
-    if cfg.arch == "sufolix":
+    if hasattr(cfg, "layer_specs"):
         return replace(cfg, layer_specs=cfg.layer_specs[:layers])
     return replace(cfg, layers=layers)
 
 
 def _work(cfg, tokens: int, seqs: int, ctx: int, decode: bool) -> tuple[float, float]:
-    """(matrix flops, bytes that must move) of one step: weights read once, keys and values,
-    and for hyper-connected models their fp32 residual streams; only the experts in use."""
+    """(matrix flops, bytes that must move) of one step: weights read once, keys and values (inside
+    the window, or latent rows), fp32 residual streams where a model has them; only the experts in use."""
     def ff(h, f):
         return 3 * h * f
 
     h, flops, byts = cfg.hidden, 0.0, 0.0
     pairs = tokens * ctx if decode else tokens * (ctx + 1) / 2
     for i in range(cfg.layers):
+        if cfg.arch == "relurax":
+            m, f = cfg.layer_specs[i].mixer, cfg.layer_specs[i].mlp
+            act = 0 if f is None else ff(h, f.ff)
+            byts += 2 * 2 * tokens * h * 4
+            if isinstance(m, LatentSpec):
+                low = h * m.q_rank + m.q_rank * m.heads * (m.dim + m.rot_dim) + h * m.heads + m.heads * m.vdim * h
+                low += h * (m.kv_rank + m.rot_dim) if m.kv_from < 0 else 0
+                up = m.heads * (m.dim + m.vdim) * m.kv_rank
+                per = m.heads * (2 * m.kv_rank + m.rot_dim if decode else m.dim + m.rot_dim + m.vdim)
+                flops += 2 * tokens * (low + up + act) + 2 * pairs * per
+                byts += 2 * (low + up + act) + 2 * (m.kv_rank + m.rot_dim) * (tokens * ctx if decode else tokens)
+            else:
+                proj = h * ((m.heads + m.kv_heads) * m.dim + m.heads) + h * m.heads * m.vdim
+                w = min(m.window or ctx, ctx)
+                seen = tokens * w if decode else tokens / ctx * (w * (w + 1) / 2 + (ctx - w) * w)
+                flops += 2 * tokens * (proj + act) + 2 * seen * m.heads * (m.dim + m.vdim)
+                byts += 2 * (proj + act) + 2 * m.kv_heads * (m.dim + m.vdim) * (tokens * w if decode else tokens)
+            continue
         if cfg.arch == "sufolix":
             a, m = cfg.layer_specs[i].mixer, cfg.layer_specs[i].mlp
             heads, kv, dk, dv = a.heads, a.kv_heads, a.dim, a.vdim
@@ -108,8 +128,6 @@ def run(names: list[str], layers: int = 4, prefill=PREFILL, decode=DECODE, emit=
             for r in reqs:
                 eng.given_end(r)
         for b, c in decode:
-            from operator_amd import ops
-
             # rows with tokens (and sampling seeds) of their own: equal rows would share their experts
             reqs = [GenRequest([1] * (c - 1), output=[int(t)], temperature=1.0, seed=i)
                     for i, t in enumerate(torch.randint(0, cfg.vocab_size, (b,)))]
@@ -117,7 +135,7 @@ def run(names: list[str], layers: int = 4, prefill=PREFILL, decode=DECODE, emit=
                 eng._reserve(r)
                 r.pages = r.pages + kv.allocator.alloc(1)   # the steps below pass the page's end
             bp = eng._bucket(b)
-            g = eng._graph(bp, ops.decode_splits(c, bp, eng.hkv))
+            g = eng._graph(bp, eng._splits(c, bp))
 
             def steps():
                 g.st.load(reqs, eng.max_pages)

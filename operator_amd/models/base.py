@@ -57,6 +57,7 @@ class DecoderModel:
     gu_block: int | None = None
     vocab_offset = 0
     hq = hkv = 1            # heads of this rank (the widest layer's), for launch heuristics
+    split_tokens: int | None = None   # shortest piece decode attention cuts a context into (None: the default)
 
     # ------------------------------------------------------------------ engine surface
     def kv_shapes(self) -> list[tuple[int, int, int]]:

@@ -46,9 +46,9 @@ class ReluraxLayer:
     wo: torch.Tensor              # [ld, ocol]
     norm1: torch.Tensor           # [ld] fp32
     norm1b: torch.Tensor
-    qnorm: torch.Tensor           # fp32: [dk] of a head, or [qp] of the query latent
+    qnorm: torch.Tensor           # [dk] of a head in the compute dtype, or [qp] of the query latent, fp32
     knorm: torch.Tensor | None = None   # [dk], or [rp] of the latent (None: it reads another layer's rows)
-    conv: torch.Tensor | None = None    # [taps, (H + G) dk] fp32
+    conv: torch.Tensor | None = None    # [taps, (H + G) dk] in the compute dtype
     wuq: torch.Tensor | None = None     # latent: [H dk, qp]
     wk: torch.Tensor | None = None      # [H dk, ck] keys of all heads from a latent row
     wv: torch.Tensor | None = None      # [H dv, ck]
@@ -81,10 +81,11 @@ class ReluraxModel(PaddedModel):
                 self.shapes.append(dec.HeadLayout(a.heads, a.kv_heads, a.dim, a.vdim, eps=cfg.rms_eps))
                 self.rot.append(None)
         self.hq = max(L.heads for L in self.shapes)
-        # decode workgroups per sequence of the layers that read whole contexts (chunks of 16 heads
+        # decode workgroups per sequence of the layers that read whole contexts (chunks of 32 heads
         # over one latent row, or key/value heads): what the split count is chosen for
-        full = [-(-L.heads // 16) for L in self.shapes if isinstance(L, dec.LatentLayout)]
+        full = [-(-L.heads // 32) for L in self.shapes if isinstance(L, dec.LatentLayout)]
         full += [L.kv_heads for L, sp in zip(self.shapes, cfg.layer_specs) if isinstance(L, dec.HeadLayout) and not sp.mixer.window]
+        self.split_tokens = 128 if full else None   # latent rows are a few cache lines: short pieces pay
         self.hkv = min(full) if full else max(L.kv_heads for L in self.shapes)
         one = torch.ones(1, device=self.device)
         self.hc = dec.Stream(one, one.view(1, 1), one)   # a single residual stream
@@ -116,9 +117,9 @@ class ReluraxModel(PaddedModel):
         L, a, W = self.shapes[i], self.cfg.layer_specs[i].mixer, self.cfg.hidden
         (dk, dv), H, G, D = L.pads, L.heads, L.kv_heads, L.dim
         rows, at = [], 0
-        conv = torch.zeros(a.conv, (H + G) * dk, device=self.device)
+        conv = torch.zeros(a.conv, (H + G) * dk, dtype=self.dtype, device=self.device)
         for n, heads in (("q", H), ("k", G)):
-            w, c = get(p + n, (heads * D, W)), get(p + n + ".conv", (heads * D, a.conv)).float()
+            w, c = get(p + n, (heads * D, W)), get(p + n + ".conv", (heads * D, a.conv))
             for h in range(heads):
                 rows.append((at, 0, w[h * D:(h + 1) * D]))
                 conv[:, at:at + D] = c[h * D:(h + 1) * D].t()
@@ -126,7 +127,7 @@ class ReluraxModel(PaddedModel):
         wo = get(p + "o", (W, H * D))
         return dict(win=self._put(dec.conv_ncol(L), self.ld, rows + [(at, 0, get(p + "g", (H, W)))]), conv=conv,
                     wo=self._put(self.ld, L.ocol, [(0, h * dv, wo[:, h * D:(h + 1) * D]) for h in range(H)]),
-                    qnorm=self._padded(get(p + "q.norm", (D,)), dk), knorm=self._padded(get(p + "k.norm", (D,)), dk))
+                    qnorm=self._padded(get(p + "q.norm", (D,)), dk).to(self.dtype), knorm=self._padded(get(p + "k.norm", (D,)), dk).to(self.dtype))
 
     def _latent(self, i: int, get, p: str) -> dict:
         L, W = self.shapes[i], self.cfg.hidden

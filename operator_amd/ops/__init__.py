@@ -595,14 +595,14 @@ def linear_fp8(x: torch.Tensor | tuple[torch.Tensor, torch.Tensor], w8: torch.Te
     return y
 
 
-def decode_splits(max_context: int, batch: int = 1, kv_heads: int = 8) -> int:
+def decode_splits(max_context: int, batch: int = 1, kv_heads: int = 8, min_tokens: int | None = None) -> int:
     """Workgroups per (sequence, kv-head) for decode attention: split only while
     ``batch * kv_heads`` workgroups cannot fill the GPU, never into pieces shorter
-    than 256 tokens (measured on MI355X, B=16 ctx=1024: 1 split 25.9 us, 4 splits
+    than ``min_tokens`` (256; measured on MI355X, B=16 ctx=1024: 1 split 25.9 us, 4 splits
     23.7 us, 16 splits 47.8 us). Powers of two, so a graph captured per value
     covers every context length with few captures."""
     want = -(-DECODE_TARGET_BLOCKS // max(1, batch * kv_heads))
-    cap = -(-max(1, int(max_context)) // DECODE_MIN_SPLIT_TOKENS)
+    cap = -(-max(1, int(max_context)) // (min_tokens or DECODE_MIN_SPLIT_TOKENS))
     ns = max(1, min(want, cap, 256))
     # the power of two at or BELOW: splits of 256-512 tokens, not 128-256 (B = 64, one kv-head,
     # ctx 1100: 4 splits 15.2 us vs 8 splits 19.9 us with the combine, profiles/attn_decode_tp8_splits_r5.jsonl)

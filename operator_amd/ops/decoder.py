@@ -252,7 +252,7 @@ def conv_heads(x, pos: torch.Tensor, L: HeadLayout, dtype: torch.dtype, conv: to
                cache: tuple, tails: torch.Tensor | None, slots: torch.Tensor, edges: SequenceEdges):
     """Packed q | k | gate rows (or SplitK slabs) -> (q [T, H, dk], k [T, G, dk], v [T, G, dv], gate [T, H]
     fp32): q and k through the short causal convolution ``conv`` [taps, (H + G) dk] and a weighted
-    per-head RMS norm, v the convolved key without the norm, gate the sigmoid. k / v (None at decode)
+    per-head RMS norm (weights in ``dtype``), v the convolved key without the norm, gate the sigmoid. k / v (None at decode)
     also go to the paged ``cache``, and the last taps - 1 projected rows to ``tails`` [pages, taps - 1, C]."""
     from . import SplitK
 

@@ -347,7 +347,7 @@ def conv_heads(x: torch.Tensor, pos: torch.Tensor, L, conv: torch.Tensor, qw: to
     dk, dv = L.pads
     H, G, R = L.heads, L.kv_heads, conv.shape[0] - 1
     C = (H + G) * dk
-    u = x[:, :C].float()
+    u, conv, qw, kw = x[:, :C].float(), conv.float(), qw.float(), kw.float()
     y = torch.zeros_like(u)
     T = u.shape[0]
     start, pages, ends = list(range(T)), [-1] * T, list(range(1, T + 1))
