@@ -210,7 +210,9 @@ class ReluraxModel(PaddedModel):
         if fb.is_prefill:
             o = self._prefill(i, q, k, v, gate, fb, L, a.window)
         else:
-            o = dec.attn_gd_decode(q, cache, fb.block_tables, fb.context_lens, L, a.scale, fb.num_splits, ws, a.window, gate)
+            # the step's split count is chosen for whole contexts; a window needs no more than its own
+            splits = min(fb.num_splits, ops.decode_splits(a.window or self.cfg.max_position, h.shape[0], L.kv_heads, self.split_tokens))
+            o = dec.attn_gd_decode(q, cache, fb.block_tables, fb.context_lens, L, a.scale, splits, ws, a.window, gate)
         return ops.linear(o, lw.wo, defer_reduce=True)
 
     def _latent_mixer(self, i: int, lw: ReluraxLayer, h, rows: dict, fb: ForwardBatch, kv: PagedKVCache, ws):
