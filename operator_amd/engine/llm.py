@@ -1081,6 +1081,7 @@ class LLMEngine:
                 fin.append(r)
             else:
                 keep.append(r)
+        self.running = keep   # before any waiter wakes: it sees an engine without its request
         if fin:
             self._active = None  # batch composition changed: reload device state next step
             with trace_range(f"finish[{len(fin)}]"):
@@ -1091,5 +1092,4 @@ class LLMEngine:
                         pass
                 for r in fin:
                     r.event.set()
-        self.running = keep
         return fin
